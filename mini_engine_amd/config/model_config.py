@@ -888,3 +888,123 @@ class GoluzenConfig:
     def flat(self) -> dict[str, Any]:
         return {"vocab_size": self.vocab_size, "hidden_size": self.hidden_size, "num_hidden_layers": len(self.layers),
                 "layer_kinds": [layer.kind for layer in self.layers]}
+
+
+# ------------------------------------------------------------------------------------ Vefulix
+@dataclass(frozen=True)
+class VefulixLayer:
+    """One entry of a Vefulix config's `layers`: which mixer it has, the mixer's sizes and constants, and the
+    feed-forward's (None: the layer has no feed-forward)."""
+
+    kind: str                  # "mlstm", "delta" or "latent_attention"
+    mixer: dict
+    mlp: dict | None
+
+
+@register_config("Vefulix")
+@dataclass(frozen=True)
+class VefulixConfig:
+    """The ``config.json`` keys of the Vefulix design: `streams` residual streams with learned shares per sublayer
+    (hyper-connections), layer norms with bias (also behind the embedding), and layers that each name their mixer. `mlstm`:
+    a matrix memory with exponential gates under a cap. `delta`: a gated delta rule with short convolutions and one decay
+    per head. `latent_attention`: keys and values made head by head from a cached latent, queries from a latent of their
+    own, no positions, a sink per head. Feed-forwards: routed experts (the largest router logits, a softmax over those
+    chosen) beside an optional shared expert, all gated by silu. The head has weights of its own and bends its logits under
+    `logit_softcap`. Every size and constant comes from the file."""
+
+    vocab_size: int
+    hidden_size: int
+    norm_eps: float
+    streams: int
+    layers: tuple
+    logit_softcap: float | None = None
+    eos_token_id: int | None = None
+    max_position_embeddings: int | None = None
+
+    MIXERS = {"mlstm": (("heads", int), ("dim", int), ("vdim", int), ("gate_cap", float)),
+              "delta": (("heads", int), ("dim", int), ("vdim", int), ("conv", int)),
+              "latent_attention": (("heads", int), ("dim", int), ("vdim", int), ("q_rank", int), ("kv_rank", int), ("scale", float))}
+
+    @property
+    def num_hidden_layers(self) -> int:
+        return len(self.layers)
+
+    @classmethod
+    def from_dict(cls, raw: dict[str, Any]) -> "VefulixConfig":
+        norm = raw.get("norm")
+        if not isinstance(norm, dict):
+            raise ConfigError("config.json lacks the object 'norm'")
+        listed = raw.get("layers")
+        if not isinstance(listed, list) or not listed:
+            raise ConfigError("config.json lacks the list 'layers'")
+        layers = []
+        for i, entry in enumerate(listed):
+            where = f"layers[{i}]"
+            kind = entry.get("type") if isinstance(entry, dict) else None
+            if kind not in cls.MIXERS:
+                raise ConfigError(f"{where}: 'type' must be one of {sorted(cls.MIXERS)}, got {kind!r}")
+            m = entry.get("mixer")
+            if not isinstance(m, dict):
+                raise ConfigError(f"{where} lacks the object 'mixer'")
+            mixer = {key: _need(m, key, typ, where + ".mixer") for key, typ in cls.MIXERS[kind]}
+            if kind == "delta":
+                mixer["kv_heads"] = _need(m, "kv_heads", int, where + ".mixer") if m.get("kv_heads") is not None else mixer["heads"]
+            mlp = entry.get("mlp")
+            ff = None
+            if mlp is not None:
+                if mlp.get("kind") != "moe":
+                    raise ConfigError(f"{where}.mlp: 'kind' must be 'moe', got {mlp.get('kind')!r}")
+                router, shared = mlp.get("router"), mlp.get("shared")
+                if not isinstance(router, dict) or not isinstance(mlp.get("expert"), dict):
+                    raise ConfigError(f"{where}.mlp lacks the objects 'router' and 'expert'")
+                ff = {"ff": _need(mlp["expert"], "ff", int, where + ".mlp.expert"),
+                      "experts": _need(router, "experts", int, where + ".mlp.router"),
+                      "top": _need(router, "top", int, where + ".mlp.router"),
+                      "shared_ff": _need(shared, "ff", int, where + ".mlp.shared") if shared else None}
+            layers.append(VefulixLayer(kind, mixer, ff))
+        cap = raw.get("logit_softcap")
+        cfg = cls(vocab_size=_need(raw, "vocab", int), hidden_size=_need(raw, "width", int),
+                  norm_eps=_need(norm, "eps", float, "config.json norm"), streams=_need(raw, "streams", int), layers=tuple(layers),
+                  logit_softcap=float(cap) if cap else None,
+                  eos_token_id=raw.get("eos_token_id"), max_position_embeddings=raw.get("max_position_embeddings"))
+        cfg.validate()
+        return cfg
+
+    def validate(self) -> None:
+        if self.vocab_size < 1 or self.hidden_size < 1 or not self.norm_eps > 0 or self.streams < 1:
+            raise ConfigError("vocab, width and streams must be positive and norm.eps above zero")
+        if self.logit_softcap is not None and not self.logit_softcap > 0:
+            raise ConfigError("logit_softcap must be positive")
+        for i, layer in enumerate(self.layers):
+            m, f, where = layer.mixer, layer.mlp, f"layers[{i}]"
+            if any(not v > 0 for v in m.values()):
+                raise ConfigError(f"{where}.mixer: sizes, the score scale and the gates' cap must be positive")
+            if layer.kind == "delta" and m["heads"] % m["kv_heads"]:
+                raise ConfigError(f"{where}: {m['heads']} heads are not a multiple of {m['kv_heads']} kv_heads")
+            if f is None:
+                continue
+            if f["ff"] < 1 or (f["shared_ff"] is not None and f["shared_ff"] < 1):
+                raise ConfigError(f"{where}.mlp: ff must be positive")
+            if f["experts"] < 1 or not 1 <= f["top"] <= f["experts"]:
+                raise ConfigError(f"{where}.mlp: experts must be positive and top at most experts")
+
+    def to_dict(self) -> dict[str, Any]:
+        """A ``config.json`` that reads back to an equal config."""
+        out = []
+        for layer in self.layers:
+            f, mlp = layer.mlp, None
+            if f is not None:
+                mlp = {"kind": "moe", "expert": {"ff": f["ff"]}, "router": {"experts": f["experts"], "top": f["top"]}}
+                if f["shared_ff"] is not None:
+                    mlp["shared"] = {"ff": f["shared_ff"]}
+            out.append({"type": layer.kind, "mixer": dict(layer.mixer), "mlp": mlp})
+        d = {"architecture": self.architecture_name, "vocab": self.vocab_size, "width": self.hidden_size,
+             "norm": {"eps": self.norm_eps}, "streams": self.streams, "layers": out}
+        for key in ("logit_softcap", "eos_token_id", "max_position_embeddings"):
+            if getattr(self, key) is not None:
+                d[key] = getattr(self, key)
+        return d
+
+    def flat(self) -> dict[str, Any]:
+        return {"vocab_size": self.vocab_size, "hidden_size": self.hidden_size, "num_hidden_layers": len(self.layers),
+                "layer_kinds": [layer.kind for layer in self.layers]}

@@ -235,6 +235,8 @@ extern "C" int me_token_shift(const void* x, int64_t x_stride, int dtype, const 
 //                    y_p = sum_n S[n, p] q_n
 //   RULE 2 (gated):  d_n = sigmoid(raw[t, h, n] + base[h, n]) ^ rate[h] = exp(-rate[h] softplus(-(raw + base)));
 //                    S[n, p] <- d_n S[n, p] + k_n v_p;   y_p = sum_n S[n, p] q_n
+//   RULE 3 (delta_head): RULE 1 with one decay per head and token, d = exp(-rate[h] softplus(raw[t, h] + base[h])): the
+//                    decay then needs no LDS and multiplies a lane's rows from a register
 // With `unit`: q and k are first divided by sqrt(sum of their squares + unit_eps) per head; q is multiplied by q_scale.
 // Every sum runs over n only, so a column p of the state never meets another: a wave takes 64 / RG columns of one head
 // and a lane NR / RG of a column's rows, kept in registers for the whole walk; with RG > 1 the RG lanes of a column,
@@ -274,6 +276,7 @@ __device__ __forceinline__ float group_sum(float v) {
 // What a token's q, k, raw decay and write strength become before the recurrence reads them, for one wave that holds
 // rows lane, lane + 64, ... of one head: q and k at unit length and scaled, the decay, and the token's own number
 // (sigmoid(beta), or sum_n q_n bonus_n k_n under the bonus rule), which every lane gets.
+// (RULE 3: every lane holds the head's one raw decay and its base in d[0], base[0] and gets the decay there.)
 template <int PER, int RULE>
 __device__ __forceinline__ float shape_token(const DrArgs& a, int lane, int nr_rows, float (&q)[PER], float (&k)[PER], float (&d)[PER],
                                              const float (&base)[PER], const float (&bonus)[PER], float rate, float beta) {
@@ -291,6 +294,7 @@ __device__ __forceinline__ float shape_token(const DrArgs& a, int lane, int nr_r
     const int n = lane + 64 * i;
     q[i] *= qs;
     k[i] *= ks;
+    if (RULE == 3) continue;
     float dv;
     if (RULE == 0) dv = expf(-expf(d[i] + base[i]));
     else if (RULE == 2) dv = expf(-rate * hy_softplus(-(d[i] + base[i])));
@@ -298,8 +302,9 @@ __device__ __forceinline__ float shape_token(const DrArgs& a, int lane, int nr_r
     d[i] = (n < a.N && n < nr_rows) ? dv : 1.0f;
     own += q[i] * bonus[i] * k[i];
   }
+  if (RULE == 3) d[0] = expf(-rate * hy_softplus(d[0] + base[0]));
   if (RULE == 2) return 0.f;
-  return RULE == 1 ? hy_sigmoid(beta) : wave_sum(own);
+  return (RULE == 1 || RULE == 3) ? hy_sigmoid(beta) : wave_sum(own);
 }
 
 // One wave per (token, head): the shaped values of every token at once, for a recurrence kernel that then only streams
@@ -317,21 +322,27 @@ __global__ void __launch_bounds__(64) decay_prepare_kernel(DrArgs a, float* __re
   for (int i = 0; i < PER; ++i) {
     const int n = lane + 64 * i;
     const bool in = n < a.N && n < NR;
-    base[i] = in ? a.base[h * a.N + n] : 0.f;
+    base[i] = RULE == 3 ? a.base[h] : (in ? a.base[h * a.N + n] : 0.f);
     bonus[i] = (RULE == 0 && in) ? a.bonus[h * a.N + n] : 0.f;
     q[i] = in ? to_f32<TX>(qp[t * a.q_stride + g * a.N + n]) : 0.f;
     k[i] = in ? to_f32<TX>(kp[t * a.k_stride + g * a.N + n]) : 0.f;
-    d[i] = in ? to_f32<TX>(rp[t * a.raw_stride + h * a.N + n]) : 0.f;
+    d[i] = RULE == 3 ? to_f32<TX>(rp[t * a.raw_stride + h]) : (in ? to_f32<TX>(rp[t * a.raw_stride + h * a.N + n]) : 0.f);
   }
-  const float beta = RULE == 1 ? to_f32<TX>(bp[t * a.beta_stride + h]) : 0.f;
+  const float beta = (RULE == 1 || RULE == 3) ? to_f32<TX>(bp[t * a.beta_stride + h]) : 0.f;
   const float x = shape_token<PER, RULE>(a, lane, NR, q, k, d, base, bonus, RULE != 0 ? a.rate[h] : 0.f, beta);
   const int64_t at = (t * a.H + h) * NR;
 #pragma unroll
   for (int i = 0; i < PER; ++i) {
     const int n = lane + 64 * i;
-    if (n < NR) { pre_q[at + n] = q[i]; pre_k[at + n] = k[i]; pre_d[at + n] = d[i]; }
+    if (n < NR) {
+      pre_q[at + n] = q[i]; pre_k[at + n] = k[i];
+      if (RULE != 3) pre_d[at + n] = d[i];
+    }
   }
-  if (lane == 0) pre_x[t * a.H + h] = x;
+  if (lane == 0) {
+    pre_x[t * a.H + h] = x;
+    if (RULE == 3) pre_d[t * a.H + h] = d[0];
+  }
 }
 
 template <typename TX, int NR, int RG, int RULE, bool PRE>
@@ -340,7 +351,7 @@ __global__ void __launch_bounds__(64) decay_rows_kernel(DrArgs a, const float* _
   constexpr int PC = 64 / RG;            // columns per wave
   constexpr int RL = NR / RG;            // rows per lane
   constexpr int PER = (NR + 63) / 64;    // rows of q, k and the decay that a lane brings to LDS for the wave
-  __shared__ float sq[2][DR_TB][NR], sk[2][DR_TB][NR], sd[2][DR_TB][NR];
+  __shared__ float sq[2][DR_TB][NR], sk[2][DR_TB][NR], sd[2][RULE == 3 ? 1 : DR_TB][RULE == 3 ? 1 : NR];
   const int lane = threadIdx.x;
   const int col_blocks = (a.P + PC - 1) / PC;
   const int cb = blockIdx.x % col_blocks;
@@ -368,14 +379,14 @@ __global__ void __launch_bounds__(64) decay_rows_kernel(DrArgs a, const float* _
   for (int i = 0; i < PER; ++i) {
     const int n = lane + 64 * i;
     const bool in = !PRE && n < a.N && n < NR;
-    base[i] = in ? a.base[h * a.N + n] : 0.f;
+    base[i] = RULE == 3 ? (PRE ? 0.f : a.base[h]) : (in ? a.base[h * a.N + n] : 0.f);
     bonus[i] = (RULE == 0 && in) ? a.bonus[h * a.N + n] : 0.f;
   }
   const float rate = (RULE != 0 && !PRE) ? a.rate[h] : 0.f;
   // a batch of tokens on its way (n*) and the batch being worked on (c*): a lane's own column's v and the token's own
   // number (the write strength, or under the bonus rule sum_n q_n bonus_n k_n)
   float nq[DR_TB][PER], nk[DR_TB][PER], nr[DR_TB][PER], nv[DR_TB], nb[DR_TB];
-  float cv[DR_TB], cx[DR_TB];
+  float cv[DR_TB], cx[DR_TB], cd[DR_TB];        // cd: the token's decay (RULE 3)
   auto fetch = [&](int t0) {
 #pragma unroll
     for (int j = 0; j < DR_TB; ++j) {
@@ -386,17 +397,19 @@ __global__ void __launch_bounds__(64) decay_rows_kernel(DrArgs a, const float* _
           const int n = lane + 64 * i;
           if (PRE) {
             const int64_t at = (row * a.H + h) * NR + (n < NR ? n : 0);
-            nq[j][i] = pre_q[at]; nk[j][i] = pre_k[at]; nr[j][i] = pre_d[at];
+            nq[j][i] = pre_q[at]; nk[j][i] = pre_k[at];
+            nr[j][i] = RULE == 3 ? (i == 0 ? pre_d[row * a.H + h] : 0.f) : pre_d[at];
           } else {
             const bool in = n < a.N && n < NR;
             nq[j][i] = in ? to_f32<TX>(qp[row * a.q_stride + g * a.N + n]) : 0.f;
             nk[j][i] = in ? to_f32<TX>(kp[row * a.k_stride + g * a.N + n]) : 0.f;
-            nr[j][i] = in ? to_f32<TX>(rp[row * a.raw_stride + h * a.N + n]) : 0.f;
+            if (RULE == 3) nr[j][i] = i == 0 ? to_f32<TX>(rp[row * a.raw_stride + h]) : 0.f;
+            else nr[j][i] = in ? to_f32<TX>(rp[row * a.raw_stride + h * a.N + n]) : 0.f;
           }
         }
         nv[j] = to_f32<TX>(vp[row * a.v_stride + h * a.P + pc]);
         if (PRE) nb[j] = pre_x[row * a.H + h];
-        else nb[j] = RULE == 1 ? to_f32<TX>(bp[row * a.beta_stride + h]) : 0.f;
+        else nb[j] = (RULE == 1 || RULE == 3) ? to_f32<TX>(bp[row * a.beta_stride + h]) : 0.f;
       }
     }
   };
@@ -413,8 +426,12 @@ __global__ void __launch_bounds__(64) decay_rows_kernel(DrArgs a, const float* _
           // row n belongs to lane n % RG of a column as its row n / RG: a lane's rows lie side by side in LDS, so that it
           // reads them four at a time
           const int at = (n % RG) * RL + n / RG;
-          if (n < NR) { sq[buf][j][at] = nq[j][i]; sk[buf][j][at] = nk[j][i]; sd[buf][j][at] = nr[j][i]; }
+          if (n < NR) {
+            sq[buf][j][at] = nq[j][i]; sk[buf][j][at] = nk[j][i];
+            if (RULE != 3) sd[buf][j][at] = nr[j][i];
+          }
         }
+        cd[j] = nr[j][0];
         cv[j] = nv[j];
         cx[j] = x;
       }
@@ -449,7 +466,7 @@ __global__ void __launch_bounds__(64) decay_rows_kernel(DrArgs a, const float* _
 #pragma unroll
           for (int i = 0; i < RL; ++i) {
             const int n = rg * RL + i;
-            S[i] *= sd[buf][j][n];
+            S[i] *= RULE == 3 ? cd[j] : sd[buf][j][n];
             dot = fmaf(S[i], sk[buf][j][n], dot);
           }
           dot = group_sum<RG>(dot);
@@ -485,10 +502,12 @@ static void launch_decay_rows(const DrArgs& a, int rule, int num_seqs, int64_t T
     const dim3 pgrid((unsigned)T, a.H);
     if (rule == 0) decay_prepare_kernel<TX, NR, 0><<<pgrid, block, 0, stream>>>(a, pq, pk, pd, px);
     else if (rule == 2) decay_prepare_kernel<TX, NR, 2><<<pgrid, block, 0, stream>>>(a, pq, pk, pd, px);
+    else if (rule == 3) decay_prepare_kernel<TX, NR, 3><<<pgrid, block, 0, stream>>>(a, pq, pk, pd, px);
     else decay_prepare_kernel<TX, NR, 1><<<pgrid, block, 0, stream>>>(a, pq, pk, pd, px);
   }
   if (rule == 0) decay_rows_kernel<TX, NR, RG, 0, PRE><<<grid, block, 0, stream>>>(a, pq, pk, pd, px);
   else if (rule == 2) decay_rows_kernel<TX, NR, RG, 2, PRE><<<grid, block, 0, stream>>>(a, pq, pk, pd, px);
+  else if (rule == 3) decay_rows_kernel<TX, NR, RG, 3, PRE><<<grid, block, 0, stream>>>(a, pq, pk, pd, px);
   else decay_rows_kernel<TX, NR, RG, 1, PRE><<<grid, block, 0, stream>>>(a, pq, pk, pd, px);
 }
 
@@ -503,7 +522,7 @@ extern "C" int me_decay_rows_recurrence(const void* q, int64_t q_stride, const v
   if (num_seqs == 0) return 0;
   ME_CHECK(H >= 1 && G >= 1 && H % G == 0 && N >= 1 && N <= 256 && P >= 1, "decay_rows_recurrence: %d heads over %d groups, state %d x %d "
            "(up to 256 rows)", H, G, N, P);
-  ME_CHECK(rule >= 0 && rule <= 2, "decay_rows_recurrence: unknown rule %d", rule);
+  ME_CHECK(rule >= 0 && rule <= 3, "decay_rows_recurrence: unknown rule %d", rule);
   ME_CHECK(rule == 0 ? bonus != nullptr : (rate != nullptr && (rule == 2 || beta != nullptr)), "decay_rows_recurrence: the rule's constants are missing");
   ME_CHECK(pre == nullptr ? (row_groups == 1 || row_groups == 4) : (row_groups == 4 || row_groups == 16),
            "decay_rows_recurrence: 1 or 4 lanes to a column, 4 or 16 over prepared values");

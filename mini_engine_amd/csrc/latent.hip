@@ -1,7 +1,8 @@
 // Attention over a latent that all heads share (one normed vector and one rotated key part per token in the cache).
 //
 //   latent_prepare   per token, from the rows of the layer's packed product: the latent's RMS norm with its weight, the
-//                    rotation of the shared key part and of every query head's rotating part (adjacent pairs), and
+//                    rotation of the shared key part and of every query head's rotating part (adjacent pairs), the
+//                    RMS norm of the queries' own latent where they have one, and
 //                    the write into the pages: the key page takes [latent | rotated part | zeros], the value page
 //                    (transposed inside a page) the latent. One pass, norm and angles in float32.
 //   heads_linear     y[t, h, :] = W[h] x[t, h, :]: a product per head (queries into the latent's space, attention
@@ -24,6 +25,7 @@ struct LatentArgs {
   const int32_t* positions; const int32_t* slots;
   void* qa; int64_t qa_stride;                // [T, H * D]: the rotated part goes to slots R .. R + dr of every head
   void* k_cache; void* v_cache; int page;     // [pages, 1, page, D], [pages, 1, D, page]; null: this layer writes none
+  int cq_off, RQ; const float* cq_w; void* cq;      // the queries' own latent: its place in a row, size, norm weight, result [T, RQ]; null: none
 };
 
 template <typename TX>
@@ -50,6 +52,14 @@ __global__ void __launch_bounds__(128) latent_prepare_kernel(LatentArgs a) {
   for (int i = threadIdx.x; i < a.H * pad; i += blockDim.x) {
     const int h = i / pad, j = i - h * pad;
     qa[(int64_t)h * a.D + a.R + a.dr + j] = from_f32<TX>(0.f);
+  }
+  if (a.cq != nullptr) {                    // the queries' latent under its norm (the same eps)
+    const TX* src = row + a.cq_off;
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < a.RQ; i += blockDim.x) { const float v = to_f32<TX>(src[i]); ss += v * v; }
+    const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / (float)a.RQ + a.eps);
+    TX* dst = (TX*)a.cq + t * a.RQ;
+    for (int i = threadIdx.x; i < a.RQ; i += blockDim.x) dst[i] = from_f32<TX>(to_f32<TX>(src[i]) * inv * a.cq_w[i]);
   }
   if (a.k_cache == nullptr) return;
   const int slot = a.slots[t];
@@ -80,15 +90,17 @@ __global__ void __launch_bounds__(128) latent_prepare_kernel(LatentArgs a) {
 extern "C" int me_latent_prepare(const void* rows, int64_t row_stride, int dtype, int q_off, int kv_off, int H, int dn, int dr, int R,
                                  int D, const float* norm_w, float eps, const float* table, int64_t table_rows,
                                  const int32_t* positions, const int32_t* slots, void* qa, int64_t qa_stride, void* k_cache,
-                                 void* v_cache, int page, int64_t T, hipStream_t stream) {
+                                 void* v_cache, int page, int cq_off, int RQ, const float* cq_w, void* cq, int64_t T, hipStream_t stream) {
   if (T == 0) return 0;
-  ME_CHECK(H >= 1 && dn >= 0 && dr >= 0 && dr % 2 == 0 && R >= 1 && D >= R + dr, "latent_prepare: %d heads of %d + %d, rank %d, head size %d",
+  ME_CHECK(cq == nullptr || (RQ >= 1 && cq_w != nullptr), "latent_prepare: the queries' latent needs its size and norm weight");
+  ME_CHECK(H >= 0 && dn >= 0 && dr >= 0 && dr % 2 == 0 && R >= 1 && D >= R + dr, "latent_prepare: %d heads of %d + %d, rank %d, head size %d",
            H, dn, dr, R, D);
   ME_CHECK(T <= 2147483647ll && (k_cache == nullptr || (v_cache && slots && norm_w && page >= 1)), "latent_prepare: missing operand");
   ME_CHECK(dr == 0 || (table != nullptr && table_rows >= 1), "latent_prepare: the rotation needs its table");
   LatentArgs a;
   a.rows = rows; a.row_stride = row_stride; a.q_off = q_off; a.kv_off = kv_off; a.H = H; a.dn = dn; a.dr = dr; a.R = R; a.D = D;
   a.norm_w = norm_w; a.eps = eps; a.table = table; a.table_rows = table_rows; a.positions = positions; a.slots = slots;
+  a.cq_off = cq_off; a.RQ = RQ; a.cq_w = cq_w; a.cq = cq;
   a.qa = qa; a.qa_stride = qa_stride; a.k_cache = k_cache; a.v_cache = v_cache; a.page = page;
   if (dtype == ME_F32) latent_prepare_kernel<float><<<dim3((unsigned)T), dim3(128), 0, stream>>>(a);
   else latent_prepare_kernel<bf16_t><<<dim3((unsigned)T), dim3(128), 0, stream>>>(a);

@@ -1,6 +1,7 @@
 // A feed-forward made of many small gated experts of which every token uses a few.
 //
-//   moe_route      float32 router: logits = W x; scores = their softmax over all experts or their sigmoids; the choice
+//   moe_route      float32 router: logits = W x (+ a bias per expert); scores = their softmax over all experts, their
+//                  sigmoids, or the logits themselves (the weights are then their softmax over the chosen); the choice
 //                  goes by the scores plus an optional correction per expert; optionally only the experts of the best
 //                  groups of neighbours stay eligible (a group scores as the sum of its `group_top` largest choice
 //                  scores); the `top` largest are chosen; their weights are the scores without the correction, times
@@ -55,7 +56,7 @@ __device__ __forceinline__ void load4(const bf16_t* p, float (&v)[4]) {
 // experts, a wave every fourth of them; a lane walks K in steps of 64 and the wave adds up. float32 [T, E] out.
 template <typename TX>
 __global__ void __launch_bounds__(256)
-moe_logits_kernel(const TX* __restrict__ x, int64_t ldx, const float* __restrict__ w, int64_t T, int n, int E,
+moe_logits_kernel(const TX* __restrict__ x, int64_t ldx, const float* __restrict__ w, const float* __restrict__ bias, int64_t T, int n, int E,
                   int tokens_per_group, int experts_per_group, float* __restrict__ logits) {
   extern __shared__ __align__(16) unsigned char route_lds[];
   const int TT = tokens_per_group;
@@ -109,12 +110,13 @@ moe_logits_kernel(const TX* __restrict__ x, int64_t ldx, const float* __restrict
     for (int tt = 0; tt < 8; ++tt)
       if (tt < TT) {
         const float s = wave_sum(acc[tt]);
-        if (lane == 0 && tt < live) logits[(t0 + tt) * E + e] = s;
+        if (lane == 0 && tt < live) logits[(t0 + tt) * E + e] = bias ? s + bias[e] : s;
       }
   }
 }
 
-// How scores become a choice. sigmoid 0: softmax over all experts, 1: a sigmoid per expert. correction: float32 [E]
+// How scores become a choice. sigmoid 0: softmax over all experts, 1: a sigmoid per expert, 2: the logits themselves, whose
+// softmax over the chosen experts alone gives the weights (normalise has no say). correction: float32 [E]
 // added to the scores for the choice only (null: none). A group's score is the sum of its group_top largest choice
 // scores. normalise: the chosen scores are divided by their sum. The weights are multiplied by scale.
 struct RouteRule {
@@ -130,7 +132,9 @@ __device__ __forceinline__ void select_token(const float* __restrict__ logits, i
   const int lane = threadIdx.x & 63;
   const int top = r.top, group_count = r.group_count, group_keep = r.group_keep;
   const int per = E / group_count;
-  if (r.sigmoid) {
+  if (r.sigmoid == 2) {
+    for (int e = lane; e < E; e += 64) s[e] = logits[t * E + e];
+  } else if (r.sigmoid) {
     for (int e = lane; e < E; e += 64) s[e] = 1.0f / (1.0f + expf(-logits[t * E + e]));
   } else {
     float hi = -INFINITY;
@@ -191,6 +195,17 @@ __device__ __forceinline__ void select_token(const float* __restrict__ logits, i
     if (lane == j) mine = bi;
     total += s[bi];
   }
+  if (r.sigmoid == 2) {                    // softmax over the chosen logits
+    const float z = lane < top ? s[mine] : -INFINITY;
+    const float hi = wave_max(z);
+    const float p = lane < top ? expf(z - hi) : 0.f;
+    const float sum = wave_sum(p);
+    if (lane < top) {
+      ids[t * top + lane] = mine;
+      weights[t * top + lane] = r.scale * (p / sum);
+    }
+    return;
+  }
   if (lane < top) {
     ids[t * top + lane] = mine;
     weights[t * top + lane] = r.scale * (r.normalise ? s[mine] / (total + 1e-20f) : s[mine]);
@@ -218,7 +233,7 @@ static bool route_rule(RouteRule& r, int E, int top, int group_count, int group_
          group_keep >= 1 && group_keep <= group_count && group_keep * (E / group_count) >= top && group_top >= 1;
 }
 
-extern "C" int me_moe_route(const void* x, int64_t ldx, int dtype, const float* w, int64_t T, int n, int E, int top,
+extern "C" int me_moe_route(const void* x, int64_t ldx, int dtype, const float* w, const float* bias, int64_t T, int n, int E, int top,
                             int group_count, int group_keep, float* logits, int32_t* ids, float* weights, int select,
                             int group_top, int sigmoid, int normalise, float scale, const float* correction,
                             hipStream_t stream) {
@@ -241,9 +256,9 @@ extern "C" int me_moe_route(const void* x, int64_t ldx, int dtype, const float* 
   const int per_group = groups <= 64 ? 4 : 8;
   const dim3 grid((unsigned)groups, (unsigned)((E + per_group - 1) / per_group));
   if (dtype == ME_F32)
-    moe_logits_kernel<float><<<grid, dim3(256), (size_t)TT * n * es, stream>>>((const float*)x, ldx, w, T, n, E, TT, per_group, logits);
+    moe_logits_kernel<float><<<grid, dim3(256), (size_t)TT * n * es, stream>>>((const float*)x, ldx, w, bias, T, n, E, TT, per_group, logits);
   else
-    moe_logits_kernel<bf16_t><<<grid, dim3(256), (size_t)TT * n * es, stream>>>((const bf16_t*)x, ldx, w, T, n, E, TT, per_group, logits);
+    moe_logits_kernel<bf16_t><<<grid, dim3(256), (size_t)TT * n * es, stream>>>((const bf16_t*)x, ldx, w, bias, T, n, E, TT, per_group, logits);
   ME_LAUNCH_CHECK();
   if (!select) return 0;           // the caller lets `me_moe_sort` choose (few tokens: one launch less)
   const size_t lds = (size_t)4 * (2 * E + group_count) * 4;

@@ -5,8 +5,11 @@
 //   activation        silu / squared relu of a row view
 //   head_gate         o[t, h, :] *= sigmoid(g[t, h])
 //   causal_conv       short causal convolution per channel over a request's tokens, continued from its state, + silu
-//   recurrence        S_t = a_t S_(t-1) + b_t k_t v_t^T,  y_t = S_t^T q_t (+ skip v_t): float32 state per head
+//   recurrence        S_t = a_t S_(t-1) + b_t k_t v_t^T,  y_t = S_t^T q_t (+ skip v_t): float32 state per head; optionally
+//                     beside it the sum of the keys under the same factors, n_t = a_t n_(t-1) + b_t k_t, and n_t . q_t
+//   soft_gates        a_t and b_t from exponential input and forget gates under a running maximum
 //   gated_rms_norm    unit root mean square per group with a gate in front of or behind it
+//   memory_readout    the same on outputs that are divided by max(|n . q|, exp(-maximum)) first
 //
 // Everything that enters a recurrence is float32: step sizes, decays, their exponentials, the state, the sums.
 #include "common.h"
@@ -316,6 +319,82 @@ extern "C" int me_causal_conv(const void* x, int64_t x_stride, int dtype, const 
   return 0;
 }
 
+// ------------------------------------------------------------------ exponential gates under a running maximum
+// Per head and token, from raw rows z_i, z_f with biases and a cap c: i = c tanh((z_i + bias) / c), the logarithm of the
+// forget gate f = log sigmoid(c tanh((z_f + bias) / c)), the maximum m' = max(f + m, i), and the factors of the
+// recurrence a = exp(f + m - m'), b = exp(i - m'). m (one number per head in the request's state row) starts at 0.
+struct SoftGates {
+  const void* i; const void* f; int64_t stride;      // [T, H] views
+  const float* bias_i; const float* bias_f; float cap;
+  float* m; int64_t m_stride;                        // [slots, H]
+};
+
+template <typename TX>
+__device__ __forceinline__ void read_gates(const SoftGates& g, int64_t t, int h, float& i, float& f) {
+  const float zi = to_f32<TX>(((const TX*)g.i)[t * g.stride + h]) + g.bias_i[h];
+  const float zf = g.cap * tanhf((to_f32<TX>(((const TX*)g.f)[t * g.stride + h]) + g.bias_f[h]) / g.cap);
+  i = g.cap * tanhf(zi / g.cap);
+  f = fminf(zf, 0.f) - log1pf(expf(-fabsf(zf)));
+}
+
+// One wave per (request, head): 64 tokens at a time, the maximum by a scan over the lanes ((F, M) then (F', M') is
+// (F + F', max(M + F', M'))), the next 64 tokens' rows on their way meanwhile. a, b, floor = exp(-m'): [T, H].
+template <typename TX>
+__global__ void __launch_bounds__(64) soft_gates_kernel(SoftGates g, const int32_t* __restrict__ slots, const int32_t* __restrict__ cu,
+                                                        float* __restrict__ a, float* __restrict__ b, float* __restrict__ floor_out, int H) {
+  const int lane = threadIdx.x;
+  const int q = blockIdx.x / H, h = blockIdx.x - q * H;
+  const int64_t first = cu[q], end = cu[q + 1];
+  if (first >= end) return;
+  float* held = g.m + (int64_t)slots[q] * g.m_stride + h;
+  float m = *held;
+  float zi, zf;
+  auto fetch = [&](int64_t t0) {
+    const int64_t t = t0 + lane < end ? t0 + lane : end - 1;
+    zi = to_f32<TX>(((const TX*)g.i)[t * g.stride + h]);
+    zf = to_f32<TX>(((const TX*)g.f)[t * g.stride + h]);
+  };
+  fetch(first);
+  const float bi = g.bias_i[h], bf = g.bias_f[h];
+  for (int64_t t0 = first; t0 < end; t0 += 64) {
+    const bool on = t0 + lane < end;
+    const float i = g.cap * tanhf((zi + bi) / g.cap);
+    const float z = g.cap * tanhf((zf + bf) / g.cap);
+    const float f = fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
+    if (t0 + 64 < end) fetch(t0 + 64);
+    float F = on ? f : 0.f, M = on ? i : -INFINITY;
+#pragma unroll
+    for (int off = 1; off < 64; off <<= 1) {
+      const float pf = __shfl_up(F, off, ME_WAVE), pm = __shfl_up(M, off, ME_WAVE);
+      if (lane >= off) { M = fmaxf(pm + F, M); F += pf; }
+    }
+    const float now = fmaxf(m + F, M);
+    float before = __shfl_up(now, 1, ME_WAVE);
+    if (lane == 0) before = m;
+    if (on) {
+      const int64_t at = (t0 + lane) * H + h;
+      a[at] = expf(f + before - now);
+      b[at] = expf(i - now);
+      floor_out[at] = expf(-now);
+    }
+    m = __shfl(now, 63, ME_WAVE);
+  }
+  if (lane == 0) *held = m;
+}
+
+extern "C" int me_soft_gates(const void* i, const void* f, int64_t stride, int dtype, const float* bias_i, const float* bias_f, float cap,
+                             float* m, int64_t m_stride, const int32_t* slots, const int32_t* cu, float* a, float* b, float* floor_out,
+                             int num_seqs, int H, hipStream_t stream) {
+  if (num_seqs == 0) return 0;
+  ME_CHECK(H >= 1 && cap > 0.f && (int64_t)num_seqs * H <= 2147483647ll, "soft_gates: bad sizes or cap");
+  SoftGates g;
+  g.i = i; g.f = f; g.stride = stride; g.bias_i = bias_i; g.bias_f = bias_f; g.cap = cap; g.m = m; g.m_stride = m_stride;
+  if (dtype == ME_F32) soft_gates_kernel<float><<<dim3(num_seqs * H), dim3(64), 0, stream>>>(g, slots, cu, a, b, floor_out, H);
+  else soft_gates_kernel<bf16_t><<<dim3(num_seqs * H), dim3(64), 0, stream>>>(g, slots, cu, a, b, floor_out, H);
+  ME_LAUNCH_CHECK();
+  return 0;
+}
+
 // ------------------------------------------------------------------ the recurrence
 // One wave per (request, one or two heads, 64 or 128 columns of P, NT rows of N, span of tokens). A lane keeps CL
 // columns of its NT state rows in registers (CL = 1, or 2: two blocks of 64 columns of one head, or the same 64
@@ -343,18 +422,28 @@ struct RecArgs {
   float* span_state; float* span_decay;             // scratch: [requests, spans, H, N, P], [requests, spans, H]
   int H, G, N, P, span, max_spans;
   int silu;                                         // q, k and v pass silu on their way in
+  const float* coef_a; const float* coef_b;         // a, b given per token and head, [T, H], or null
+  float* keys;                                      // the summed keys' state [slots, H * N] (stride state_stride), or null: none
+  float* key_dot; int64_t dot_slice_stride;         // n . q: [slices of N, T, H]
+  float* span_keys;                                 // scratch: [requests, spans, H, N]
+  SoftGates gates;                                  // a step of single tokens forms a and b itself (gates.i null: not)
 };
 
 #define REC_TB 8
 
-// HPB heads and PPB blocks of 64 columns per wave; CL = HPB * PPB columns per lane.
-template <typename TX, int NT, int PASS, int HPB, int PPB>
+// HPB heads and PPB blocks of 64 columns per wave; CL = HPB * PPB columns per lane. KEYS: the waves of the first column
+// block also keep the summed keys of their NT rows, one row per lane; a batch's products with q meet in LDS, where eight
+// lanes add up a token's (HPB 1 only).
+template <typename TX, int NT, int PASS, int HPB, int PPB, bool KEYS>
 __global__ void __launch_bounds__(64) recurrence_kernel(RecArgs a) {
+  static_assert(!KEYS || HPB == 1, "summed keys: one head per wave");
   constexpr int CL = HPB * PPB;
   constexpr int KR = REC_TB * NT / 64;               // k (and q) values a lane carries to LDS per batch of tokens
   using Cell = std::conditional_t<PASS == 1, float, float2>;       // the first pass of spans reads no q
   __shared__ Cell skq[REC_TB][NT];
   __shared__ float sa[HPB][REC_TB], sb[HPB][REC_TB];
+  __shared__ float nd[KEYS && PASS != 1 ? REC_TB : 1][KEYS && PASS != 1 ? NT : 1];
+  const bool keys = KEYS && blockIdx.y == 0;
   const int lane = threadIdx.x;
   const int heads_blocks = a.H / HPB;
   const int b = blockIdx.x / heads_blocks, h0 = (blockIdx.x - b * heads_blocks) * HPB;
@@ -419,6 +508,9 @@ __global__ void __launch_bounds__(64) recurrence_kernel(RecArgs a) {
         const float step = z > 20.f ? z : log1pf(expf(z));
         areg = expf(-a.rate[hh] * step);
         breg = step;
+      } else if (a.coef_a) {
+        areg = a.coef_a[at * a.H + hh];
+        breg = a.coef_b[at * a.H + hh];
       } else {
         areg = a.decay[hh];
         breg = 1.f;
@@ -446,6 +538,15 @@ __global__ void __launch_bounds__(64) recurrence_kernel(RecArgs a) {
         S[j][i] = (on[j] && i <= n_last) ? held : 0.f;
       }
     }
+  }
+  float* key_row = nullptr;
+  float* span_key_row = nullptr;
+  float nk = 0.f;
+  const bool my_key = keys && lane < NT && lane <= n_last;
+  if (KEYS) {
+    key_row = a.keys + (int64_t)a.slots[b] * a.state_stride + (int64_t)h0 * a.N + n0;
+    if (PASS != 0) span_key_row = a.span_keys + (((int64_t)b * a.max_spans + c) * a.H + h0) * (int64_t)a.N + n0;
+    if (PASS != 1 && my_key) nk = (PASS == 0 ? key_row : span_key_row)[lane];
   }
   float skip[CL];
 #pragma unroll
@@ -511,6 +612,32 @@ __global__ void __launch_bounds__(64) recurrence_kernel(RecArgs a) {
           }
       }
     }
+    if (KEYS && keys) {
+      if (lane < NT)
+        for (int tt = 0; tt < nt; ++tt) {
+          if constexpr (PASS == 1) nk = fmaf(sa[0][tt], nk, sb[0][tt] * skq[tt][lane]);
+          else {
+            const float2 kq = skq[tt][lane];
+            nk = fmaf(sa[0][tt], nk, sb[0][tt] * kq.x);
+            nd[tt][lane] = nk * kq.y;
+          }
+        }
+    }
+    if (KEYS && PASS != 1 && keys) {
+      __syncthreads();                                // the batch's products are in LDS
+      const int tt = lane >> 3, part = lane & 7;
+      float dot = 0.f;
+      if (tt < nt)
+        for (int i = part; i < NT; i += 8) dot += nd[tt][i];
+      dot += __shfl_xor(dot, 1, ME_WAVE);
+      dot += __shfl_xor(dot, 2, ME_WAVE);
+      dot += __shfl_xor(dot, 4, ME_WAVE);
+      if (part == 0 && tt < nt) a.key_dot[slice * a.dot_slice_stride + (tb + tt) * a.H + h0] = dot;
+    }
+  }
+  if (KEYS && my_key) {
+    if (PASS == 1) span_key_row[lane] = nk;
+    else if (t1 == end_all) key_row[lane] = nk;
   }
 #pragma unroll
   for (int j = 0; j < CL; ++j) {
@@ -535,15 +662,17 @@ __global__ void __launch_bounds__(64) recurrence_kernel(RecArgs a) {
 __global__ void recurrence_carry_kernel(RecArgs a) {
   const int b = blockIdx.y;
   const int64_t per_head = (int64_t)a.N * a.P, per_req = per_head * a.H;
-  const int64_t e = blockIdx.x * (int64_t)blockDim.x + threadIdx.x;
-  if (e >= per_req) return;
-  const int h = (int)(e / per_head);
+  int64_t e = blockIdx.x * (int64_t)blockDim.x + threadIdx.x;
+  const bool key = e >= per_req;                     // behind the states: the summed keys
+  if (key) e -= per_req;
+  if (e >= (key ? (a.keys ? (int64_t)a.H * a.N : 0) : per_req)) return;
+  const int h = (int)(e / (key ? a.N : per_head));
   const int64_t len = a.cu[b + 1] - a.cu[b];
   const int spans = (int)((len + a.span - 1) / a.span);
   if (spans <= 0) return;
-  float carry = a.state[(int64_t)a.slots[b] * a.state_stride + e];
+  float carry = (key ? a.keys : a.state)[(int64_t)a.slots[b] * a.state_stride + e];
   for (int c = 0; c < spans; ++c) {
-    float* at = a.span_state + ((int64_t)b * a.max_spans + c) * per_req + e;
+    float* at = key ? a.span_keys + ((int64_t)b * a.max_spans + c) * a.H * a.N + e : a.span_state + ((int64_t)b * a.max_spans + c) * per_req + e;
     const float ended = *at;
     *at = carry;
     carry = a.span_decay[((int64_t)b * a.max_spans + c) * a.H + h] * carry + ended;
@@ -581,6 +710,16 @@ __global__ void __launch_bounds__(256) recurrence_step_kernel(RecArgs a) {
     const float step = z > 20.f ? z : log1pf(expf(z));
     da = expf(-a.rate[h] * step);
     db = step;
+  } else if (a.gates.i) {
+    float gi, gf;
+    read_gates<TX>(a.gates, b, h, gi, gf);
+    const float before = a.gates.m[(int64_t)a.slots[b] * a.gates.m_stride + h];     // moved on by whoever reads the outputs
+    const float now = fmaxf(gf + before, gi);
+    da = expf(gf + before - now);
+    db = expf(gi - now);
+  } else if (a.coef_a) {
+    da = a.coef_a[(int64_t)b * a.H + h];
+    db = a.coef_b[(int64_t)b * a.H + h];
   } else {
     da = a.decay[h];
     db = 1.f;
@@ -610,31 +749,44 @@ __global__ void __launch_bounds__(256) recurrence_step_kernel(RecArgs a) {
     if (a.skip) y += a.skip[h] * vv;
     a.y[(int64_t)b * a.H * a.P + (int64_t)h * a.P + p] = y;
   }
+  if (a.keys != nullptr && blockIdx.y == 0) {         // the summed keys and their product with q
+    __shared__ float scratch[16];
+    float* kr = a.keys + (int64_t)a.slots[b] * a.state_stride + (int64_t)h * a.N;
+    float dot = 0.f;
+    for (int i = threadIdx.x; i < a.N; i += 256) {
+      const float next = fmaf(da, kr[i], db * sk[i]);
+      kr[i] = next;
+      dot += next * sq[i];
+    }
+    dot = block_sum(dot, scratch);
+    if (threadIdx.x == 0) a.key_dot[(int64_t)b * a.H + h] = dot;
+  }
 }
 
-template <typename TX, int NT, int HPB, int PPB>
+template <typename TX, int NT, int HPB, int PPB, bool KEYS>
 static int launch_recurrence(RecArgs& a, int num_seqs, int spans, hipStream_t stream) {
   const int slices = (a.N + NT - 1) / NT;
   const dim3 block(64);
   const unsigned pblocks = (a.P + 64 * PPB - 1) / (64 * PPB);
   if (spans <= 1) {
-    recurrence_kernel<TX, NT, 0, HPB, PPB><<<dim3(num_seqs * (a.H / HPB), pblocks, slices), block, 0, stream>>>(a);
+    recurrence_kernel<TX, NT, 0, HPB, PPB, KEYS><<<dim3(num_seqs * (a.H / HPB), pblocks, slices), block, 0, stream>>>(a);
     ME_LAUNCH_CHECK();
     return 0;
   }
   const dim3 grid(num_seqs * (a.H / HPB), pblocks, slices * spans);
-  recurrence_kernel<TX, NT, 1, HPB, PPB><<<grid, block, 0, stream>>>(a);
+  recurrence_kernel<TX, NT, 1, HPB, PPB, KEYS><<<grid, block, 0, stream>>>(a);
   ME_LAUNCH_CHECK();
-  const int64_t per_req = (int64_t)a.H * a.N * a.P;
+  const int64_t per_req = (int64_t)a.H * a.N * a.P + (KEYS ? (int64_t)a.H * a.N : 0);
   recurrence_carry_kernel<<<dim3((unsigned)((per_req + 255) / 256), num_seqs), dim3(256), 0, stream>>>(a);
   ME_LAUNCH_CHECK();
-  recurrence_kernel<TX, NT, 2, HPB, PPB><<<grid, block, 0, stream>>>(a);
+  recurrence_kernel<TX, NT, 2, HPB, PPB, KEYS><<<grid, block, 0, stream>>>(a);
   ME_LAUNCH_CHECK();
   return 0;
 }
 
 // spans <= 1: every request's tokens in one pass. Otherwise the tokens are cut into spans of `span` tokens that run
 // side by side (at most `spans` per request), and scratch holds spans * H * N * P + spans * H floats per request.
+// keys: the summed keys beside the states, in the same state rows (see RecArgs); scratch then holds spans * H * N more.
 // columns: 1, or 2: a lane keeps two columns of the state (two blocks of 64 columns of one head where P > 64, else
 // the same columns of two neighbouring heads of one group, which needs an even number of heads per group).
 extern "C" int me_linear_recurrence(const void* q, int64_t q_stride, const void* k, int64_t k_stride, const void* v,
@@ -642,10 +794,17 @@ extern "C" int me_linear_recurrence(const void* q, int64_t q_stride, const void*
                                     const float* dt_bias, const float* rate, const float* skip, float* state,
                                     int64_t state_stride, const int32_t* slots, const int32_t* cu, float* y,
                                     int64_t y_slice_stride, int num_seqs, int H, int G, int N, int P, int rows_per_wave,
-                                    int columns, int silu, int span, int spans, float* scratch, hipStream_t stream) {
+                                    int columns, int silu, int span, int spans, float* scratch, const float* coef_a,
+                                    const float* coef_b, float* keys, float* key_dot, int64_t dot_slice_stride, const void* gate_i,
+                                    const void* gate_f, int64_t gate_stride, const float* bias_i, const float* bias_f, float cap,
+                                    float* gate_m, int64_t gate_m_stride, hipStream_t stream) {
   if (num_seqs == 0) return 0;
   ME_CHECK(H >= 1 && G >= 1 && H % G == 0 && N >= 1 && P >= 1, "recurrence: bad sizes H=%d G=%d N=%d P=%d", H, G, N, P);
-  ME_CHECK((dt != nullptr) != (decay != nullptr), "recurrence: give fixed decays or step sizes, not both");
+  ME_CHECK((dt != nullptr) + (decay != nullptr) + (coef_a != nullptr) + (gate_i != nullptr) == 1,
+           "recurrence: give one of fixed decays, step sizes, factors per token, gates");
+  ME_CHECK((coef_a != nullptr) == (coef_b != nullptr) && (gate_i == nullptr || (gate_f && bias_i && bias_f && gate_m && cap > 0.f && rows_per_wave == 0)),
+           "recurrence: factors come in pairs, gates belong to steps of single tokens");
+  ME_CHECK((keys != nullptr) == (key_dot != nullptr) && (keys == nullptr || columns == 1), "recurrence: summed keys with one column per lane");
   ME_CHECK(dt == nullptr || (dt_bias && rate), "recurrence: step sizes need their bias and rates");
   ME_CHECK((int64_t)num_seqs * H <= 2147483647ll, "recurrence: too many (request, head) pairs");
   ME_CHECK(spans <= 1 || (span >= 1 && scratch != nullptr), "recurrence: spans need a length and scratch");
@@ -660,6 +819,10 @@ extern "C" int me_linear_recurrence(const void* q, int64_t q_stride, const void*
   a.silu = silu;
   a.span_state = scratch;
   a.span_decay = scratch ? scratch + (int64_t)num_seqs * a.max_spans * H * N * P : nullptr;
+  a.span_keys = scratch && keys ? a.span_decay + (int64_t)num_seqs * a.max_spans * H : nullptr;
+  a.coef_a = coef_a; a.coef_b = coef_b; a.keys = keys; a.key_dot = key_dot; a.dot_slice_stride = dot_slice_stride;
+  a.gates.i = gate_i; a.gates.f = gate_f; a.gates.stride = gate_stride; a.gates.bias_i = bias_i; a.gates.bias_f = bias_f;
+  a.gates.cap = cap; a.gates.m = gate_m; a.gates.m_stride = gate_m_stride;
   if (rows_per_wave == 0) {                // a step of single tokens: one pass over the state, one output
     ME_CHECK((int64_t)(2 * N + 256) * 4 <= 64 * 1024 && (P + 63) / 64 <= 65535, "recurrence: a state of %d rows does not fit the step kernel", N);
     const dim3 grid(num_seqs * H, (P + 63) / 64);
@@ -673,9 +836,10 @@ extern "C" int me_linear_recurrence(const void* q, int64_t q_stride, const void*
   ME_CHECK((int64_t)slices * a.max_spans <= 65535, "recurrence: too many slices and spans for one launch");
 #define REC_NT(TX, NT)                                                                               \
   do {                                                                                               \
-    if (columns == 1) return launch_recurrence<TX, NT, 1, 1>(a, num_seqs, spans, stream);            \
-    if (two_heads) return launch_recurrence<TX, NT, 2, 1>(a, num_seqs, spans, stream);               \
-    return launch_recurrence<TX, NT, 1, 2>(a, num_seqs, spans, stream);                              \
+    if (keys) return launch_recurrence<TX, NT, 1, 1, true>(a, num_seqs, spans, stream);              \
+    if (columns == 1) return launch_recurrence<TX, NT, 1, 1, false>(a, num_seqs, spans, stream);     \
+    if (two_heads) return launch_recurrence<TX, NT, 2, 1, false>(a, num_seqs, spans, stream);        \
+    return launch_recurrence<TX, NT, 1, 2, false>(a, num_seqs, spans, stream);                       \
   } while (0)
 #define REC(TX)                                                                              \
   switch (rows_per_wave) {                                                                   \
@@ -725,12 +889,186 @@ __global__ void gated_rms_norm_kernel(const float* __restrict__ y, int parts, in
   }
 }
 
+// The same with several groups of up to 1,024 numbers in whole steps of 4: LPG lanes to a group (16, 32 or 64, a lane holds
+// up to four groups of 4 neighbours), the group's sum by exchanges between those lanes, no meeting of the workgroup.
+// With `dot` (memory_readout): y is divided by max(|dot|, floor) + 1e-6 first, dot being the `parts` slices [parts, T,
+// groups] added up; floor [T, groups], or, for a step of single tokens, exp(-m') of the gates, whose maximum moves on here.
+// y and dot are multiplied by `scale` on the way in.
+struct Readout {
+  const float* dot; const float* floor_in; float scale;
+  SoftGates gates; const int32_t* slots;
+};
+
+template <typename TX, int KIND, int LPG, int J, bool READ>
+__global__ void __launch_bounds__(256) grouped_norm_kernel(const float* __restrict__ y, int parts, int64_t part_stride, const TX* __restrict__ gate,
+                                                           int64_t gate_stride, const float* __restrict__ w, TX* __restrict__ out, int n,
+                                                           int groups, float eps, int64_t T, Readout r) {
+  constexpr int GPW = 256 / LPG;
+  const int64_t tg = (int64_t)blockIdx.x * GPW + threadIdx.x / LPG;
+  const int lane = threadIdx.x % LPG;
+  const int per = n / groups;
+  const bool live = tg < T * groups;
+  const int64_t t = live ? tg / groups : 0;
+  const int g = live ? (int)(tg - t * groups) : 0;
+  float v[J][4], gt[J][4], wv[J][4];
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < J; ++j) {
+    const int i = (lane + j * LPG) * 4;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) { v[j][e] = 0.f; gt[j][e] = 0.f; wv[j][e] = 0.f; }
+    if (i < per && live) {
+      const int64_t at = t * n + g * per + i;
+      for (int p = 0; p < parts; ++p) {
+        float x[4];
+        Group4<float>::load(y + p * part_stride + at, x);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[j][e] += x[e];
+      }
+      Group4<TX>::load(gate + t * gate_stride + g * per + i, gt[j]);
+      Group4<float>::load(w + g * per + i, wv[j]);
+    }
+  }
+  float under = 1.f;
+  if (READ) {
+    float dot = 0.f;
+    for (int p = 0; p < parts; ++p) dot += r.dot[p * T * groups + t * groups + g];
+    float low;
+    if (r.gates.i) {
+      float gi, gf;
+      read_gates<TX>(r.gates, t, g, gi, gf);
+      float* held = r.gates.m + (int64_t)r.slots[t] * r.gates.m_stride + g;
+      const float now = fmaxf(gf + *held, gi);
+      low = expf(-now);
+      if (live && lane == 0) *held = now;
+    } else low = r.floor_in[t * groups + g];
+    under = r.scale / (fmaxf(fabsf(r.scale * dot), low) + 1e-6f);
+  }
+#pragma unroll
+  for (int j = 0; j < J; ++j)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      if (READ) v[j][e] *= under;
+      if (KIND == 0) v[j][e] *= silu_f(gt[j][e]);
+      ss += v[j][e] * v[j][e];
+    }
+#pragma unroll
+  for (int off = LPG / 2; off > 0; off >>= 1) ss += __shfl_xor(ss, off, LPG);
+  const float inv = 1.0f / sqrtf(ss / (float)per + eps);
+#pragma unroll
+  for (int j = 0; j < J; ++j) {
+    const int i = (lane + j * LPG) * 4;
+    if (i < per && live) {
+      float o[4];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        o[e] = v[j][e] * inv * wv[j][e];
+        if (KIND == 1) o[e] *= sigmoid_f(gt[j][e]);
+        if (KIND == 2) o[e] *= silu_f(gt[j][e]);
+      }
+      Group4<TX>::store(out + t * n + g * per + i, o);
+    }
+  }
+}
+
+// One workgroup of a wave per (token, group) for groups of any size (memory_readout only).
+template <typename TX>
+__global__ void __launch_bounds__(64) memory_readout_any_kernel(const float* __restrict__ y, int parts, int64_t part_stride, const TX* __restrict__ gate,
+                                                                int64_t gate_stride, const float* __restrict__ w, TX* __restrict__ out, int n,
+                                                                int groups, float eps, int64_t T, Readout r) {
+  const int64_t t = blockIdx.x / groups;
+  const int g = (int)(blockIdx.x - t * groups), lane = threadIdx.x, per = n / groups;
+  float dot = 0.f;
+  for (int p = 0; p < parts; ++p) dot += r.dot[p * T * groups + t * groups + g];
+  float low;
+  if (r.gates.i) {
+    float gi, gf;
+    read_gates<TX>(r.gates, t, g, gi, gf);
+    float* held = r.gates.m + (int64_t)r.slots[t] * r.gates.m_stride + g;
+    const float now = fmaxf(gf + *held, gi);
+    low = expf(-now);
+    __syncthreads();                        // every lane has read the maximum
+    if (lane == 0) *held = now;
+  } else low = r.floor_in[t * groups + g];
+  const float under = r.scale / (fmaxf(fabsf(r.scale * dot), low) + 1e-6f);
+  float ss = 0.f;
+  for (int i = lane; i < per; i += 64) {
+    float v = 0.f;
+    for (int p = 0; p < parts; ++p) v += y[p * part_stride + t * n + g * per + i];
+    v *= under;
+    ss += v * v;
+  }
+  ss = wave_sum(ss);
+  const float inv = 1.0f / sqrtf(ss / (float)per + eps);
+  for (int i = lane; i < per; i += 64) {
+    float v = 0.f;
+    for (int p = 0; p < parts; ++p) v += y[p * part_stride + t * n + g * per + i];
+    const int c = g * per + i;
+    out[t * n + c] = from_f32<TX>(v * under * inv * w[c] * sigmoid_f(to_f32<TX>(gate[t * gate_stride + c])));
+  }
+}
+
+template <typename TX, int KIND, bool READ>
+static bool launch_grouped_norm(const float* y, int parts, int64_t part_stride, const TX* gate, int64_t gate_stride, const float* w, TX* out,
+                                int64_t T, int n, int groups, float eps, const Readout& r, hipStream_t stream) {
+  const int per = n / groups;
+  const bool aligned = ((reinterpret_cast<uintptr_t>(y) | reinterpret_cast<uintptr_t>(w) | reinterpret_cast<uintptr_t>(out)) % 16) == 0 &&
+                       reinterpret_cast<uintptr_t>(gate) % (4 * sizeof(TX)) == 0;
+  if (per % 4 || per > 1024 || gate_stride % 4 || part_stride % 4 || !aligned || T * groups > (1ll << 33)) return false;
+#define GR(LPG, J)                                                                                                                   \
+  grouped_norm_kernel<TX, KIND, LPG, J, READ><<<dim3((unsigned)((T * groups + 256 / LPG - 1) / (256 / LPG))), dim3(256), 0, stream>>>( \
+      y, parts, part_stride, gate, gate_stride, w, out, n, groups, eps, T, r)
+  if (per <= 64) GR(16, 1);
+  else if (per <= 128) GR(32, 1);
+  else if (per <= 256) GR(64, 1);
+  else if (per <= 512) GR(64, 2);
+  else GR(64, 4);
+#undef GR
+  return true;
+}
+
+extern "C" int me_memory_readout(const float* y, int parts, int64_t part_stride, const float* dot, const float* floor_in, float scale,
+                                 const void* gate, int64_t gate_stride, int dtype, const float* w, void* out, int64_t T, int n, int groups,
+                                 float eps, const void* gate_i, const void* gate_f, int64_t soft_stride, const float* bias_i,
+                                 const float* bias_f, float cap, float* gate_m, int64_t gate_m_stride, const int32_t* slots, hipStream_t stream) {
+  if (T == 0) return 0;
+  ME_CHECK(n >= 1 && groups >= 1 && n % groups == 0 && parts >= 1, "memory_readout: width %d, %d heads", n, groups);
+  ME_CHECK((floor_in != nullptr) != (gate_i != nullptr) && (gate_i == nullptr || (gate_f && bias_i && bias_f && gate_m && slots && cap > 0.f)),
+           "memory_readout: give the floors or the gates");
+  ME_CHECK(T * groups <= 2147483647ll, "memory_readout: too many tokens");
+  Readout r;
+  r.dot = dot; r.floor_in = floor_in; r.scale = scale; r.slots = slots;
+  r.gates.i = gate_i; r.gates.f = gate_f; r.gates.stride = soft_stride; r.gates.bias_i = bias_i; r.gates.bias_f = bias_f; r.gates.cap = cap;
+  r.gates.m = gate_m; r.gates.m_stride = gate_m_stride;
+  bool done;
+  if (dtype == ME_F32) done = launch_grouped_norm<float, 1, true>(y, parts, part_stride, (const float*)gate, gate_stride, w, (float*)out, T, n, groups, eps, r, stream);
+  else done = launch_grouped_norm<bf16_t, 1, true>(y, parts, part_stride, (const bf16_t*)gate, gate_stride, w, (bf16_t*)out, T, n, groups, eps, r, stream);
+  if (!done) {
+    const dim3 grid((unsigned)(T * groups)), block(64);
+    if (dtype == ME_F32) memory_readout_any_kernel<float><<<grid, block, 0, stream>>>(y, parts, part_stride, (const float*)gate, gate_stride, w, (float*)out, n, groups, eps, T, r);
+    else memory_readout_any_kernel<bf16_t><<<grid, block, 0, stream>>>(y, parts, part_stride, (const bf16_t*)gate, gate_stride, w, (bf16_t*)out, n, groups, eps, T, r);
+  }
+  ME_LAUNCH_CHECK();
+  return 0;
+}
+
 extern "C" int me_gated_rms_norm(const float* y, int parts, int64_t part_stride, const void* gate, int64_t gate_stride,
                                  int dtype, const float* w, void* out, int64_t T, int n, int groups, int kind, float eps,
                                  hipStream_t stream) {
   if (T == 0) return 0;
   ME_CHECK(n >= 1 && n <= 15360 && groups >= 1 && n % groups == 0, "gated_rms_norm: width %d, %d groups", n, groups);
   ME_CHECK(parts >= 1 && parts <= 64 && kind >= 0 && kind <= 2, "gated_rms_norm: bad slice count or kind");
+  if (groups > 1) {
+    bool done;
+#define GG(TX, K) done = launch_grouped_norm<TX, K, false>(y, parts, part_stride, (const TX*)gate, gate_stride, w, (TX*)out, T, n, groups, eps, Readout{}, stream)
+    if (dtype == ME_F32) { if (kind == 0) GG(float, 0); else if (kind == 1) GG(float, 1); else GG(float, 2); }
+    else { if (kind == 0) GG(bf16_t, 0); else if (kind == 1) GG(bf16_t, 1); else GG(bf16_t, 2); }
+#undef GG
+    if (done) {
+      ME_LAUNCH_CHECK();
+      return 0;
+    }
+  }
   const dim3 grid((unsigned)T), block(n >= 1024 ? 256 : (n > 256 ? 128 : 64));
   const size_t lds = (size_t)n * sizeof(float);
 #define GN(TX, K) gated_rms_norm_kernel<TX, K><<<grid, block, lds, stream>>>(y, parts, part_stride, (const TX*)gate, gate_stride, w, (TX*)out, n, groups, eps)

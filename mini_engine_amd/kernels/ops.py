@@ -21,7 +21,7 @@ from . import build
 ME_BF16, ME_F32 = 0, 1
 ACTIVATIONS = {"silu": 0, "relu2": 1, "tanh": 2, "gelu_tanh": 3}          # elementwise activations of `activation`
 GATED_NORMS = {"silu_before": 0, "sigmoid_behind": 1, "silu_behind": 2}
-DECAY_RULES = {"bonus": 0, "delta": 1, "gated": 2}         # update rules of `decay_rows_recurrence`
+DECAY_RULES = {"bonus": 0, "delta": 1, "gated": 2, "delta_head": 3}         # update rules of `decay_rows_recurrence`
 _DT = {torch.bfloat16: ME_BF16, torch.float32: ME_F32}
 
 
@@ -78,12 +78,16 @@ _CORE_PROTOS = {
     "me_activation": [P, L, P, I, I, L, I, P],
     "me_head_gate": [P, P, L, I, L, I, I, P],
     "me_causal_conv": [P, L, I, P, P, P, L, P, P, I, P, L, I, I, I, P],
-    "me_linear_recurrence": [P, L, P, L, P, L, I, P, L, P, P, P, P, P, L, P, P, P, L, I, I, I, I, I, I, I, I, I, I, P, P],
+    "me_linear_recurrence": [P, L, P, L, P, L, I, P, L, P, P, P, P, P, L, P, P, P, L, I, I, I, I, I, I, I, I, I, I, P,
+                             P, P, P, P, L, P, P, L, P, P, F, P, L, P],
+    "me_soft_gates": [P, P, L, I, P, P, F, P, L, P, P, P, P, P, I, I, P],
+    "me_memory_readout": [P, I, L, P, P, F, P, L, I, P, P, L, I, I, F, P, P, L, P, P, F, P, L, P, P],
+    "me_stream_mix_norm": [P, I, L, L, P, L, I, P, P, P, P, P, P, P, P, P, P, I, F, P, I, L, I, I, P],
     "me_gated_rms_norm": [P, I, L, P, L, I, P, P, L, I, I, I, F, P],
     "me_scaled_sum_norm": [P, I, I, P, P, P, P, P, F, P, P, P, P, P, I, L, I, F, P],
     "me_softcap": [P, L, L, I, F, P],
     "me_qkv_prepare": [P, L, P, P, P, F, I, I, F, I, P, P, P, P, P, L, I, L, I, I, I, I, I, I, P, P, L, P],
-    "me_moe_route": [P, L, I, P, L, I, I, I, I, I, P, P, P, I, I, I, I, F, P, P],
+    "me_moe_route": [P, L, I, P, P, L, I, I, I, I, I, P, P, P, I, I, I, I, F, P, P],
     "me_moe_sort": [P, L, I, I, I, P, P, P, P, P, P, I, I, I, I, I, I, F, P, P],
     "me_moe_gate_up": [P, L, P, P, P, P, P, P, L, I, I, I, I, I, I, P],
     "me_moe_down": [P, P, P, P, P, P, P, P, L, I, I, I, I, I, P],
@@ -92,7 +96,7 @@ _CORE_PROTOS = {
     "me_sigmoid_gate": [P, L, P, L, I, L, I, P],
     "me_glu_clamped": [P, L, P, I, L, I, F, F, P],
     "me_weighted_sum": [I, P, P, P, P, P, P, P, P, F, P, P, P, I, L, I, P, P, P, P],
-    "me_latent_prepare": [P, L, I, I, I, I, I, I, I, I, P, F, P, L, P, P, P, L, P, P, I, L, P],
+    "me_latent_prepare": [P, L, I, I, I, I, I, I, I, I, P, F, P, L, P, P, P, L, P, P, I, I, I, P, P, L, P],
     "me_heads_linear": [P, L, L, P, P, L, L, I, L, I, I, I, P],
     "me_token_shift": [P, L, I, P, I, P, L, P, P, P, P, L, I, P],
     "me_decay_rows_recurrence": [P, L, P, L, P, L, P, L, P, L, I, P, P, P, P, L, P, P, P, I, I, I, I, I, I, I, F, F, I, L, P, P],
@@ -245,23 +249,59 @@ def library_product(x: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype, sp
 
 
 class RouteRule:
-    """How a router's float32 logits become a choice of experts and their weights (`moe_route`). scoring: "softmax" over
-    all experts or "sigmoid" per expert; correction: float32 [experts] added to the scores for the choice only, or None;
+    """How a router's float32 logits become a choice of experts and their weights (`moe_route`). bias: float32 [experts]
+    added to the logits, or None. scoring: "softmax" over all experts, "sigmoid" per expert, or "chosen": the choice goes by
+    the logits and the weights are their softmax over the chosen experts alone (`normalise` has no say); correction: float32 [experts] added to the scores for the choice only, or None;
     group_top: a group of neighbours scores as the sum of its so many largest choice scores; normalise: the chosen
     experts' scores are divided by their sum; scale: a constant on the weights."""
 
-    def __init__(self, scoring: str = "softmax", correction=None, group_top: int = 1, normalise: bool = True, scale: float = 1.0):
-        if scoring not in ("softmax", "sigmoid") or group_top < 1:
-            raise ValueError("scoring is 'softmax' or 'sigmoid', group_top positive")
+    SCORINGS = {"softmax": 0, "sigmoid": 1, "chosen": 2}
+
+    def __init__(self, scoring: str = "softmax", correction=None, group_top: int = 1, normalise: bool = True, scale: float = 1.0, bias=None):
+        if scoring not in self.SCORINGS or group_top < 1:
+            raise ValueError(f"scoring is one of {sorted(self.SCORINGS)}, group_top positive")
+        self.bias = bias
         self.scoring, self.correction, self.group_top = scoring, correction, int(group_top)
         self.normalise, self.scale = bool(normalise), float(scale)
 
     def check(self, E: int) -> None:
-        c = self.correction
-        _check(c is None or (c.dtype == torch.float32 and c.shape == (E,) and c.is_contiguous()), "moe_route: the correction must be float32 [experts]")
+        for c in (self.correction, self.bias):
+            _check(c is None or (c.dtype == torch.float32 and c.shape == (E,) and c.is_contiguous()),
+                   "moe_route: the correction and the bias must be float32 [experts]")
 
     def args(self) -> tuple:
-        return (self.group_top, int(self.scoring == "sigmoid"), int(self.normalise), self.scale, _ptr(self.correction))
+        return (self.group_top, self.SCORINGS[self.scoring], int(self.normalise), self.scale, _ptr(self.correction))
+
+
+class SoftGates:
+    """Exponential input and forget gates of a recurrence under a running maximum m (one number per head in the request's
+    state, starting at 0): with z the raw rows plus bias, bent under a cap c: i = c tanh(z_i / c), f = log sigmoid(c tanh(z_f /
+    c)); m' = max(f + m, i); a = exp(f + m - m'), b = exp(i - m'). i, f: row views [T, H] of one stride; bias_i, bias_f: float32
+    [H]; m: a float32 view [slots, H]; slots: int32, the requests' state rows."""
+
+    def __init__(self, i, f, bias_i, bias_f, cap: float, m, slots):
+        self.i, self.f, self.bias_i, self.bias_f, self.cap, self.m, self.slots = i, f, bias_i, bias_f, float(cap), m, slots
+
+    def check(self, T: int, H: int, dtype: torch.dtype) -> None:
+        for t in (self.i, self.f):
+            _check(t.shape == (T, H) and t.stride(1) == 1 and t.stride(0) == self.i.stride(0) and t.dtype == dtype, "gates: row views [T, H] of one stride")
+        for t in (self.bias_i, self.bias_f):
+            _check(t.dtype == torch.float32 and t.shape == (H,) and t.is_contiguous(), "gates: biases float32 [H]")
+        _check(self.m.dtype == torch.float32 and self.m.dim() == 2 and self.m.shape[1] == H and self.m.stride(1) == 1 and self.cap > 0
+               and _is_i32(self.slots), "gates: the maxima float32 [slots, H], a positive cap")
+
+    def args(self) -> tuple:
+        return (self.i.data_ptr(), self.f.data_ptr(), self.i.stride(0), self.bias_i.data_ptr(), self.bias_f.data_ptr(), self.cap,
+                self.m.data_ptr(), self.m.stride(0))
+
+
+class MemoryReads:
+    """What a recurrence with summed keys has read: y (S^T q) and dot (n . q), float32 [T, H * P] and [T, H] or slices of both
+    that are still to be added; floor: exp(-m) [T, H], or None after a step of single tokens, where the gates' maximum has not
+    moved on yet (`memory_readout` does that)."""
+
+    def __init__(self, y, dot, floor, gates: SoftGates):
+        self.y, self.dot, self.floor, self.gates = y, dot, floor, gates
 
 
 class HipBackend:
@@ -718,13 +758,17 @@ class HipBackend:
         return out
 
     def linear_recurrence(self, q, k, v, state, state_slots, cu_seqlens, q_lens, H: int, G: int, N: int, P: int,
-                          decay=None, dt=None, dt_bias=None, rate=None, skip=None, silu: bool = False) -> torch.Tensor:
+                          decay=None, dt=None, dt_bias=None, rate=None, skip=None, silu: bool = False, gates: "SoftGates | None" = None,
+                          key_state=None):
         """Per request and head, over the request's tokens of this step in order, from its state row:
             S_t = a_t S_(t-1) + b_t k_t v_t^T,   y_t = S_t^T q_t (+ skip_h v_t),      S [N, P] float32.
         q, k: row views [T, G * N] (heads share them by groups of H / G), v: [T, H * P]; state: float32 view
         [slots, H * N * P], rows `state_slots`, left at the state behind the last token. a, b: `decay` (float32 [H])
         and 1; or exp(-rate_h dt), dt with dt = softplus(dt[t, h] + dt_bias_h) (`dt` a row view [T, H], the others
-        float32 [H]). `silu`: q, k and v pass silu on their way in. `q_lens`: the requests' token counts on the host: long ones are cut into spans that run side
+        float32 [H]); or `gates` (`SoftGates`): exponential input and forget gates under a running maximum, whose state moves
+        on too. With gates the summed keys are kept beside the states, n_t = a_t n_(t-1) + b_t k_t (`key_state`: a float32 view [slots,
+        H * N] of the same state rows), and the result is a `MemoryReads` for `memory_readout`. `silu`: q, k and v pass silu
+        on their way in. `q_lens`: the requests' token counts on the host: long ones are cut into spans that run side
         by side (`recurrence_spans`). Returns float32 [T, H * P], or partial sums [S, T, H * P] over slices of N
         for a consumer that adds them."""
         T, B = v.shape[0], state_slots.numel()
@@ -733,32 +777,105 @@ class HipBackend:
             _check(t.dim() == 2 and t.shape == (T, width) and t.stride(1) == 1 and t.dtype == dtype, "recurrence: bad q, k or v rows")
         _check(state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1 and state.shape[1] == H * N * P,
                "recurrence: state must be float32 [slots, H * N * P]")
-        _check((decay is None) != (dt is None), "recurrence: fixed decays or step sizes")
+        _check((decay is not None) + (dt is not None) + (gates is not None) == 1, "recurrence: fixed decays, step sizes or gates")
+        _check((gates is None) == (key_state is None), "recurrence: gates come with the summed keys' state")
+        if gates is not None:
+            gates.check(T, H, dtype)
+            _check(key_state.dtype == torch.float32 and key_state.shape[1] == H * N and key_state.stride() == state.stride(),
+                   "recurrence: the summed keys' state must be float32 [slots, H * N] of the same state rows")
         for w in (decay, dt_bias, rate, skip):
             _check(w is None or (w.dtype == torch.float32 and w.shape == (H,) and w.is_contiguous()), "recurrence: per-head constants float32 [H]")
         if dt is not None:
             _check(dt.shape == (T, H) and dt.stride(1) == 1 and dt.dtype == dtype and dt_bias is not None and rate is not None,
                    "recurrence: step sizes [T, H] with bias and rates")
         _check(_is_i32(state_slots) and _is_i32(cu_seqlens, B + 1) and len(q_lens) == B, "recurrence: metadata")
+        none = (None, None, None, None, 0)                # factors, summed keys and their product with q
+        no_gates = (None, None, 0, None, None, 0.0, None, 0)
         if T == B and N <= RECURRENCE_STEP_MAX_ROWS:
-            # every request brings one token: the state streams through once, one output row per token
+            # every request brings one token: the state streams through once, one output row per token (with gates: a and b
+            # are formed by whoever needs them, and the readout moves the maximum on)
+            dot = torch.empty((T, H), dtype=torch.float32, device=v.device) if gates is not None else None
             y = torch.empty((T, H * P), dtype=torch.float32, device=v.device)
             core().call("me_linear_recurrence", q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0),
                         _code(dtype), _ptr(dt), 0 if dt is None else dt.stride(0), _ptr(decay), _ptr(dt_bias), _ptr(rate), _ptr(skip),
                         state.data_ptr(), state.stride(0), state_slots.data_ptr(), cu_seqlens.data_ptr(), y.data_ptr(), T * H * P,
-                        B, H, G, N, P, 0, 1, int(silu), 0, 1, None, _stream())
-            return y
+                        B, H, G, N, P, 0, 1, int(silu), 0, 1, None,
+                        *(none if gates is None else (None, None, key_state.data_ptr(), dot.data_ptr(), T * H)),
+                        *(no_gates if gates is None else gates.args()), _stream())
+            return y if gates is None else MemoryReads(y, dot, None, gates)
         per_wave = recurrence_rows_per_wave(N)
         slices = -(-N // per_wave)
-        columns = recurrence_columns(q_lens, H, G, P, slices)
+        columns = recurrence_columns(q_lens, H, G, P, slices) if gates is None else 1
         span, spans = recurrence_spans(q_lens, H * -(-P // 64) * slices // columns, 65535 // slices)
-        scratch = _scratch(B * spans * (H * N * P + H), v.device, "recurrence") if spans > 1 else None
+        if gates is not None:
+            factors = torch.empty((3, T, H), dtype=torch.float32, device=v.device)            # a, b, exp(-m)
+            dot = torch.empty((slices, T, H) if slices > 1 else (T, H), dtype=torch.float32, device=v.device)
+            i, f, stride, bi, bf, cap, m, m_stride = gates.args()
+            core().call("me_soft_gates", i, f, stride, _code(dtype), bi, bf, cap, m, m_stride, state_slots.data_ptr(), cu_seqlens.data_ptr(),
+                        factors[0].data_ptr(), factors[1].data_ptr(), factors[2].data_ptr(), B, H, _stream())
+        scratch = _scratch(B * spans * (H * N * P + H + (H * N if gates is not None else 0)), v.device, "recurrence") if spans > 1 else None
         y = torch.empty((slices, T, H * P) if slices > 1 else (T, H * P), dtype=torch.float32, device=v.device)
         core().call("me_linear_recurrence", q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0),
                     _code(dtype), _ptr(dt), 0 if dt is None else dt.stride(0), _ptr(decay), _ptr(dt_bias), _ptr(rate), _ptr(skip),
                     state.data_ptr(), state.stride(0), state_slots.data_ptr(), cu_seqlens.data_ptr(), y.data_ptr(), T * H * P,
-                    B, H, G, N, P, per_wave, columns, int(silu), span, spans, _ptr(scratch), _stream())
-        return y
+                    B, H, G, N, P, per_wave, columns, int(silu), span, spans, _ptr(scratch),
+                    *(none if gates is None else (factors[0].data_ptr(), factors[1].data_ptr(), key_state.data_ptr(), dot.data_ptr(), T * H)),
+                    *no_gates, _stream())
+        return y if gates is None else MemoryReads(y, dot, factors[2], gates)
+
+    def memory_readout(self, reads: "MemoryReads", gate, weight, eps: float, heads: int, q_scale: float, out_dtype: torch.dtype) -> torch.Tensor:
+        """o = c y / (max(|c n . q|, exp(-m)) + 1e-6) per head (c: `q_scale`, a factor of the queries), then o / rms(o) * weight *
+        sigmoid(gate), the root mean square over each head. reads: what `linear_recurrence` returns with gates; gate: a row
+        view [T, n] of out_dtype; weight: float32 [n]. Returns [T, n]."""
+        y, dot = reads.y, reads.dot
+        parts = y.shape[0] if y.dim() == 3 else 1
+        T, n = y.shape[-2], y.shape[-1]
+        _check(y.dtype == torch.float32 and y.is_contiguous() and dot.is_contiguous() and dot.shape[-2:] == (T, heads)
+               and (dot.shape[0] if dot.dim() == 3 else 1) == parts, "memory_readout: outputs and key products of one recurrence")
+        _check(gate.shape == (T, n) and gate.stride(1) == 1 and gate.dtype == out_dtype, "memory_readout: gate [T, n] of the output dtype")
+        _check(weight.dtype == torch.float32 and weight.shape == (n,) and weight.is_contiguous() and n % heads == 0, "memory_readout: weight float32 [n]")
+        out = torch.empty((T, n), dtype=out_dtype, device=y.device)
+        step = reads.floor is None                        # a step of single tokens: the maximum moves on here
+        g = reads.gates
+        core().call("me_memory_readout", y.data_ptr(), parts, T * n, dot.data_ptr(), _ptr(reads.floor), float(q_scale), gate.data_ptr(),
+                    gate.stride(0), _code(out_dtype), weight.data_ptr(), out.data_ptr(), T, n, heads, float(eps),
+                    *(g.args() if step else (None, None, 0, None, None, 0.0, None, 0)), g.slots.data_ptr() if step else None, _stream())
+        return out
+
+    # -- several residual streams ----------------------------------------------------------------
+    def stream_mix_norm(self, streams, count: int, terms, mix, out_weights, read, norm, out_dtype: torch.dtype, rows=None, keep: bool = True):
+        """Several residual streams x_1 .. x_S (S = `count`), float32 [T, S, n], or rows [T, n] (any dtype) that all streams
+        share. x'_t = sum_s mix[s, t] x_s + out_weights[t] y, y the sum of up to four `terms` (rows [T, n] or float32 partial
+        sums [P, T, n]); without mix x'_t = x_t + y. u = sum_t read[t] x'_t (read None: the plain sum). `norm`: (weight float32
+        [n], bias float32 [n] or None, eps, centred): a layer norm (centred: the mean is taken off, the variance is that of the
+        deviations) or an RMS norm of u; None: u itself comes out. `rows` (int32 [R]): only these rows, one result each, in
+        order. `keep`: the new streams are wanted. Returns (x' float32 [R, S, n] or None, the result [R, n] in out_dtype). Where
+        nothing changes the streams and they are float32 [T, S, n] already, they are handed back as they are."""
+        T, n = streams.shape[0], streams.shape[-1]
+        S = int(count)
+        shared = streams.dim() == 2
+        _check(streams.is_contiguous() and (shared or streams.shape[1] == S), "stream_mix_norm: streams [T, S, n] or rows [T, n]")
+        _check(len(terms) <= 4, "stream_mix_norm: up to four terms")
+        f32 = lambda t, shape: t is None or (t.dtype == torch.float32 and t.shape == shape and t.is_contiguous())
+        _check(f32(mix, (S, S)) and f32(out_weights, (S,)) and f32(read, (S,)) and (mix is None) == (out_weights is None),
+               "stream_mix_norm: mix float32 [S, S] with weights [S], read float32 [S]")
+        _check(rows is None or (_is_i32(rows) and rows.dim() == 1), "stream_mix_norm: rows int32 [R]")
+        w, b, eps, centred = norm if norm is not None else (None, None, 0.0, False)
+        _check(f32(w, (n,)) and f32(b, (n,)), "stream_mix_norm: norm weight and bias float32 [n]")
+        k = len(terms)
+        ptrs, dts, parts, strides = (c_void_p * 4)(), (c_int * 4)(), (c_int * 4)(), (c_int64 * 4)()
+        for i, t in enumerate(terms):
+            _check(t.is_contiguous() and t.shape[-2:] == (T, n) and (t.dim() == 2 or (t.dim() == 3 and t.dtype == torch.float32)),
+                   "stream_mix_norm: a term is rows [T, n] or float32 partial sums [P, T, n]")
+            ptrs[i], dts[i], parts[i], strides[i] = t.data_ptr(), _code(t.dtype), (t.shape[0] if t.dim() == 3 else 1), T * n
+        R = T if rows is None else rows.numel()
+        as_they_are = k == 0 and mix is None and not shared and rows is None and streams.dtype == torch.float32
+        new = torch.empty((R, S, n), dtype=torch.float32, device=streams.device) if keep and not as_they_are else None
+        y = torch.empty((R, n), dtype=out_dtype, device=streams.device)
+        core().call("me_stream_mix_norm", streams.data_ptr(), _code(streams.dtype), n if shared else S * n, 0 if shared else n, _ptr(rows), T,
+                    k, ptrs, dts, parts, strides, _ptr(mix), _ptr(out_weights), _ptr(read), _ptr(new), _ptr(w), _ptr(b), int(bool(centred)),
+                    float(eps), y.data_ptr(), _code(out_dtype), R, S, n, _stream())
+        return (streams if as_they_are and keep else new), y
 
     def gated_rms_norm(self, y, gate, weight, eps: float, groups: int, kind: str, out_dtype: torch.dtype) -> torch.Tensor:
         """`kind` "silu_before": u = y * silu(gate), out = u / rms(u) * weight with the root mean square taken over
@@ -947,6 +1064,7 @@ class HipBackend:
         rule "delta":  d = exp(-rate_h softplus(raw + base));  S <- diag(d) S;  u = sigmoid(beta) (v - S^T k);
                        S <- S + k u^T;  y = S^T q.
         rule "gated":  d = sigmoid(raw + base) ^ rate_h;  S <- diag(d) S + k v^T;  y = S^T q.
+        rule "delta_head": the delta rule with one decay per head: raw [T, H], base [H].
         q, k: row views [T, G * N] (heads share them by groups of H / G); v: [T, H * P]; raw: [T, H * N]; beta: [T, H];
         base, bonus: float32 [H * N]; rate: float32 [H]. `unit_eps`: q and k are made unit vectors per head first, x /
         sqrt(sum(x^2) + unit_eps); q is multiplied by q_scale. Everything but the rows read is float32. Returns float32
@@ -954,11 +1072,12 @@ class HipBackend:
         T, B = v.shape[0], state_slots.numel()
         dtype = v.dtype
         _check(rule in DECAY_RULES, f"decay_rows_recurrence: rule must be one of {sorted(DECAY_RULES)}")
-        for t, width in ((q, G * N), (k, G * N), (v, H * P), (raw, H * N)):
+        per_head = rule == "delta_head"
+        for t, width in ((q, G * N), (k, G * N), (v, H * P), (raw, H if per_head else H * N)):
             _check(t.dim() == 2 and t.shape == (T, width) and t.stride(1) == 1 and t.dtype == dtype, "decay_rows_recurrence: bad q, k, v or decay rows")
         _check(state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1 and state.shape[1] == H * N * P,
                "decay_rows_recurrence: state must be float32 [slots, H * N * P]")
-        for w, width in ((base, H * N), (bonus, H * N), (rate, H)):
+        for w, width in ((base, H if per_head else H * N), (bonus, H * N), (rate, H)):
             _check(w is None or (w.dtype == torch.float32 and w.numel() == width and w.is_contiguous()), "decay_rows_recurrence: constants float32")
         _check(base is not None and (bonus is not None if rule == "bonus" else (rate is not None and (beta is not None or rule == "gated"))),
                "decay_rows_recurrence: the rule's constants are missing")
@@ -995,7 +1114,7 @@ class HipBackend:
         ids = torch.empty((T, top), dtype=torch.int32, device=x.device)
         weights = torch.empty((T, top), dtype=torch.float32, device=x.device)
         logits = torch.empty((T, E), dtype=torch.float32, device=x.device)
-        core().call("me_moe_route", x.data_ptr(), x.stride(0), _code(x.dtype), router.data_ptr(), T, n, E, int(top), int(group_count),
+        core().call("me_moe_route", x.data_ptr(), x.stride(0), _code(x.dtype), router.data_ptr(), _ptr(rule.bias), T, n, E, int(top), int(group_count),
                     int(group_keep), logits.data_ptr(), ids.data_ptr(), weights.data_ptr(), 1, *rule.args(), _stream())
         return ids, weights
 
@@ -1018,7 +1137,7 @@ class HipBackend:
         ids = torch.empty((T, top), dtype=torch.int32, device=x.device)
         weights = torch.empty((T, top), dtype=torch.float32, device=x.device)
         logits = torch.empty((T, E), dtype=torch.float32, device=x.device)
-        core().call("me_moe_route", x.data_ptr(), x.stride(0), _code(x.dtype), router.data_ptr(), T, n, E, int(top), int(group_count),
+        core().call("me_moe_route", x.data_ptr(), x.stride(0), _code(x.dtype), router.data_ptr(), _ptr(rule.bias), T, n, E, int(top), int(group_count),
                     int(group_keep), logits.data_ptr(), ids.data_ptr(), weights.data_ptr(), 0, *rule.args(), _stream())
         return self.routed_experts(x, ids, weights, gate_up, down, choose_from=(logits, group_count, group_keep, rule), gated=gated)
 
@@ -1067,7 +1186,7 @@ class HipBackend:
 
     # -- attention over a latent that all heads share ------------------------------------------
     def latent_prepare(self, rows, q_off: int, kv_off: int | None, H: int, dn: int, dr: int, R: int, D: int, norm_weight, eps: float,
-                       table, positions, slots, k_cache, v_cache, page: int) -> torch.Tensor:
+                       table, positions, slots, k_cache, v_cache, page: int, query_latent: tuple | None = None):
         """From the rows of a layer's packed product ([T, ...]: H query heads of dn unrotated and dr rotating dimensions from
         column q_off; from column kv_off the latent's R rows and dr rows of a key part that all heads share): the RMS norm
         of the latent with `norm_weight` (float32 [R]), the rotation of the shared key part and of every head's rotating
@@ -1075,7 +1194,9 @@ class HipBackend:
         `slots`: k_cache [pages, 1, page, D] takes [latent | rotated part | zeros], v_cache [pages, 1, D, page] the latent.
         kv_off None: a layer that reads another layer's pages writes none. Returns the queries' frame [T, H * D] in the
         rows' dtype with slots R .. R + dr of every head filled (the rotated part; zeros behind it): slots 0 .. R wait for
-        the queries carried into the latent's space (`heads_linear`)."""
+        the queries carried into the latent's space (`heads_linear`). `query_latent`: (first column, norm weight float32 [RQ]) of
+        a latent that the queries pass: its RMS norm (the same eps) is formed in the same pass, and (the frame, the normed
+        latent [T, RQ]) comes back; H may then be 0 (the queries are not in these rows: no frame is filled)."""
         T = rows.shape[0]
         _check(rows.dim() == 2 and rows.stride(1) == 1 and q_off + H * (dn + dr) <= rows.shape[1], "latent_prepare: rows [T, n], unit inner stride")
         _check(dr % 2 == 0 and D >= R + dr and (dr == 0 or (table is not None and table.dtype == torch.float32 and table.is_contiguous()
@@ -1087,12 +1208,17 @@ class HipBackend:
                    and norm_weight.is_contiguous(), "latent_prepare: slots int32, norm weight float32 [rank]")
             _check(k_cache.shape[1:] == (1, page, D) and v_cache.shape[1:] == (1, D, page) and k_cache.dtype == rows.dtype
                    and v_cache.dtype == rows.dtype, "latent_prepare: cache layout mismatch")
+        cq_off, cq_w = query_latent if query_latent is not None else (0, None)
+        RQ = 0 if cq_w is None else cq_w.numel()
+        _check(cq_w is None or (cq_w.dtype == torch.float32 and cq_w.dim() == 1 and cq_w.is_contiguous() and cq_off + RQ <= rows.shape[1]),
+               "latent_prepare: the queries' latent needs a float32 norm weight")
+        cq = torch.empty((T, RQ), dtype=rows.dtype, device=rows.device) if cq_w is not None else None
         qa = torch.empty((T, H * D), dtype=rows.dtype, device=rows.device)
         core().call("me_latent_prepare", rows.data_ptr(), rows.stride(0), _code(rows.dtype), int(q_off), int(kv_off or 0), H, dn, dr, R, D,
                     _ptr(norm_weight) if write else None, float(eps), _ptr(table), 0 if table is None else table.shape[0],
                     positions.data_ptr(), slots.data_ptr() if write else None, qa.data_ptr(), qa.stride(0),
-                    k_cache.data_ptr() if write else None, v_cache.data_ptr() if write else None, int(page), T, _stream())
-        return qa
+                    k_cache.data_ptr() if write else None, v_cache.data_ptr() if write else None, int(page), int(cq_off), RQ, _ptr(cq_w), _ptr(cq), T, _stream())
+        return qa if cq is None else (qa, cq)
 
     def heads_linear(self, x, w, out) -> torch.Tensor:
         """out[t, h, :] = w[h] x[t, h, :]: a product per head. x: a view [T, H, K], w: [H, N, K] contiguous, out: a view [T, H, N],
@@ -1737,3 +1863,5 @@ def routed_experts(*a, **k): return backend().routed_experts(*a, **k)
 def route_and_run_experts(*a, **k): return backend().route_and_run_experts(*a, **k)
 def latent_prepare(*a, **k): return backend().latent_prepare(*a, **k)
 def heads_linear(*a, **k): return backend().heads_linear(*a, **k)
+def memory_readout(*a, **k): return backend().memory_readout(*a, **k)
+def stream_mix_norm(*a, **k): return backend().stream_mix_norm(*a, **k)

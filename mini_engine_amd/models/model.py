@@ -11,7 +11,7 @@ from dataclasses import dataclass, replace
 import torch
 
 from ..kernels import ops
-from ..parts.base import CacheNeed, LayerCall, Part, Settled, StateNeed
+from ..parts.base import CacheNeed, LayerCall, Part, Settled, StateNeed, StreamSum
 from ..parts.block import norm_of, settled
 
 
@@ -118,6 +118,10 @@ class DecoderModel(Part):
         """Final norm of (h + residual), then the rows that want logits, then the head: float32
         [len(rows), vocab] (reference models/qwen3.py:91,116-117; layers/embed_head.py:19-23).
         `out`: where the head puts them (`parts.Head.forward(x, out)`)."""
+        if isinstance(h, StreamSum):        # the last layer's streams: mixed, summed and normed at the wanted rows only
+            x = h.normed_rows(residual, self.final_norm, rows)
+            if x is not None:
+                return self.head.forward(x, out=out)
         h, residual = settled(h, residual)
         if isinstance(h, Settled):          # the last layer has added its output to the stream already: wanted rows first
             x, _ = self.final_norm.forward(ops.gather_rows(residual, rows), None)

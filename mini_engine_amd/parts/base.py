@@ -189,6 +189,8 @@ class Norm(Part):
         """
         raise NotImplementedError
 
+    # Optional: row_norm() -> (float32 weight, float32 bias or None, eps, whether the mean is taken off): what a kernel needs
+    # to run the norm inside its own pass over the rows (`ops.stream_mix_norm`).
     # Optional: linear_behind(x, residual, weight, out_dtype, gated=False) -> (forward(x, residual)[0] . weight^T,
     # new residual), norm and product as one kernel, or None where there is no such kernel for these shapes
     # (gated: weight is a packed gate/up weight and the product is silu(gate) * up).
@@ -254,6 +256,30 @@ class ScaledSum:
         """The new stream, float32 [T, n]."""
         from ..kernels import ops
         return ops.scaled_sum_norm(stream, self.terms, self.mult, None, None, 0.0, torch.float32)[0]
+
+
+class StreamSum:
+    """What a layer with several residual streams (hyper-connections) returns in place of its output, beside the streams
+    as its last sublayer found them: every stream takes a share of every stream and of that sublayer's output,
+        x'_t = sum_s mix[s, t] x_s + out[t] * sum(terms).
+    Whoever runs next forms it, a block of the same kind together with what its own sublayer reads and the norm in front of
+    that in one pass (`ops.stream_mix_norm`). The model's residual is the sum of the streams: `settle` (float32 [T, n]);
+    `normed_rows` is a norm of that sum for chosen rows only (the model's final norm)."""
+
+    def __init__(self, terms: list, mix: torch.Tensor, out: torch.Tensor):
+        self.terms, self.mix, self.out = list(terms), mix, out
+
+    def settle(self, streams: torch.Tensor) -> torch.Tensor:
+        from ..kernels import ops
+        return ops.stream_mix_norm(streams, self.out.numel(), self.terms, self.mix, self.out, None, None, torch.float32, keep=False)[1]
+
+    def normed_rows(self, streams: torch.Tensor, norm: "Norm", rows: torch.Tensor):
+        """The norm of the sum of the streams at `rows`, or None for a norm that no kernel can run inside."""
+        if not hasattr(norm, "row_norm"):
+            return None
+        from ..kernels import ops
+        return ops.stream_mix_norm(streams, self.out.numel(), self.terms, self.mix, self.out, None, norm.row_norm(), norm.out_dtype,
+                                   rows=rows, keep=False)[1]
 
 
 # Steps of up to this many tokens are chains of short launches: parts that have independent work then put it on further

@@ -1,8 +1,11 @@
 """How norm, mixer and feed-forward are arranged in a layer (reference models/qwen3.py:55-74)."""
 from __future__ import annotations
 
+import torch
+
 from ..kernels import ops
-from .base import FeedForward, Mixer, Norm, ParamSpec, Part, PendingNorm, ScaledSum, Settled, few_tokens, register_part, side_branch
+from .base import (FeedForward, Mixer, Norm, ParamSpec, Part, PendingNorm, ScaledSum, Settled, StreamSum, few_tokens, register_part,
+                   side_branch)
 
 
 def one_tensor(x):
@@ -17,8 +20,8 @@ def one_tensor(x):
 
 
 def settled(h, residual):
-    """(h, residual) with a `ScaledSum` in place of h turned into a `Settled` stream."""
-    if isinstance(h, ScaledSum):
+    """(h, residual) with a `ScaledSum` or `StreamSum` in place of h turned into a `Settled` stream."""
+    if isinstance(h, (ScaledSum, StreamSum)):
         return Settled(None), h.settle(residual)
     return h, residual
 
@@ -128,7 +131,6 @@ class OutputNormBlock(Part):
 
 
 def _ones(shape, generator, device):
-    import torch
     return 1.0 + 0.2 * (torch.rand(shape, generator=generator, dtype=torch.float32, device=device) - 0.5)
 
 
@@ -202,3 +204,79 @@ class ParallelBlock(Part):
         if b is not None:
             out += [(t, self.scale2 if self.layer_scale else None) for t in (b if isinstance(b, (tuple, list)) else (b,))]
         return ScaledSum(out, self.residual_mult), stream
+
+
+def _near_even(shape, generator, device):
+    """Shares of streams that start near the plain residual sum: 1/S each, give or take."""
+    return (1.0 + 0.2 * (torch.rand(shape, generator=generator, dtype=torch.float32, device=device) - 0.5)) / shape[0]
+
+
+def _near_identity(shape, generator, device):
+    return torch.eye(shape[0], device=device) + 0.1 * (torch.rand(shape, generator=generator, dtype=torch.float32, device=device) - 0.5)
+
+
+@register_part("block", "hyper_connected")
+class HyperConnectedBlock(Part):
+    """Instead of one residual stream `streams` of them, x_1 .. x_S, all equal at the model's start. Each sublayer has
+    learned shares: it reads u = sum_s read[s] x_s through its norm, and when it has run, all streams at once from the old
+    ones, x_t <- sum_s mix[s, t] x_s + out[t] * y (mix is indexed from, to). Without a feed-forward the layer is its
+    mixer's half. The streams are float32 [T, S, n]; behind the last layer the residual is their sum.
+
+    What a sublayer leaves is added by whoever runs next (`StreamSum`), in one kernel with what that one reads and its
+    norm (`ops.stream_mix_norm`): per sublayer one pass over the streams, and the terms of a sublayer's output (partial
+    sums of a split product, one partial sum per chosen expert, a shared expert's rows) are added up inside that pass. The
+    norms may be of any kind that has `row_norm`."""
+
+    def __init__(self, streams: int, norm1: Norm, mixer: Mixer, norm2: Norm | None = None, feed_forward: FeedForward | None = None):
+        super().__init__()
+        if streams < 1:
+            raise ValueError("a positive number of streams")
+        if (norm2 is None) != (feed_forward is None):
+            raise ValueError("a feed-forward and its norm come together")
+        for norm in (norm1, norm2):
+            if norm is not None and not hasattr(norm, "row_norm"):
+                raise ValueError("the norms run inside the block's own kernel and need `row_norm`")
+        self.streams = int(streams)
+        self.add_child("norm1", norm1)
+        self.add_child("mixer", mixer)
+        if feed_forward is not None:
+            self.add_child("norm2", norm2)
+            self.add_child("feed_forward", feed_forward)
+        else:
+            self.norm2 = self.feed_forward = None
+        for i in (1, 2) if feed_forward is not None else (1,):
+            self.add_param(f"read{i}", ParamSpec((streams,), init=_near_even, dtype="float32"))
+            self.add_param(f"out{i}", ParamSpec((streams,), init=_ones, dtype="float32"))
+            self.add_param(f"mix{i}", ParamSpec((streams, streams), init=_near_identity, dtype="float32"))
+
+    def cache_need(self):
+        return self.mixer.cache_need()
+
+    def state_need(self):
+        return self.mixer.state_need()
+
+    def _read(self, h, streams, read, norm):
+        """The streams with what waits in h added, and the normed rows that the next sublayer reads."""
+        terms, mix, out = (h.terms, h.mix, h.out) if isinstance(h, StreamSum) else ([], None, None)
+        new, x = ops.stream_mix_norm(streams, self.streams, terms, mix, out, read, norm.row_norm(), norm.out_dtype,
+                                     keep=streams.dim() == 3 or bool(terms))
+        return (streams if new is None else new), x
+
+    def forward(self, h, residual, step, cache, state):
+        if isinstance(h, StreamSum):
+            streams = residual
+        elif residual is None:               # the first layer: the embedding's rows are every stream
+            streams, h = h, None
+        else:                                # behind a layer of another kind: its stream, with what waits to be added, is every stream
+            h, residual = settled(h, residual)
+            streams, h = (residual if isinstance(h, Settled) else residual + one_tensor(h)), None
+        streams, x = self._read(h, streams, self.read1, self.norm1)
+        h = StreamSum(_terms(self.mixer.forward(x, step, cache, state)), self.mix1, self.out1)
+        if self.feed_forward is not None:
+            streams, x = self._read(h, streams, self.read2, self.norm2)
+            h = StreamSum(_terms(self.feed_forward.forward(x)), self.mix2, self.out2)
+        return h, streams
+
+
+def _terms(y) -> list:
+    return list(y) if isinstance(y, (tuple, list)) else [y]

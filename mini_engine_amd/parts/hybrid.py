@@ -169,25 +169,47 @@ class GatedDelta(Mixer):
         S <- diag(d) S;   u = beta (v - S^T k);   S <- S + k u^T;   y = S^T q.
     Every head's y is divided by its root mean square, multiplied by a weight shared by the heads and by
     sigmoid(W_g2 (W_g1 x)), and projected. A request's state row holds the heads' matrices and, behind them, the
-    convolutions' last taps - 1 inputs per channel."""
+    convolutions' last taps - 1 inputs per channel.
+
+    `decay_rank=None`: one decay per head instead, d = exp(-exp(A_log_h) softplus(W_a x + dt_bias_h)) with W_a [heads, hidden]
+    (rows of the packed product). `gate_rank=None`: the gate is one product W_g x (rows of the packed product too).
+    `gate_activation`: "sigmoid" or "silu"."""
+
+    takes_pending_norm = True      # x goes to the packed product and nowhere else
 
     def __init__(self, hidden_size: int, num_heads: int, key_heads: int, key_dim: int, value_dim: int, taps: int,
-                 decay_rank: int, gate_rank: int, norm_eps: float, unit_eps: float = 1e-6):
+                 decay_rank: int | None, gate_rank: int | None, norm_eps: float, unit_eps: float = 1e-6, gate_activation: str = "sigmoid"):
         super().__init__()
+        if gate_activation not in ("sigmoid", "silu"):
+            raise ValueError("the gate passes 'sigmoid' or 'silu'")
+        self.gate_kind = gate_activation + "_behind"
         if num_heads % key_heads or taps < 1:
             raise ValueError("heads must be a multiple of the key heads, taps positive")
         self.hidden_size, self.num_heads, self.key_heads = hidden_size, num_heads, key_heads
         self.key_dim, self.value_dim, self.taps = key_dim, value_dim, taps
         self.norm_eps, self.unit_eps = float(norm_eps), float(unit_eps)
-        self.qk, self.inner, self.decays = key_heads * key_dim, num_heads * value_dim, num_heads * key_dim
+        self.qk, self.inner = key_heads * key_dim, num_heads * value_dim
+        self.decays = num_heads * key_dim if decay_rank is not None else num_heads
         self.channels = 2 * self.qk + self.inner
-        # one product for everything that reads x directly: q | k | v | beta | a1 | g1
-        self.add_child("in_proj", Linear(hidden_size, self.channels + num_heads + decay_rank + gate_rank,
-                                         parts={"q": self.qk, "k": self.qk, "v": self.inner, "b": num_heads, "a1": decay_rank, "g1": gate_rank}))
+        # one product for everything that reads x directly: q | k | v | (g) | beta | a1 or a | (g1)
+        blocks = {"q": self.qk, "k": self.qk, "v": self.inner}
+        if gate_rank is None:
+            blocks["g"] = self.inner
+        blocks["b"] = num_heads
+        blocks["a" if decay_rank is None else "a1"] = num_heads if decay_rank is None else decay_rank
+        if gate_rank is not None:
+            blocks["g1"] = gate_rank
+        self.block_starts, at = {}, 0                       # block name -> its first row
+        for name, size in blocks.items():
+            self.block_starts[name] = at
+            at += size
+        self.add_child("in_proj", Linear(hidden_size, at, parts=blocks))
         self.decay_rank, self.gate_rank = decay_rank, gate_rank
         self.add_param("conv_weight", ParamSpec((self.channels, taps), init=_taps, dtype="float32"))
-        self.add_child("a2", Linear(decay_rank, self.decays))
-        self.add_child("g2", Linear(gate_rank, self.inner))
+        if decay_rank is not None:
+            self.add_child("a2", Linear(decay_rank, self.decays))
+        if gate_rank is not None:
+            self.add_child("g2", Linear(gate_rank, self.inner))
         self.add_param("dt_bias", ParamSpec((self.decays,), init=_step_bias, dtype="float32"))
         self.add_param("A_log", ParamSpec((num_heads,), init=_log_rates, dtype="float32"))
         self.add_param("norm_weight", ParamSpec((value_dim,), init="norm", dtype="float32"))
@@ -207,18 +229,18 @@ class GatedDelta(Mixer):
 
     def forward(self, x, step, cache, state):
         H, G, N, P = self.num_heads, self.key_heads, self.key_dim, self.value_dim
-        rows = self.in_proj.forward(x)                                # [T, q | k | v | b | a1 | g1 (| padding)]
-        C = self.channels
+        rows = self.in_proj.forward(x)                                # [T, q | k | v | ... (| padding)]
+        C, at = self.channels, self.block_starts
         qkv = ops.causal_conv(rows[:, :C], self.conv_weight, None, state[:, self.matrix_floats:], step.state_slots,
                               step.cu_seqlens, step.q_lens)
-        at = C + H
-        raw = self.a2.forward(_rows(rows, at, self.decay_rank))
-        gate = self.g2.forward(_rows(rows, at + self.decay_rank, self.gate_rank))
+        raw = rows[:, at["a"]: at["a"] + H] if self.decay_rank is None else self.a2.forward(_rows(rows, at["a1"], self.decay_rank))
+        gate = rows[:, at["g"]: at["g"] + self.inner] if self.gate_rank is None else self.g2.forward(_rows(rows, at["g1"], self.gate_rank))
         y = ops.decay_rows_recurrence(qkv[:, : self.qk], qkv[:, self.qk: 2 * self.qk], qkv[:, 2 * self.qk:], raw,
                                       state[:, : self.matrix_floats], step.state_slots, step.cu_seqlens, step.q_lens, H, G, N, P,
-                                      "delta", base=self.dt_bias, rate=self.rate, beta=rows[:, C: C + H],
+                                      "delta" if self.decay_rank is not None else "delta_head", base=self.dt_bias, rate=self.rate,
+                                      beta=rows[:, at["b"]: at["b"] + H],
                                       unit_eps=self.unit_eps, q_scale=N ** -0.5)
-        o = ops.gated_rms_norm(y, gate, self.wide_norm, self.norm_eps, H, "sigmoid_behind", gate.dtype)
+        o = ops.gated_rms_norm(y, gate, self.wide_norm, self.norm_eps, H, self.gate_kind, gate.dtype)
         return self.o.forward(o, allow_partials=True)
 
 

@@ -22,6 +22,10 @@ class LatentAttention(Mixer):
     single tokens alike), and W_uv[h] carries each head's result out of the latent's space again. `own_kv=False`: a layer
     call that reads the pages of an earlier latent layer with its own queries and W_uk, W_uv; it has no W_dkv.
 
+    `query_rank`: the queries pass a latent of their own, q = W_uq (norm(W_dq x)) (RMS norm with a weight; W_dq's rows take W_q's
+    place in the packed product, its norm runs in the kernel that norms the cached latent). `sinks`: a learned number per
+    head whose exponential joins the softmax's denominator without a key or a value.
+
     `position`: a rotary encoding over `rot_dim` dimensions in adjacent pairs (its table is read as it stands; any scaling
     of the positions lives there). q, the latent's rows and the gate are one packed product."""
 
@@ -29,7 +33,7 @@ class LatentAttention(Mixer):
 
     def __init__(self, hidden_size: int, num_heads: int, nope_dim: int, rot_dim: int, value_dim: int, rank: int, scale: float,
                  norm_eps: float, position: PositionEncoding | None, window: int | None = None, own_kv: bool = True,
-                 output_gate: bool = False):
+                 output_gate: bool = False, query_rank: int | None = None, sinks: bool = False):
         super().__init__()
         if rot_dim % 2 or (rot_dim and position is None):
             raise ValueError("the rotating part has an even size and needs a position encoding")
@@ -40,18 +44,27 @@ class LatentAttention(Mixer):
         self.window, self.own_kv, self.output_gate = window, bool(own_kv), bool(output_gate)
         self.head_dim = -(-(rank + rot_dim) // 16) * 16          # the attention kernels' head size: whole steps of 16
         H = num_heads
-        blocks = {"q": H * (nope_dim + rot_dim)}
+        self.query_rank = None if query_rank is None else int(query_rank)
+        blocks = {"q": H * (nope_dim + rot_dim)} if query_rank is None else {"dq": self.query_rank}
+        first = sum(blocks.values())
         if own_kv:
             blocks["dkv"] = rank + rot_dim
         if output_gate:
             blocks["g"] = H * value_dim
-        self.kv_at = blocks["q"] if own_kv else None
-        self.gate_at = blocks["q"] + (blocks["dkv"] if own_kv else 0)
+        self.kv_at = first if own_kv else None
+        self.gate_at = first + (blocks["dkv"] if own_kv else 0)
         self.add_child("in_proj", Linear(hidden_size, sum(blocks.values()), parts=blocks))
         if own_kv:
             self.add_param("latent_norm_weight", ParamSpec((rank,), init="norm", dtype="float32"))
         else:
             self.latent_norm_weight = None
+        if query_rank is not None:
+            self.add_param("query_norm_weight", ParamSpec((self.query_rank,), init="norm", dtype="float32"))
+            self.add_child("uq", Linear(self.query_rank, H * (nope_dim + rot_dim)))
+        if sinks:
+            self.add_param("sinks", ParamSpec((H,), init="matrix", dtype="float32"))
+        else:
+            self.sinks = None
         self.add_param("uk", ParamSpec((H * nope_dim, rank), init="matrix", dtype="compute"))
         self.add_param("uv", ParamSpec((H * value_dim, rank), init="matrix", dtype="compute"))
         self.add_child("o", Linear(H * value_dim, hidden_size))
@@ -71,6 +84,9 @@ class LatentAttention(Mixer):
     def finalize(self, device, dtype, max_positions):
         # W_uk[h]^T, [heads, rank, nope_dim]: the matrix that carries a head's unrotated query part into the latent's space
         self._uk_t = self.uk.view(self.num_heads, self.nope_dim, self.rank).transpose(1, 2).contiguous()
+        w = self.in_proj.weight
+        if w.shape[0] % 8:                  # the packed rows in whole steps of 8: views of them keep 16-byte row strides
+            self.in_proj.weight = torch.cat((w, w.new_zeros(8 - w.shape[0] % 8, w.shape[1])), 0).contiguous()
 
     def forward(self, x, step, cache, state):
         H, dn, dr, R, D, nv = self.num_heads, self.nope_dim, self.rot_dim, self.rank, self.head_dim, self.value_dim
@@ -79,14 +95,24 @@ class LatentAttention(Mixer):
         T = rows.shape[0]
         write = self.own_kv and cache.write
         table = self.position.rotary_table() if self.position is not None else None
-        qa = ops.latent_prepare(rows, 0, self.kv_at if write else None, H, dn, dr, R, D, self.latent_norm_weight, self.norm_eps,
-                                table, step.positions, grp.slot_mapping, cache.k, cache.v, cache.page_size)
+        kv_at = self.kv_at if write else None
+        tail = (self.norm_eps, table, step.positions, grp.slot_mapping, cache.k, cache.v, cache.page_size)
+        if self.query_rank is None:
+            queries = rows
+            qa = ops.latent_prepare(rows, 0, kv_at, H, dn, dr, R, D, self.latent_norm_weight, *tail)
+        else:
+            # both latents' norms and the page writes in one kernel; the queries come out of their latent behind it
+            qa, cq = ops.latent_prepare(rows, 0, kv_at, 0 if dr else H, 0, dr, R, D, self.latent_norm_weight, *tail,
+                                        query_latent=(0, self.query_norm_weight))
+            queries = self.uq.forward(cq)
+            if dr:
+                qa = ops.latent_prepare(queries, 0, None, H, dn, dr, R, D, None, *tail)
         q3 = qa.view(T, H, D)
-        ops.heads_linear(rows[:, : H * (dn + dr)].view(T, H, dn + dr)[:, :, :dn], self._uk_t, q3[:, :, :R])
+        ops.heads_linear(queries[:, : H * (dn + dr)].view(T, H, dn + dr)[:, :, :dn], self._uk_t, q3[:, :, :R])
         o = ops.paged_attention(qa, cache.k, cache.v, cache.page_size, grp.block_tables, step.context_lens, step.seq_of_token,
                                 step.positions, step.prefill_cu, step.num_decodes, step.max_decode_context, self.scale,
                                 self.window, H, 1, D, max_prefill_context=step.max_prefill_context,
-                                even_contexts=step.decode_contexts_even)
+                                even_contexts=step.decode_contexts_even, sinks=self.sinks)
         heads = torch.empty((T, H * nv), dtype=rows.dtype, device=rows.device)
         ops.heads_linear(o.view(T, H, D)[:, :, :R], self.uv.view(H, nv, R), heads.view(T, H, nv))
         if self.output_gate:

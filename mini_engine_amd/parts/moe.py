@@ -12,7 +12,8 @@ class RoutedExperts(FeedForward):
     `gated=False` W_down[e] relu(W_up[e] x)^2.
 
     The router is float32. `scoring` "softmax": scores = softmax(W_router x) over all experts; "sigmoid": a sigmoid
-    each. `correction`: a stored number per expert joins the scores for the choice only (the weights use the scores
+    each; "chosen": the choice goes by the logits themselves and the weights are their softmax over the chosen experts alone.
+    `router_bias`: a stored number per expert is part of the logits. `correction`: a stored number per expert joins the scores for the choice only (the weights use the scores
     without it). `group_count` > 1: the experts form that many equal groups of neighbours, a group scores as the sum of
     its `group_top` largest choice scores (1: as its best expert), and only the experts of the `group_keep` best groups
     can be chosen. The `top` largest choice scores are chosen; their weights are the scores, divided by their sum
@@ -31,7 +32,7 @@ class RoutedExperts(FeedForward):
     def __init__(self, hidden_size: int, intermediate_size: int, num_experts: int, top: int, group_count: int = 1,
                  group_keep: int = 1, shared: FeedForward | None = None, gated: bool = True, scoring: str = "softmax",
                  correction: bool = False, group_top: int = 1, normalise: bool = True, route_scale: float = 1.0,
-                 sum_outputs: bool = False):
+                 sum_outputs: bool = False, router_bias: bool = False):
         super().__init__()
         if not 1 <= top <= num_experts:
             raise ValueError(f"top {top} of {num_experts} experts")
@@ -39,8 +40,8 @@ class RoutedExperts(FeedForward):
             raise ValueError(f"{num_experts} experts do not form {group_count} equal groups of which {group_keep} are kept")
         if group_keep * (num_experts // group_count) < top:
             raise ValueError("the kept groups hold fewer experts than a token uses")
-        if scoring not in ("softmax", "sigmoid") or group_top < 1:
-            raise ValueError("scoring is 'softmax' or 'sigmoid', group_top positive")
+        if scoring not in ops.RouteRule.SCORINGS or group_top < 1:
+            raise ValueError(f"scoring is one of {sorted(ops.RouteRule.SCORINGS)}, group_top positive")
         self.hidden_size, self.intermediate_size = hidden_size, intermediate_size
         self.num_experts, self.top, self.group_count, self.group_keep = num_experts, top, group_count, group_keep
         self.gated, self.scoring, self.group_top = bool(gated), scoring, int(group_top)
@@ -49,6 +50,10 @@ class RoutedExperts(FeedForward):
         self.add_param("router", ParamSpec((num_experts, hidden_size), init="matrix", dtype="float32"))
         self.add_param("gate_up", ParamSpec((num_experts * rows, hidden_size), init="matrix", dtype="compute"))
         self.add_param("down", ParamSpec((num_experts * hidden_size, intermediate_size), init="matrix", dtype="compute"))
+        if router_bias:
+            self.add_param("router_bias", ParamSpec((num_experts,), init="matrix", dtype="float32"))
+        else:
+            self.router_bias = None
         if correction:
             self.add_param("correction", ParamSpec((num_experts,), init="matrix", dtype="float32"))
         else:
@@ -65,7 +70,8 @@ class RoutedExperts(FeedForward):
 
     def rule(self) -> "ops.RouteRule":
         if self._rule is None:
-            self._rule = ops.RouteRule(self.scoring, self.correction, self.group_top, self.normalise, self.route_scale)
+            self._rule = ops.RouteRule(self.scoring, self.correction, self.group_top, self.normalise, self.route_scale,
+                                       bias=self.router_bias)
         return self._rule
 
     def forward(self, x):

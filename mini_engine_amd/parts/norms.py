@@ -1,4 +1,4 @@
-"""RMSNorm, fused with the residual sum (reference layers/layernorm.py:5-24)."""
+"""RMSNorm, fused with the residual sum (reference layers/layernorm.py:5-24), and layer norm."""
 from __future__ import annotations
 
 import torch
@@ -52,6 +52,9 @@ class RMSNorm(Norm):
         scale, bias or None); sum, norm and residual sum are one kernel (`ops.weighted_sum`)."""
         return ops.weighted_sum(terms.terms, self.weight, self.eps, stream, self.out_dtype)
 
+    def row_norm(self):
+        return self.weight, None, self.eps, False
+
     def forward(self, x, residual, want_residual: bool = True):
         return ops.rms_norm(x, self.weight, self.eps, residual, self.out_dtype, want_residual)
 
@@ -59,3 +62,32 @@ class RMSNorm(Norm):
         if weight.dtype != self.out_dtype or not ops.norm_linear_fuses(x, weight):
             return None
         return ops.norm_linear(x, residual, self.weight, self.eps, weight, out_dtype, gated=gated)
+
+
+@register_part("norm", "layer")
+class LayerNorm(Norm):
+    """y = weight * (r - mean(r)) / sqrt(mean((r - mean(r))^2) + eps) + bias, r = x + residual, all in float32."""
+
+    accepts_partials = True
+
+    def __init__(self, size: int, eps: float):
+        super().__init__()
+        self.size, self.eps = size, eps
+        self.add_param("weight", ParamSpec((size,), init="norm", dtype="float32"))
+        self.add_param("bias", ParamSpec((size,), init=_around_zero, dtype="float32"))
+        self.out_dtype = torch.float32
+
+    def finalize(self, device, dtype, max_positions):
+        self.out_dtype = dtype
+
+    def row_norm(self):
+        return self.weight, self.bias, self.eps, True
+
+    def forward(self, x, residual):
+        if residual is None:
+            x = x.sum(0) if x.dim() == 3 else x
+            stream, terms = x, []
+        else:
+            stream, terms = residual.view(residual.shape[0], 1, -1), [x]
+        new, y = ops.stream_mix_norm(stream, 1, terms, None, None, None, self.row_norm(), self.out_dtype)
+        return y, new.view(new.shape[0], -1)

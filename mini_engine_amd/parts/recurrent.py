@@ -1,10 +1,11 @@
 """Mixers that keep a matrix of fixed size per request and head instead of keys and values per token.
 
-Both run on one recurrence kernel (`ops.linear_recurrence`): per head a state S [N, P] in float32,
+All run on one recurrence kernel (`ops.linear_recurrence`): per head a state S [N, P] in float32,
     S_t = a_t * S_(t-1) + b_t * k_t v_t^T,      y_t = S_t^T q_t (+ skip * v_t),
 with k_t, q_t of size N (shared by the heads of a group) and v_t of size P. What differs is where a_t and b_t
 come from: one fixed decay per head and b = 1 (`LinearAttention`), or a step size per token and head that a
-projection gives, a = exp(-rate * dt), b = dt (`SelectiveStateSpace`). The state lives in a request's state
+projection gives, a = exp(-rate * dt), b = dt (`SelectiveStateSpace`); or exponential input and forget gates under a
+running maximum, with the summed keys beside the state as what the output is divided by (`MatrixMemory`). The state lives in a request's state
 slot; the step function zeroes it when the request's tokens start at position 0, and a step carries it on from
 wherever the step before left it, so a prompt may be cut anywhere.
 """
@@ -120,4 +121,58 @@ class SelectiveStateSpace(Mixer):
                                   dt=rows[:, self.inner + self.channels:], dt_bias=self.dt_bias, rate=self.rate, skip=self.D)
         o = ops.gated_rms_norm(y, rows[:, : self.inner], self.norm_weight, self.norm_eps, self.norm_groups, "silu_before",
                                rows.dtype)
+        return self.o.forward(o, allow_partials=True)
+
+
+def _forget_bias(shape, generator, device):
+    """Biases of the forget gate spread over 3..6: per-step decays between 0.95 and 0.998."""
+    return 3.0 + 3.0 * torch.rand(shape, generator=generator, dtype=torch.float32, device=device)
+
+
+@register_part("mixer", "mlstm")
+class MatrixMemory(Mixer):
+    """The matrix memory of xLSTM: q = W_q x * key_dim^(-1/2) and k = W_k x ([heads, key_dim]), v = W_v x ([heads,
+    value_dim]); per head a logarithmic input gate i = c tanh((W_i x + b_i) / c) and a logarithmic forget gate f = log
+    sigmoid(c tanh((W_f x + b_f) / c)) with a cap c. With a running maximum m (0 before the first token)
+        m' = max(f + m, i),  S <- exp(f + m - m') S + exp(i - m') k v^T,  n the same with k alone,
+        o = S^T q / (max(|n . q|, exp(-m')) + 1e-6).
+    Every head's o is divided by its root mean square; the heads side by side are multiplied by a weight and by sigmoid(W_g
+    x) and projected. Everything that reads x is one packed product. A request's state row holds the heads' matrices, the
+    summed keys behind them, and the maxima, all float32."""
+
+    takes_pending_norm = True      # x goes to the packed product and nowhere else
+
+    def __init__(self, hidden_size: int, num_heads: int, key_dim: int, value_dim: int, gate_cap: float, norm_eps: float):
+        super().__init__()
+        if not gate_cap > 0:
+            raise ValueError("the gates' cap must be positive")
+        self.hidden_size, self.num_heads, self.key_dim, self.value_dim = hidden_size, num_heads, key_dim, value_dim
+        self.gate_cap, self.norm_eps = float(gate_cap), float(norm_eps)
+        self.qk, self.inner = num_heads * key_dim, num_heads * value_dim
+        self.add_child("in_proj", Linear(hidden_size, 2 * self.qk + 2 * self.inner + 2 * num_heads,
+                                         parts={"q": self.qk, "k": self.qk, "v": self.inner, "g": self.inner, "i": num_heads, "f": num_heads}))
+        self.add_param("i_bias", ParamSpec((num_heads,), init="matrix", dtype="float32"))
+        self.add_param("f_bias", ParamSpec((num_heads,), init=_forget_bias, dtype="float32"))
+        self.add_param("norm_weight", ParamSpec((self.inner,), init="norm", dtype="float32"))
+        self.add_child("o", Linear(self.inner, hidden_size))
+        self.matrix_floats = num_heads * key_dim * value_dim
+
+    def state_need(self):
+        # rows in whole steps of 4 numbers: every request's state starts at 16 bytes
+        return StateNeed((-(-(self.matrix_floats + self.qk + self.num_heads) // 4) * 4,), "float32")
+
+    def finalize(self, device, dtype, max_positions):
+        w = self.in_proj.weight
+        if w.shape[0] % 8:                  # the packed rows in whole steps of 8: views of them keep 16-byte row strides
+            self.in_proj.weight = torch.cat((w, w.new_zeros(8 - w.shape[0] % 8, w.shape[1])), 0).contiguous()
+
+    def forward(self, x, step, cache, state):
+        H, N, P, qk, inner, M = self.num_heads, self.key_dim, self.value_dim, self.qk, self.inner, self.matrix_floats
+        rows = self.in_proj.forward(x)                                # [T, q | k | v | g | i | f (| padding)]
+        at = 2 * qk + 2 * inner
+        gates = ops.SoftGates(rows[:, at: at + H], rows[:, at + H: at + 2 * H], self.i_bias, self.f_bias, self.gate_cap,
+                              state[:, M + qk: M + qk + H], step.state_slots)
+        reads = ops.linear_recurrence(rows[:, :qk], rows[:, qk: 2 * qk], rows[:, 2 * qk: 2 * qk + inner], state[:, :M], step.state_slots,
+                                      step.cu_seqlens, step.q_lens, H, H, N, P, gates=gates, key_state=state[:, M: M + qk])
+        o = ops.memory_readout(reads, rows[:, 2 * qk + inner: at], self.norm_weight, self.norm_eps, H, N ** -0.5, rows.dtype)
         return self.o.forward(o, allow_partials=True)

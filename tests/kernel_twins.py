@@ -12,6 +12,8 @@ from __future__ import annotations
 
 import torch
 
+from mini_engine_amd.kernels import ops
+
 
 def gather_rows(src, idx, scale=None):
     if scale is not None:
@@ -223,21 +225,33 @@ def softplus(x):
 
 
 def linear_recurrence(q, k, v, state, state_slots, cu_seqlens, q_lens, H, G, N, P, decay=None, dt=None, dt_bias=None,
-                      rate=None, skip=None, silu=False):
+                      rate=None, skip=None, silu=False, gates=None, key_state=None):
     """S_t = a S_(t-1) + b k_t v_t^T, y_t = S_t^T q_t (+ skip v_t), float32, token by token. q, k [T, G * N], v [T, H * P];
-    state [slots, H * N * P]. a, b: decay[h], 1; or exp(-rate[h] dt), dt with dt = softplus(dt[t, h] + dt_bias[h])."""
+    state [slots, H * N * P]. a, b: decay[h], 1; or exp(-rate[h] dt), dt with dt = softplus(dt[t, h] + dt_bias[h]);
+    or with `gates` exp(f + m - m'), exp(i - m'), m' = max(f + m, i), beside n_t = a n_(t-1) + b k_t in `key_state`."""
     T = v.shape[0]
+    if gates is not None:
+        dots, floors = (torch.zeros((T, H), dtype=torch.float32, device=v.device) for _ in range(2))
+        bent = lambda z, bias: gates.cap * torch.tanh((z.float() + bias) / gates.cap)
     y = torch.zeros((T, H * P), dtype=torch.float32, device=v.device)
     cu, slots = cu_seqlens.tolist(), state_slots.tolist()
     per = H // G
     for b in range(len(cu) - 1):
         S = state[slots[b]].view(H, N, P).clone()
+        if gates is not None:
+            n, m = key_state[slots[b]].view(H, N).clone(), gates.m[slots[b]].clone()
         for t in range(cu[b], cu[b + 1]):
             kt, qt, vt = k[t].float().view(G, N), q[t].float().view(G, N), v[t].float().view(H, P)
             if silu:
                 kt, qt, vt = (z * torch.sigmoid(z) for z in (kt, qt, vt))
             if decay is not None:
                 a, bb = decay.float(), torch.ones(H)
+            elif gates is not None:
+                i, f = bent(gates.i[t], gates.bias_i), -softplus(-bent(gates.f[t], gates.bias_f))
+                now = torch.maximum(f + m, i)
+                a, bb, m = torch.exp(f + m - now), torch.exp(i - now), now
+                n = a[:, None] * n + bb[:, None] * kt
+                dots[t], floors[t] = (n * qt).sum(-1), torch.exp(-m)
             else:
                 step = softplus(dt[t].float() + dt_bias)
                 a, bb = torch.exp(-rate * step), step
@@ -248,7 +262,39 @@ def linear_recurrence(q, k, v, state, state_slots, cu_seqlens, q_lens, H, G, N, 
                 out = out + skip[:, None] * vt
             y[t] = out.reshape(-1)
         state[slots[b]] = S.reshape(-1)
-    return y
+        if gates is not None:
+            key_state[slots[b]], gates.m[slots[b]] = n.reshape(-1), m
+    return y if gates is None else ops.MemoryReads(y, dots, floors, gates)
+
+
+def memory_readout(reads, gate, weight, eps, heads, q_scale, out_dtype):
+    T, n = reads.y.shape
+    below = torch.maximum((q_scale * reads.dot).abs(), reads.floor) + 1e-6
+    o = q_scale * reads.y.view(T, heads, -1) / below[:, :, None]
+    o = (o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps)).view(T, n)
+    return (o * weight * torch.sigmoid(gate.float())).to(out_dtype)
+
+
+def stream_mix_norm(streams, count, terms, mix, out_weights, read, norm, out_dtype, rows=None, keep=True):
+    """Streams [T, S, n] (or rows that all share): mixed, the terms added, read, normed; all in float32."""
+    x = streams.float()
+    if x.dim() == 2:
+        x = x[:, None, :].expand(-1, count, -1)
+    y = sum((t.float().sum(0) if t.dim() == 3 else t.float()) for t in terms) if terms else None
+    if mix is not None:
+        x = torch.einsum("st,bsn->btn", mix, x) + (0 if y is None else out_weights[None, :, None] * y[:, None, :])
+    elif y is not None:
+        x = x + y[:, None, :]
+    if rows is not None:
+        x = x[rows.long()]
+    u = x.sum(1) if read is None else torch.einsum("s,bsn->bn", read, x)
+    if norm is not None:
+        w, b, eps, centred = norm
+        if centred:
+            u = u - u.mean(-1, keepdim=True)
+        u = u / torch.sqrt(u.pow(2).mean(-1, keepdim=True) + eps) * w
+        u = u if b is None else u + b
+    return (x.contiguous() if keep else None), u.to(out_dtype)
 
 
 def gated_rms_norm(y, gate, weight, eps, groups, kind, out_dtype):
@@ -321,7 +367,9 @@ def decay_rows_recurrence(q, k, v, raw, state, state_slots, cu_seqlens, q_lens, 
                           beta=None, unit_eps=None, q_scale=1.0):
     """Token by token, float32. rule "bonus": y = (S + diag(bonus) k v^T)^T q, S <- diag(d) S + k v^T with d =
     exp(-exp(raw + base)); rule "delta": S <- diag(d) S with d = exp(-rate softplus(raw + base)), u = sigmoid(beta) (v -
-    S^T k), S <- S + k u^T, y = S^T q."""
+    S^T k), S <- S + k u^T, y = S^T q; rule "delta_head": the same with raw [T, H] and base [H], one decay per head."""
+    if rule == "delta_head":
+        raw, base, rule = raw.repeat_interleave(N, 1), base.repeat_interleave(N), "delta"
     T = v.shape[0]
     y = torch.zeros((T, H * P), dtype=torch.float32, device=v.device)
     cu, slots = cu_seqlens.tolist(), state_slots.tolist()
@@ -405,6 +453,11 @@ def qkv_prepare_store(rows, bias, q_weight, k_weight, eps, nq, nk, temperature, 
 
 def moe_route(x, router, top, group_count=1, group_keep=1, rule=None):
     z = x.float() @ router.float().t()
+    if rule is not None and rule.bias is not None:
+        z = z + rule.bias
+    if rule is not None and rule.scoring == "chosen":
+        values, ids = torch.sort(z, dim=-1, descending=True, stable=True)
+        return ids[:, :top].to(torch.int32), (torch.softmax(values[:, :top], -1) * rule.scale).float()
     sigmoid = rule is not None and rule.scoring == "sigmoid"
     s = torch.sigmoid(z) if sigmoid else torch.softmax(z, dim=-1)
     T, E = s.shape
@@ -449,7 +502,8 @@ def routed_experts(x, ids, weights, gate_up, down, force_simple=False, tile_rows
     return out
 
 
-def latent_prepare(rows, q_off, kv_off, H, dn, dr, R, D, norm_weight, eps, table, positions, slots, k_cache, v_cache, page):
+def latent_prepare(rows, q_off, kv_off, H, dn, dr, R, D, norm_weight, eps, table, positions, slots, k_cache, v_cache, page,
+                   query_latent=None):
     T = rows.shape[0]
     qa = torch.zeros((T, H, D), dtype=rows.dtype, device=rows.device)
     cs = table[positions.long()] if dr else None                      # [T, dr / 2, 2]
@@ -464,7 +518,7 @@ def latent_prepare(rows, q_off, kv_off, H, dn, dr, R, D, norm_weight, eps, table
         return out
 
     q = rows[:, q_off:q_off + H * (dn + dr)].reshape(T, H, dn + dr)
-    if dr:
+    if dr and H:
         qa[:, :, R:R + dr] = turn(q[:, :, dn:]).to(rows.dtype)
     if kv_off is not None:
         kv = rows[:, kv_off:kv_off + R + dr].float()
@@ -476,6 +530,10 @@ def latent_prepare(rows, q_off, kv_off, H, dn, dr, R, D, norm_weight, eps, table
         val = torch.zeros((T, 1, D), dtype=torch.float32, device=rows.device)
         val[:, 0, :R] = c
         write_pages(key.to(rows.dtype), val.to(rows.dtype), slots, k_cache, v_cache, page)
+    if query_latent is not None:
+        at, w = query_latent
+        c = rows[:, at:at + w.numel()].float()
+        return qa.reshape(T, H * D), (c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + eps) * w).to(rows.dtype)
     return qa.view(T, H * D)
 
 
@@ -571,3 +629,5 @@ class PlainBackend:
     route_and_run_experts = staticmethod(route_and_run_experts)
     latent_prepare = staticmethod(latent_prepare)
     heads_linear = staticmethod(heads_linear)
+    memory_readout = staticmethod(memory_readout)
+    stream_mix_norm = staticmethod(stream_mix_norm)
