@@ -37,7 +37,7 @@ import time
 HBM_PEAK = 8.0e12
 FLOP_PEAK = {"bfloat16": 2.5e15, "float32": 157.3e12}
 
-from mini_engine_amd.config.sizes import SIZES, model_config, named_config   # noqa: E402  (the named layer sizes)
+from mini_engine_amd.config.sizes import DESIGNS, SIZES, model_config, named_config   # noqa: E402  (the named layer sizes)
 
 
 def log(msg: str) -> None:
@@ -472,9 +472,9 @@ def main(argv=None) -> int:
     ap.add_argument("--no-graphs", action="store_true", help="launch decode kernels one by one instead of replaying HIP graphs")
     ap.add_argument("--no-run-ahead", action="store_true",
                     help="fetch every decode step's tokens before the next step is launched")
-    ap.add_argument("--beside", default="qwen3", choices=["qwen3", "sigosun", "negosun", "tavevik", "goluzen"],
+    ap.add_argument("--beside", default="qwen3", choices=["qwen3", *DESIGNS],
                     help="with --design: the model the design is measured beside, at the same width, depth and vocabulary")
-    ap.add_argument("--design", default=None, choices=["sigosun", "negosun", "tavevik", "goluzen"],
+    ap.add_argument("--design", default=None, choices=list(DESIGNS),
                     help="instead of the default workload: prefill and decode throughput of this design at the layer sizes "
                          "named by --design-sizes (random weights), each beside Qwen3 at the same width, depth and vocabulary")
     ap.add_argument("--design-sizes", default="0.6b,8b")

@@ -3,7 +3,7 @@ with random weights (no model folder at hand). The figures are those of the publ
 files; a model folder's own config.json always wins where there is one."""
 from __future__ import annotations
 
-from .model_config import GoluzenConfig, NegosunConfig, Qwen3Config, SigosunConfig, TavevikConfig
+from .model_config import GoluzenConfig, NegosunConfig, Qwen3Config, SigosunConfig, TavevikConfig, VefulixConfig
 
 SIZES = {
     # name: (layers, hidden, q heads, kv heads, head_dim, intermediate, vocab, tied)
@@ -139,7 +139,26 @@ def goluzen_config(size: str, layers: int | None = None):
                                     "layers": out, "max_position_embeddings": 40960}), L
 
 
-DESIGNS = ("sigosun", "negosun", "tavevik", "goluzen")
+def vefulix_config(size: str, layers: int | None = None):
+    """(a Vefulix configuration whose layers resemble that size's: the same width, vocabulary and attention heads, with
+    `layers` layers or as many as the size has; that count). Four residual streams. The mixers take turns: a delta rule with
+    half of the attention's heads at its head size (half as many key heads, four taps), attention over a latent of two head
+    sizes with queries from a latent of three, a matrix memory with a quarter of the heads and values twice as wide as keys,
+    latent attention again. Every layer has 32 experts of an eighth of the size's feed-forward width, four per token, and a
+    shared expert of half that width."""
+    L, h, Hq, Hkv, D, I, V, _ = SIZES[size]
+    n = layers or L
+    moe = {"kind": "moe", "expert": {"ff": max(8, I // 8)}, "shared": {"ff": max(8, I // 2)}, "router": {"experts": 32, "top": 4}}
+    heads = max(2, Hq // 2)
+    latent = {"type": "latent_attention", "mlp": moe,
+              "mixer": {"heads": Hq, "dim": D, "vdim": D, "q_rank": 3 * D, "kv_rank": 2 * D, "scale": D ** -0.5}}
+    turns = ({"type": "delta", "mlp": moe, "mixer": {"heads": heads, "kv_heads": heads // 2, "dim": D, "vdim": D, "conv": 4}}, latent,
+             {"type": "mlstm", "mlp": moe, "mixer": {"heads": max(1, Hq // 4), "dim": D, "vdim": 2 * D, "gate_cap": 15.0}}, latent)
+    return VefulixConfig.from_dict({"architecture": "Vefulix", "vocab": V, "width": h, "norm": {"eps": 1e-6}, "streams": 4,
+                                    "logit_softcap": 30.0, "layers": [turns[i % 4] for i in range(n)], "max_position_embeddings": 40960}), L
+
+
+DESIGNS = ("sigosun", "negosun", "tavevik", "goluzen", "vefulix")
 
 
 def named_config(name: str, layers: int | None = None):
@@ -148,6 +167,8 @@ def named_config(name: str, layers: int | None = None):
     design, _, size = name.rpartition(":")
     if size not in SIZES or design not in ("", "qwen3") + DESIGNS:
         raise KeyError(f"{name!r} is not one of {sorted(SIZES)}, optionally behind one of {[d + ':' for d in DESIGNS]}")
+    if design == "vefulix":
+        return vefulix_config(size, layers)
     if design == "goluzen":
         return goluzen_config(size, layers)
     if design == "negosun":
