@@ -1,7 +1,8 @@
 """The engine against a plain evaluation of whole sequences under every way of cutting the work, for any design.
 
 `Cuts(configs, pages, plain_logits)`: the test configurations by name (dictionaries with "vocab"), their page sizes, and a
-function (folder, token ids) -> float64 logits of every position. Each case takes `env` with .device, .dtype, .tol and
+function (folder, token ids) -> float64 logits of every position. Each case takes `env` with .device, .dtype, .tol (optionally
+.mean_tol: what the rows' errors have to stay within in the mean) and
 .runner(name, pages, slots) -> (runner, manager, folder); the same cases run on the CPU (plain kernel twins, float32) and on
 the GPU (HIP kernels, float32 and bfloat16). Pools start filled with NaN, so a read of a key or state nobody wrote poisons
 the logits.
@@ -28,6 +29,8 @@ class Cuts:
         ref = self.plain_logits(folder, ids)[: got.shape[0]]
         err = rel_err(got, ref)
         assert err <= env.tol, f"{what}: error {err:.3g} > {env.tol:g}; first bad position {helpers.first_bad_row(got, ref, env.tol)}"
+        mean = float(((got.double() - ref).abs().amax(-1) / ref.abs().max()).mean())
+        assert got.shape[0] < 9 or mean <= getattr(env, "mean_tol", env.tol), f"{what}: mean error of the rows {mean:.3g} > {env.mean_tol:g}"
 
     def whole(self, env, name):
         """Each request alone and whole: one token, two, lengths around pages and chunks."""
