@@ -1086,7 +1086,7 @@ class HipBackend:
         _check(_is_i32(state_slots) and _is_i32(cu_seqlens, B + 1) and len(q_lens) == B and sum(q_lens) == T, "decay_rows_recurrence: metadata")
         _check(1 <= N <= 256 and H % G == 0, "decay_rows_recurrence: up to 256 state rows, heads a multiple of the groups")
         y = torch.empty((T, H * P), dtype=torch.float32, device=v.device)
-        groups, prepared = decay_row_groups(B, H, N, P, max(q_lens))
+        groups, prepared = decay_row_groups(B, H, N, P, max(q_lens), T, per_head)
         NR = 32 if N <= 32 else 64 if N <= 64 else 128 if N <= 128 else 256
         pre = _scratch(3 * T * H * NR + T * H, v.device, "decay_rows") if prepared else None
         core().call("me_decay_rows_recurrence", q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0),
@@ -1732,15 +1732,22 @@ def expert_tile_rows(T: int, top: int, E: int) -> int:
 DECAY_PREPARE_MIN_TOKENS = 9      # requests of this many tokens or more: the tokens' values are shaped by a kernel of its own
 
 
-def decay_row_groups(num_seqs: int, H: int, N: int, P: int, longest: int = 1) -> tuple:
+def decay_row_groups(num_seqs: int, H: int, N: int, P: int, longest: int = 1, tokens: int | None = None, one_decay: bool = False) -> tuple:
     """(lanes that share a column of the state in `decay_rows_recurrence`, whether a first kernel shapes the tokens' values).
     A request is a chain: the fewer rows a lane walks per token, the shorter the chain's step, at the price of more waves
     and an exchange between lanes. Steps of long requests: the values of all tokens are shaped at once by a kernel of its
-    own (unit lengths, decays and their exponentials leave the chain), and 16 lanes share a column while that keeps the
-    launch within 16 waves a compute unit, else 4. Short steps shape inside the kernel: 4 lanes where a lane could not
-    keep a whole column in registers, or while one lane to a column leaves compute units without a wave; else 1."""
+    own (unit lengths, decays and their exponentials leave the chain), and 16 lanes share a column while the waves all run at
+    once (up to 16 a compute unit, and as many as its 160 KB of LDS hold: a wave keeps q, k and, unless a head has one decay,
+    the decays of 16 tokens there), else 4: 8 prompts of 2,048 tokens over 8 heads of 128 x 128, 2,048 waves of 16 lanes to a
+    column, take 1,249 us with one decay per head (all at once) and 2,793 with a decay per row (two rounds; 2,156 with 4
+    lanes). Requests of a few tokens in such a step (`tokens`: the step's) end early and are not counted. Short steps shape inside the
+    kernel: 4 lanes where a lane could not keep a whole column in registers, or while one lane to a column leaves compute
+    units without a wave; else 1."""
     if longest >= DECAY_PREPARE_MIN_TOKENS:
-        return (16 if num_seqs * H * -(-P // 4) <= 16 * _COMPUTE_UNITS else 4), True
+        chains = num_seqs if tokens is None else min(num_seqs, -(-tokens // longest))
+        rows = 32 if N <= 32 else 64 if N <= 64 else 128 if N <= 128 else 256
+        per_unit = min(16, 160 * 1024 // ((2 if one_decay else 3) * 16 * rows * 4 + 64))
+        return (16 if chains * H * -(-P // 4) <= per_unit * _COMPUTE_UNITS else 4), True
     if N > 64:
         return 4, False
     return (4 if num_seqs * H * -(-P // 64) < 2 * _COMPUTE_UNITS and N >= 16 else 1), False

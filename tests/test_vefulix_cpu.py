@@ -400,3 +400,14 @@ def test_named_sizes_build():
     cfg, _ = named_config("vefulix:0.6b", 8)
     plan = build_model(cfg).cache_plan()
     assert plan.call_writes == [False, True] * 4 and math.prod(plan.state_needs[2].shape) == 4 * 128 * 256 + 4 * 128 + 4
+
+
+def test_launch_rule_of_the_delta_rule_with_one_decay_per_head():
+    """Sixteen lanes to a column while the waves run in one round (a wave keeps fewer values in LDS than with a decay per row);
+    single tokens beside long portions do not count as chains."""
+    from mini_engine_amd.kernels import ops
+    rule = lambda lens, one: ops.decay_row_groups(len(lens), 8, 128, 128, max(lens), sum(lens), one)
+    assert rule([700] * 8, True) == (16, True) and rule([700] * 8, False) == (4, True)
+    assert rule([700] * 4, False) == (16, True) and rule([700] * 16, True) == (4, True)
+    assert rule([700] * 7 + [1] * 40, True) == (16, True)
+    assert rule([1] * 64, True) == (4, False)
