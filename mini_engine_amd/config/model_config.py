@@ -1008,3 +1008,173 @@ class VefulixConfig:
     def flat(self) -> dict[str, Any]:
         return {"vocab_size": self.vocab_size, "hidden_size": self.hidden_size, "num_hidden_layers": len(self.layers),
                 "layer_kinds": [layer.kind for layer in self.layers]}
+
+
+# ------------------------------------------------------------------------------------ Venezen
+@dataclass(frozen=True)
+class VenezenLayer:
+    """One entry of a Venezen config's `layers`: which mixer it has, the mixer's sizes and constants, and the
+    feed-forward's (None: the layer has no feed-forward)."""
+
+    kind: str                  # "latent_attention" or "attention"
+    mixer: dict
+    mlp: dict | None
+
+
+@register_config("Venezen")
+@dataclass(frozen=True)
+class VenezenConfig:
+    """The ``config.json`` keys of the Venezen design: pre-norm layers (layer norms without biases) that each name their
+    mixer, a run of layers that is passed several times with the same weights, the embedding's output joining the stream
+    again before every pass but the first. `latent_attention`: keys and values made head by head from a cached latent beside
+    one shared rotated key part (pairs half the rotating part apart). `attention`: grouped heads whose values are their keys,
+    a bias that falls with the distance at a slope per head, a trailing window, a sink that scores 0. Feed-forwards: dense with
+    biases, or routed experts under a clamped gate (a softmax over all scores, a correction for the choice, weights divided by
+    their sum times a constant; the last `router.identity` of them hand their input on) beside an optional shared one. The
+    embedding's rows are multiplied by `embedding.scale`; the head is the embedding table without it. Every size and constant
+    comes from the file."""
+
+    vocab_size: int
+    hidden_size: int
+    norm_eps: float
+    embedding_scale: float
+    layers: tuple
+    loop: tuple = (0, 0, 1)                # layers start .. stop - 1 run `times` times in a row
+    eos_token_id: int | None = None
+    max_position_embeddings: int | None = None
+
+    MIXERS = {"latent_attention": (("heads", int), ("dim", int), ("rot_dim", int), ("vdim", int), ("kv_rank", int), ("scale", float)),
+              "attention": (("heads", int), ("dim", int), ("scale", float))}
+
+    @property
+    def num_hidden_layers(self) -> int:
+        return len(self.layers)
+
+    def run_order(self) -> list:
+        """(layer, whether it begins a pass of the loop behind the first) in the order the layers run."""
+        start, stop, times = self.loop
+        order = [(i, False) for i in range(start)]
+        for k in range(times):
+            order += [(i, k > 0 and i == start) for i in range(start, stop)]
+        return order + [(i, False) for i in range(stop, len(self.layers))]
+
+    @classmethod
+    def from_dict(cls, raw: dict[str, Any]) -> "VenezenConfig":
+        norm = raw.get("norm")
+        if not isinstance(norm, dict):
+            raise ConfigError("config.json lacks the object 'norm'")
+        listed = raw.get("layers")
+        if not isinstance(listed, list) or not listed:
+            raise ConfigError("config.json lacks the list 'layers'")
+        layers = []
+        for i, entry in enumerate(listed):
+            where = f"layers[{i}]"
+            kind = entry.get("type") if isinstance(entry, dict) else None
+            if kind not in cls.MIXERS:
+                raise ConfigError(f"{where}: 'type' must be one of {sorted(cls.MIXERS)}, got {kind!r}")
+            m = entry.get("mixer")
+            if not isinstance(m, dict):
+                raise ConfigError(f"{where} lacks the object 'mixer'")
+            at = where + ".mixer"
+            mixer = {key: _need(m, key, typ, at) for key, typ in cls.MIXERS[kind]}
+            if kind == "latent_attention":
+                rot = m.get("rot")
+                mixer["rot_base"] = _need(rot, "base", float, at + ".rot") if rot else 1.0
+                if rot and rot.get("dims") is not None and int(rot["dims"]) != mixer["rot_dim"]:
+                    raise ConfigError(f"{at}: rot.dims must equal rot_dim")
+                if not rot and mixer["rot_dim"]:
+                    raise ConfigError(f"{at} lacks the object 'rot'")
+            else:
+                mask = m.get("mask")
+                mixer["kv_heads"] = _need(m, "kv_heads", int, at) if m.get("kv_heads") is not None else mixer["heads"]
+                mixer["window"] = _need(mask, "size", int, at + ".mask") if mask else None
+                if m.get("vdim") is not None and int(m["vdim"]) != mixer["dim"]:
+                    raise ConfigError(f"{at}: the values are the keys, vdim must equal dim")
+            mlp = entry.get("mlp")
+            ff = None
+            if mlp is not None:
+                fkind, at = mlp.get("kind"), where + ".mlp"
+                if fkind == "dense":
+                    ff = {"kind": "dense", "ff": _need(mlp, "ff", int, at)}
+                elif fkind == "moe":
+                    router, expert, shared = mlp.get("router"), mlp.get("expert"), mlp.get("shared")
+                    if not isinstance(router, dict) or not isinstance(expert, dict):
+                        raise ConfigError(f"{at} lacks the objects 'router' and 'expert'")
+                    ff = {"kind": "moe", "ff": _need(expert, "ff", int, at + ".expert"), "limit": _need(expert, "limit", float, at + ".expert"),
+                          "experts": _need(router, "experts", int, at + ".router"), "top": _need(router, "top", int, at + ".router"),
+                          "identity": int(router.get("identity") or 0),
+                          "scale": float(router["scale"]) if router.get("scale") is not None else 1.0,
+                          "shared_ff": _need(shared, "ff", int, at + ".shared") if shared else None,
+                          "shared_limit": _need(shared, "limit", float, at + ".shared") if shared else None}
+                else:
+                    raise ConfigError(f"{at}: 'kind' must be 'dense' or 'moe', got {fkind!r}")
+            layers.append(VenezenLayer(kind, mixer, ff))
+        emb, loop = raw.get("embedding") or {}, raw.get("loop")
+        cfg = cls(vocab_size=_need(raw, "vocab", int), hidden_size=_need(raw, "width", int),
+                  norm_eps=_need(norm, "eps", float, "config.json norm"),
+                  embedding_scale=float(emb["scale"]) if emb.get("scale") is not None else 1.0, layers=tuple(layers),
+                  loop=tuple(_need(loop, k, int, "config.json loop") for k in ("start", "stop", "times")) if loop else (0, 0, 1),
+                  eos_token_id=raw.get("eos_token_id"), max_position_embeddings=raw.get("max_position_embeddings"))
+        cfg.validate()
+        return cfg
+
+    def validate(self) -> None:
+        if self.vocab_size < 1 or self.hidden_size < 1 or not self.norm_eps > 0:
+            raise ConfigError("vocab and width must be positive and norm.eps above zero")
+        start, stop, times = self.loop
+        if not 0 <= start <= stop <= len(self.layers) or times < 1:
+            raise ConfigError(f"loop: layers {start} .. {stop} of {len(self.layers)}, {times} times")
+        for i, layer in enumerate(self.layers):
+            m, f, where = layer.mixer, layer.mlp, f"layers[{i}]"
+            if any(m[k] < 1 for k in ("heads", "dim", "vdim", "kv_rank", "kv_heads") if k in m) or not m["scale"] > 0:
+                raise ConfigError(f"{where}: sizes and the score scale must be positive")
+            if layer.kind == "attention":
+                if m["heads"] % m["kv_heads"]:
+                    raise ConfigError(f"{where}: {m['heads']} heads are not a multiple of {m['kv_heads']} kv_heads")
+                if m["window"] is not None and m["window"] < 1:
+                    raise ConfigError(f"{where}: mask.size must be positive")
+            elif m["rot_dim"] < 0 or m["rot_dim"] % 2 or not m["rot_base"] > 0:
+                raise ConfigError(f"{where}: rot_dim must be even and rot.base positive")
+            if f is None:
+                continue
+            if f["ff"] < 1:
+                raise ConfigError(f"{where}.mlp: ff must be positive")
+            if f["kind"] == "moe":
+                if f["experts"] < 1 or f["identity"] < 0 or not 1 <= f["top"] <= f["experts"] + f["identity"]:
+                    raise ConfigError(f"{where}.mlp: experts must be positive and top at most experts and identity experts together")
+                if not f["limit"] > 0 or (f["shared_ff"] is not None and (f["shared_ff"] < 1 or not f["shared_limit"] > 0)):
+                    raise ConfigError(f"{where}.mlp: the limits and shared.ff must be positive")
+
+    def to_dict(self) -> dict[str, Any]:
+        """A ``config.json`` that reads back to an equal config."""
+        out = []
+        for layer in self.layers:
+            m = {k: layer.mixer[k] for k, _ in self.MIXERS[layer.kind]}
+            if layer.kind == "latent_attention":
+                if m["rot_dim"]:
+                    m["rot"] = {"dims": m["rot_dim"], "base": layer.mixer["rot_base"]}
+            else:
+                m["kv_heads"], m["vdim"] = layer.mixer["kv_heads"], m["dim"]
+                if layer.mixer["window"] is not None:
+                    m["mask"] = {"size": layer.mixer["window"]}
+            f, mlp = layer.mlp, None
+            if f is not None and f["kind"] == "dense":
+                mlp = {"kind": "dense", "ff": f["ff"]}
+            elif f is not None:
+                mlp = {"kind": "moe", "expert": {"ff": f["ff"], "limit": f["limit"]},
+                       "router": {k: f[k] for k in ("experts", "top", "identity", "scale")}}
+                if f["shared_ff"] is not None:
+                    mlp["shared"] = {"ff": f["shared_ff"], "limit": f["shared_limit"]}
+            out.append({"type": layer.kind, "mixer": m, "mlp": mlp})
+        d = {"architecture": self.architecture_name, "vocab": self.vocab_size, "width": self.hidden_size, "norm": {"eps": self.norm_eps},
+             "embedding": {"scale": self.embedding_scale}, "layers": out}
+        if self.loop != (0, 0, 1):
+            d["loop"] = dict(zip(("start", "stop", "times"), self.loop))
+        for key in ("eos_token_id", "max_position_embeddings"):
+            if getattr(self, key) is not None:
+                d[key] = getattr(self, key)
+        return d
+
+    def flat(self) -> dict[str, Any]:
+        return {"vocab_size": self.vocab_size, "hidden_size": self.hidden_size, "num_hidden_layers": len(self.layers),
+                "layer_kinds": [layer.kind for layer in self.layers]}

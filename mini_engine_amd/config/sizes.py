@@ -3,7 +3,7 @@ with random weights (no model folder at hand). The figures are those of the publ
 files; a model folder's own config.json always wins where there is one."""
 from __future__ import annotations
 
-from .model_config import GoluzenConfig, NegosunConfig, Qwen3Config, SigosunConfig, TavevikConfig, VefulixConfig
+from .model_config import GoluzenConfig, NegosunConfig, Qwen3Config, SigosunConfig, TavevikConfig, VefulixConfig, VenezenConfig
 
 SIZES = {
     # name: (layers, hidden, q heads, kv heads, head_dim, intermediate, vocab, tied)
@@ -158,7 +158,31 @@ def vefulix_config(size: str, layers: int | None = None):
                                     "logit_softcap": 30.0, "layers": [turns[i % 4] for i in range(n)], "max_position_embeddings": 40960}), L
 
 
-DESIGNS = ("sigosun", "negosun", "tavevik", "goluzen", "vefulix")
+def venezen_config(size: str, layers: int | None = None):
+    """(a Venezen configuration whose layers resemble that size's: the same width, vocabulary and attention heads; `layers`
+    layer runs or as many as the size has layers; that count). The mixers take turns: latent attention (a latent of one and a
+    half head sizes, a rotating part of half a head size) twice, then attention under a window of 1,024 positions whose
+    values are its keys. The first layer's feed-forward is dense; the others have 32 experts of an eighth of the size's
+    feed-forward width beside 16 identity experts, four per token, and a shared expert of half that width. From four runs on,
+    the second quarter of the runs repeats in the third: layers that run twice."""
+    L, h, Hq, Hkv, D, I, V, _ = SIZES[size]
+    n = layers or L
+    again = n // 4                            # layers that run a second time
+    latent = {"type": "latent_attention",
+              "mixer": {"heads": Hq, "dim": D, "rot_dim": D // 2, "vdim": D, "kv_rank": 3 * D // 2, "scale": (3 * D // 2) ** -0.5,
+                        "rot": {"dims": D // 2, "base": 1e6}}}
+    attention = {"type": "attention", "mixer": {"heads": Hq, "kv_heads": Hkv, "dim": D, "vdim": D, "scale": D ** -0.5, "mask": {"size": 1024}}}
+    moe = {"kind": "moe", "expert": {"ff": max(8, I // 8), "limit": 7.0}, "shared": {"ff": max(8, I // 2), "limit": 7.0},
+           "router": {"experts": 32, "identity": 16, "top": 4, "scale": 2.5}}
+    out = [dict(attention if i % 3 == 2 else latent, mlp={"kind": "dense", "ff": I} if i == 0 else moe) for i in range(n - again)]
+    d = {"architecture": "Venezen", "vocab": V, "width": h, "norm": {"eps": 1e-6}, "embedding": {"scale": 8.0}, "layers": out,
+         "max_position_embeddings": 40960}
+    if again:
+        d["loop"] = {"start": again, "stop": 2 * again, "times": 2}
+    return VenezenConfig.from_dict(d), L
+
+
+DESIGNS = ("sigosun", "negosun", "tavevik", "goluzen", "vefulix", "venezen")
 
 
 def named_config(name: str, layers: int | None = None):
@@ -167,6 +191,8 @@ def named_config(name: str, layers: int | None = None):
     design, _, size = name.rpartition(":")
     if size not in SIZES or design not in ("", "qwen3") + DESIGNS:
         raise KeyError(f"{name!r} is not one of {sorted(SIZES)}, optionally behind one of {[d + ':' for d in DESIGNS]}")
+    if design == "venezen":
+        return venezen_config(size, layers)
     if design == "vefulix":
         return vefulix_config(size, layers)
     if design == "goluzen":

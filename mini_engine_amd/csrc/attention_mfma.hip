@@ -89,6 +89,11 @@ struct AttnArgs {
   // [rows, Hq] or nullptr: the natural logarithm of every (token, head)'s softmax denominator, -inf where it saw no key,
   // for a caller that joins further terms to the softmax afterwards
   float* lse_out;
+  // [Hq] or nullptr: e^sink joins a head's softmax denominator, a term without key or value
+  const float* sinks;
+  // [Hq], not negative: a score loses slope * (query position - key position) behind the cap (compiled in with
+  // ME_ATTN_DISTANCE only)
+  const float* slopes;
 };
 
 #ifndef ME_ATTN_SOFTCAP
@@ -108,6 +113,30 @@ __device__ __forceinline__ void cap_scores(const AttnArgs& a, float (&sv)[8]) {
     for (int i = 0; i < 8; ++i) sv[i] = back * fast_tanh(sv[i] * in);
   }
 #endif
+}
+#ifndef ME_ATTN_DISTANCE
+#define ME_ATTN_DISTANCE 0
+#endif
+// A head's slope in units of the raw dot product, which is still to be multiplied by the scale.
+__device__ __forceinline__ float column_slope(const AttnArgs& a, int head, bool valid) {
+#if ME_ATTN_DISTANCE
+  return valid ? a.slopes[head] / a.scale : 0.f;
+#else
+  return 0.f;
+#endif
+}
+// Eight neighbouring keys from first_key on, seen from the query at pos: each raw score loses slope * distance.
+__device__ __forceinline__ void distance_scores(float slope, int first_key, int pos, float (&sv)[8]) {
+#if ME_ATTN_DISTANCE
+  const float d = (float)(first_key - pos);
+#pragma unroll
+  for (int i = 0; i < 8; ++i) sv[i] = fmaf(slope, d + (float)i, sv[i]);
+#endif
+}
+// A softmax's denominator (under the reference point m, in the log2 domain) with its head's sink. A column that saw no key
+// stays at zero.
+__device__ __forceinline__ float with_sink(const AttnArgs& a, int head, float m, float ls) {
+  return (a.sinks != nullptr && ls > 0.f) ? ls + exp2f(fmaf(a.sinks[head], 1.4426950408889634f, -m)) : ls;
 }
 __device__ __forceinline__ float natural_lse(float m_log2, float ls) {
   return ls > 0.f ? (m_log2 + log2f(ls)) * 0.6931471805599453f : -INFINITY;
@@ -291,8 +320,8 @@ __device__ __forceinline__ void load_block(const AttnArgs& a, const int32_t* __r
 //   The accumulators are rescaled only when some column's max has risen (a wave-wide test).
 template <bool FULL>
 __device__ __forceinline__ void attend_block(const AttnArgs& a, const KVBlock& blk, const VBlock& vblk, int t0,
-                                             const bf16x8 (&qb)[KS], int col_lo, int col_hi, float& m, float& l,
-                                             f32x4 (&acc)[DT], int g) {
+                                             const bf16x8 (&qb)[KS], int col_lo, int col_hi, float slope, float& m,
+                                             float& l, f32x4 (&acc)[DT], int g) {
   const bf16x8 z = zero8();
   const float c = a.scale * 1.4426950408889634f;
   f32x4 st[2];
@@ -313,6 +342,7 @@ __device__ __forceinline__ void attend_block(const AttnArgs& a, const KVBlock& b
 #pragma unroll
   for (int i = 0; i < 8; ++i) sv[i] = st[i >> 2][i & 3];
   cap_scores(a, sv);
+  distance_scores(slope, t0 + 8 * g, col_hi, sv);
 #pragma unroll
   for (int i = 0; i < 8; ++i) {
     if (!FULL) {
@@ -398,12 +428,14 @@ __device__ __forceinline__ void block_scores(const KVBlock& blk, const bf16x8 (&
 // operand of the value product.
 template <bool FULL>
 __device__ __forceinline__ void block_softmax(const AttnArgs& a, const f32x4 (&st)[2], int t0, int col_lo,
-                                              int col_hi, float& m, float& l, f32x4 (&acc)[DT], int g, bf16x8& pb) {
+                                              int col_hi, float slope, float& m, float& l, f32x4 (&acc)[DT], int g,
+                                              bf16x8& pb) {
   const float c = a.scale * 1.4426950408889634f;
   float sv[8];
 #pragma unroll
   for (int i = 0; i < 8; ++i) sv[i] = st[i >> 2][i & 3];
   cap_scores(a, sv);
+  distance_scores(slope, t0 + 8 * g, col_hi, sv);
   if (!FULL) {
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
@@ -506,6 +538,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
     int64_t tq[CT];
     int head[CT];
     bool valid[CT];
+    float slope[CT];
 #pragma unroll
     for (int ct = 0; ct < CT; ++ct) {
       const int c = c0 + 16 * ct + n;
@@ -516,6 +549,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
       head[ct] = kvh * a.G + hh;
       const int pos = start + tok0 + tl;
       col_hi[ct] = valid[ct] ? pos : -1;
+      slope[ct] = column_slope(a, head[ct], valid[ct]);
       col_lo[ct] = a.window > 0 ? lower_edge(a, pos) : 0;
       load_q(a.q + tq[ct] * a.q_stride + (int64_t)head[ct] * HD, valid[ct], g, qb[ct]);
     }
@@ -574,11 +608,11 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
         if (full) {
 #pragma unroll
           for (int ct = 0; ct < CT; ++ct)
-            block_softmax<true>(a, st[ct], t0, col_lo[ct], col_hi[ct], m[ct], l[ct], acc[ct], g, pb[ct]);
+            block_softmax<true>(a, st[ct], t0, col_lo[ct], col_hi[ct], slope[ct], m[ct], l[ct], acc[ct], g, pb[ct]);
         } else {
 #pragma unroll
           for (int ct = 0; ct < CT; ++ct)
-            block_softmax<false>(a, st[ct], t0, col_lo[ct], col_hi[ct], m[ct], l[ct], acc[ct], g, pb[ct]);
+            block_softmax<false>(a, st[ct], t0, col_lo[ct], col_hi[ct], slope[ct], m[ct], l[ct], acc[ct], g, pb[ct]);
           hide_values(V);
         }
 #pragma unroll
@@ -605,7 +639,8 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
           *reinterpret_cast<f32x4*>(p + 16 * dt + 4 * g) = acc[ct][dt];
         if (g == 0) { p[HD] = m[ct]; p[HD + 1] = ls; }
       } else if (valid[ct]) {
-        const float inv = ls > 0.f ? 1.f / ls : 0.f;
+        const float dn = with_sink(a, head[ct], m[ct], ls);
+        const float inv = dn > 0.f ? 1.f / dn : 0.f;
         if (a.lse_out != nullptr && g == 0) a.lse_out[(int64_t)tq[ct] * a.Hq + head[ct]] = natural_lse(m[ct], ls);
         bf16_t* o = a.out + tq[ct] * a.out_stride + (int64_t)head[ct] * HD + 4 * g;
 #pragma unroll
@@ -806,6 +841,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
     int64_t tq[CT];
     int head[CT];
     bool valid[CT];
+    float slope[CT];
 #pragma unroll
     for (int ct = 0; ct < CT; ++ct) {
       const int cc = c0 + 16 * ct + n;
@@ -816,6 +852,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
       head[ct] = kvh * a.G + hh;
       const int pos = start + tok0 + tl;
       col_hi[ct] = valid[ct] ? pos : -1;
+      slope[ct] = column_slope(a, head[ct], valid[ct]);
       col_lo[ct] = a.window > 0 ? lower_edge(a, pos) : 0;
       load_q(a.q + tq[ct] * a.q_stride + (int64_t)head[ct] * HD, valid[ct], g, qb[ct]);
     }
@@ -872,11 +909,11 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
       if (full) {
 #pragma unroll
         for (int ct = 0; ct < CT; ++ct)
-          block_softmax<true>(a, st[ct], t0, col_lo[ct], col_hi[ct], m[ct], l[ct], acc[ct], g, pb[ct]);
+          block_softmax<true>(a, st[ct], t0, col_lo[ct], col_hi[ct], slope[ct], m[ct], l[ct], acc[ct], g, pb[ct]);
       } else {
 #pragma unroll
         for (int ct = 0; ct < CT; ++ct)
-          block_softmax<false>(a, st[ct], t0, col_lo[ct], col_hi[ct], m[ct], l[ct], acc[ct], g, pb[ct]);
+          block_softmax<false>(a, st[ct], t0, col_lo[ct], col_hi[ct], slope[ct], m[ct], l[ct], acc[ct], g, pb[ct]);
       }
 #pragma unroll
       for (int dt = 0; dt < DT; ++dt) {
@@ -902,7 +939,8 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
           *reinterpret_cast<f32x4*>(p + 16 * dt + 4 * g) = acc[ct][dt];
         if (g == 0) { p[HD] = m[ct]; p[HD + 1] = ls; }
       } else if (valid[ct]) {
-        const float inv = ls > 0.f ? 1.f / ls : 0.f;
+        const float dn = with_sink(a, head[ct], m[ct], ls);
+        const float inv = dn > 0.f ? 1.f / dn : 0.f;
         if (a.lse_out != nullptr && g == 0) a.lse_out[(int64_t)tq[ct] * a.Hq + head[ct]] = natural_lse(m[ct], ls);
         bf16_t* o = a.out + tq[ct] * a.out_stride + (int64_t)head[ct] * HD + 4 * g;
 #pragma unroll
@@ -1105,6 +1143,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(W, W))
     int64_t tq[CT];
     int head[CT];
     bool valid[CT];
+    float slope[CT];
 #pragma unroll
     for (int ct = 0; ct < CT; ++ct) {
       const int cc = c0 + 16 * ct + n;
@@ -1115,6 +1154,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(W, W))
       head[ct] = kvh * a.G + hh;
       const int pos = start + tok0 + tl;
       col_hi[ct] = valid[ct] ? pos : -1;
+      slope[ct] = column_slope(a, head[ct], valid[ct]);
       col_lo[ct] = WINDOW ? lower_edge(a, pos) : 0;
       load_q(a.q + tq[ct] * a.q_stride + (int64_t)head[ct] * HD, valid[ct], g, qb[ct]);
     }
@@ -1186,7 +1226,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(W, W))
         softmax_priority(true);
 #pragma unroll
         for (int ct = 0; ct < CT; ++ct)
-          block_softmax<FULL>(a, st[ct], t0, col_lo[ct], col_hi[ct], m[ct], l[ct], acc[ct], g, pb[ct]);
+          block_softmax<FULL>(a, st[ct], t0, col_lo[ct], col_hi[ct], slope[ct], m[ct], l[ct], acc[ct], g, pb[ct]);
         softmax_priority(false);
         lds_reads_done(va);
 #pragma unroll
@@ -1211,7 +1251,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(W, W))
         softmax_priority(true);
 #pragma unroll
         for (int ct = 0; ct < CT; ++ct)
-          block_softmax<FULL>(a, st[ct], t0, col_lo[ct], col_hi[ct], m[ct], l[ct], acc[ct], g, pb[ct]);
+          block_softmax<FULL>(a, st[ct], t0, col_lo[ct], col_hi[ct], slope[ct], m[ct], l[ct], acc[ct], g, pb[ct]);
         softmax_priority(false);
         const unsigned char* vb = pf_lds + cur * DMA_BUF + rd_v;
 #pragma unroll
@@ -1245,7 +1285,8 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(W, W))
           *reinterpret_cast<f32x4*>(p + 16 * dt + 4 * g) = acc[ct][dt];
         if (g == 0) { p[HD] = m[ct]; p[HD + 1] = ls; }
       } else if (valid[ct]) {
-        const float inv = ls > 0.f ? 1.f / ls : 0.f;
+        const float dn = with_sink(a, head[ct], m[ct], ls);
+        const float inv = dn > 0.f ? 1.f / dn : 0.f;
         if (a.lse_out != nullptr && g == 0) a.lse_out[(int64_t)tq[ct] * a.Hq + head[ct]] = natural_lse(m[ct], ls);
         bf16_t* o = a.out + tq[ct] * a.out_stride + (int64_t)head[ct] * HD + 4 * g;
 #pragma unroll
@@ -1301,7 +1342,8 @@ __global__ void __launch_bounds__(256) attn_prefill_merge_kernel(AttnArgs a, int
 #pragma unroll
     for (int i = 0; i < MERGE_EPL; ++i) o[i] += w * v[i];
   }
-  const float inv = ls > 0.f ? 1.f / ls : 0.f;
+  const float dn = with_sink(a, hq, M, ls);
+  const float inv = dn > 0.f ? 1.f / dn : 0.f;
   if (a.lse_out != nullptr && part == 0) a.lse_out[row] = natural_lse(M, ls);
   bf16_t* dst = a.out + t * a.out_stride + (int64_t)hq * HD + part * MERGE_EPL;
 #pragma unroll
@@ -1485,6 +1527,7 @@ __global__ void __launch_bounds__(256, HD <= 128 ? 3 : (HD <= 256 ? 2 : 1)) attn
     if (PROLOGUE) load_q(q_s + (valid ? n : 0) * HD, valid, g, qb);
     else load_q(a.q + t * a.q_stride + (int64_t)head * HD, valid, g, qb);
     const int col_hi = valid ? pos : -1;
+    const float slope = column_slope(a, head, valid);
     // one block: what the new token brings comes from LDS, then scores, softmax and the weighted sum
     auto work_on = [&](KVBlock& A, VBlock& vb, int t0) {
       if (holds_new && pos >= t0 && pos < t0 + 32) {
@@ -1510,8 +1553,8 @@ __global__ void __launch_bounds__(256, HD <= 128 ? 3 : (HD <= 256 ? 2 : 1)) attn
           }
         }
       }
-      if (t0 + 32 <= L && t0 >= lo) attend_block<true>(a, A, vb, t0, qb, lo, col_hi, m, l, acc, g);
-      else attend_block<false>(a, A, vb, t0, qb, lo, col_hi, m, l, acc, g);
+      if (t0 + 32 <= L && t0 >= lo) attend_block<true>(a, A, vb, t0, qb, lo, col_hi, slope, m, l, acc, g);
+      else attend_block<false>(a, A, vb, t0, qb, lo, col_hi, slope, m, l, acc, g);
     };
     if constexpr (AHEAD) {
       VBlock vb;
@@ -1559,7 +1602,8 @@ __global__ void __launch_bounds__(256, HD <= 128 ? 3 : (HD <= 256 ? 2 : 1)) attn
     }
     const int hq = kvh * a.G + ctile * 16 + c;
     if (a.num_parts == 1) {
-      a.out[t * a.out_stride + (int64_t)hq * HD + d] = static_cast<bf16_t>(ls > 0.f ? o / ls : 0.f);
+      const float dn = with_sink(a, hq, M, ls);
+      a.out[t * a.out_stride + (int64_t)hq * HD + d] = static_cast<bf16_t>(dn > 0.f ? o / dn : 0.f);
       if (a.lse_out != nullptr && d == 0) a.lse_out[(int64_t)t * a.Hq + hq] = natural_lse(M, ls);
     } else {
       const int64_t row = ((int64_t)b * a.Hq + hq) * a.num_parts + part;
@@ -1596,7 +1640,8 @@ __global__ void __launch_bounds__(128) attn_reduce_kernel(AttnArgs a) {
     const float ls = wave_sum(f * lp);
     wgt[p] = f;
     if (p == 0) {
-      inv_s = ls > 0.f ? 1.f / ls : 0.f;
+      const float dn = with_sink(a, hq, M, ls);
+      inv_s = dn > 0.f ? 1.f / dn : 0.f;
       if (a.lse_out != nullptr) a.lse_out[(int64_t)b * a.Hq + hq] = natural_lse(M, ls);
     }
   }
@@ -1626,7 +1671,9 @@ extern "C" int me_attn_head_dim() { return HD; }
 static int fill_common(AttnArgs& a, const void* q, int64_t q_stride, void* out, int64_t out_stride,
                        const void* k_cache, const void* v_cache, const int32_t* block_tables, int bt_stride,
                        const int32_t* context_lens, int num_seqs, int Hq, int Hkv, int page, float scale,
-                       int window, float softcap = 0.f, float* lse_out = nullptr) {
+                       int window, float softcap, const float* sinks, const float* slopes, float* lse_out) {
+  ME_CHECK(ME_ATTN_DISTANCE || slopes == nullptr, "attention: this library was built without distance biases");
+  ME_CHECK(!ME_ATTN_DISTANCE || slopes != nullptr, "attention: this library was built for distance biases and needs the slopes");
   ME_CHECK(ME_ATTN_SOFTCAP || softcap == 0.f, "attention: this library was built without the score cap");
   ME_CHECK(softcap >= 0.f, "attention: the score cap must not be negative");
   ME_CHECK(Hq >= 1 && Hkv >= 1 && Hq % Hkv == 0, "attention: %d query heads are not a multiple of %d key heads", Hq, Hkv);
@@ -1650,7 +1697,7 @@ static int fill_common(AttnArgs& a, const void* q, int64_t q_stride, void* out, 
   a.seg_keys = 0; a.max_segs = 1; a.pf_scratch = nullptr; a.seq_of_token = nullptr; a.seq_base = 0;
   a.raw_k = a.raw_v = nullptr; a.q_w = a.k_w = nullptr; a.eps = 0.f; a.rope = nullptr;
   a.k_cache_w = a.v_cache_w = nullptr;
-  a.softcap = softcap; a.lse_out = lse_out;
+  a.softcap = softcap; a.lse_out = lse_out; a.sinks = sinks; a.slopes = slopes;
   return 0;
 }
 
@@ -1661,11 +1708,12 @@ extern "C" int me_attn_prefill(const void* q, int64_t q_stride, void* out, int64
                                int bt_stride, const int32_t* context_lens, const int32_t* cu_seqlens,
                                int num_seqs, int64_t num_tokens, int Hq, int Hkv, int page, float scale,
                                int window, int col_tiles_per_wave, int shared, int waves, int seg_keys, int max_segs, float* pf_scratch,
-                               const int32_t* seq_of_token, int seq_base, float softcap, float* lse_out, hipStream_t stream) {
+                               const int32_t* seq_of_token, int seq_base, float softcap, const float* sinks, const float* slopes,
+                               float* lse_out, hipStream_t stream) {
   if (num_seqs == 0 || num_tokens == 0) return 0;
   AttnArgs a;
   if (fill_common(a, q, q_stride, out, out_stride, k_cache, v_cache, block_tables, bt_stride, context_lens,
-                  num_seqs, Hq, Hkv, page, scale, window, softcap, lse_out)) return -1;
+                  num_seqs, Hq, Hkv, page, scale, window, softcap, sinks, slopes, lse_out)) return -1;
   a.cu_seqlens = cu_seqlens;
   // column tiles per wave: 2 when the step has enough tokens to fill the GPU with the larger tiles
   const int ct = (col_tiles_per_wave == 1 || col_tiles_per_wave == 2) ? col_tiles_per_wave
@@ -1775,15 +1823,17 @@ extern "C" int me_attn_decode(const void* q, int64_t q_stride, void* out, int64_
                               const void* k_cache, const void* v_cache, const int32_t* block_tables,
                               int bt_stride, const int32_t* context_lens, int num_seqs, int Hq, int Hkv,
                               int page, float scale, int window, int part_size, int num_parts,
-                              float* scratch, int spread_heads, float softcap, float* lse_out, hipStream_t stream) {
+                              float* scratch, int spread_heads, float softcap, const float* sinks, const float* slopes,
+                              float* lse_out, hipStream_t stream) {
   if (num_seqs == 0) return 0;
   AttnArgs a;
   if (fill_common(a, q, q_stride, out, out_stride, k_cache, v_cache, block_tables, bt_stride, context_lens,
-                  num_seqs, Hq, Hkv, page, scale, window, softcap, lse_out)) return -1;
+                  num_seqs, Hq, Hkv, page, scale, window, softcap, sinks, slopes, lse_out)) return -1;
   return launch_decode(a, num_seqs, part_size, num_parts, scratch, spread_heads, false, stream);
 }
 
-// A whole decode step's attention from the packed projection rows [num_seqs, (Hq + 2 Hkv) * HD] (row r belongs
+// A whole decode step's attention from the packed projection rows [num_seqs, (Hq + 2 Hkv) * HD], or with values_are_keys
+// [num_seqs, (Hq + Hkv) * HD]: the values are then the keys as projected, in front of norm and rotation (row r belongs
 // to sequence r, its token stands at position context_lens[r] - 1): per-head norms of q and k (q_w, k_w
 // float32 [HD], or both null), rotation by `rope` [rope_rows, HD/2, 2] (or null), the new key and value into
 // their page (the one the block table names for that position), attention over the pages. The rows are left as
@@ -1794,18 +1844,19 @@ extern "C" int me_attn_decode_fused(const void* qkv, int64_t row_stride, void* o
                                     void* k_cache, void* v_cache, const int32_t* block_tables, int bt_stride,
                                     const int32_t* context_lens, int max_context, int num_seqs, int Hq, int Hkv,
                                     int page, float scale, int window, int part_size, int num_parts,
-                                    float* scratch, int spread_heads, float softcap, float* lse_out, hipStream_t stream) {
+                                    float* scratch, int spread_heads, float softcap, const float* sinks,
+                                    const float* slopes, float* lse_out, int values_are_keys, hipStream_t stream) {
   if (num_seqs == 0) return 0;
   AttnArgs a;
   if (fill_common(a, qkv, row_stride, out, out_stride, k_cache, v_cache, block_tables, bt_stride, context_lens,
-                  num_seqs, Hq, Hkv, page, scale, window, softcap, lse_out)) return -1;
+                  num_seqs, Hq, Hkv, page, scale, window, softcap, sinks, slopes, lse_out)) return -1;
   ME_CHECK((q_w == nullptr) == (k_w == nullptr), "attention: give both norm weights or neither");
   ME_CHECK(rope == nullptr || (max_context >= 0 && max_context <= rope_rows),
            "attention: a context of %d tokens is beyond the rotation table's %d positions", max_context, rope_rows);
   ME_CHECK(rope == nullptr || reinterpret_cast<uintptr_t>(rope) % 8 == 0, "attention: the rotation table must be 8-byte aligned");
-  ME_CHECK(row_stride >= (int64_t)(Hq + 2 * Hkv) * HD, "attention: packed rows must hold q, k and v");
+  ME_CHECK(row_stride >= (int64_t)(Hq + (values_are_keys ? 1 : 2) * Hkv) * HD, "attention: packed rows must hold q, k and v");
   a.raw_k = (const bf16_t*)qkv + (int64_t)Hq * HD;
-  a.raw_v = a.raw_k + (int64_t)Hkv * HD;
+  a.raw_v = values_are_keys ? a.raw_k : a.raw_k + (int64_t)Hkv * HD;
   a.q_w = q_w; a.k_w = k_w; a.eps = eps; a.rope = rope;
   a.k_cache_w = (bf16_t*)k_cache; a.v_cache_w = (bf16_t*)v_cache;
   return launch_decode(a, num_seqs, part_size, num_parts, scratch, spread_heads, true, stream);

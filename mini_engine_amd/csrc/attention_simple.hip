@@ -7,7 +7,8 @@
 // scale * q.k; softmax over kept keys; output = sum p_j v_j. A window w additionally keeps
 // only j > position - w (not in the reference). Three further options: `keep_first` n keeps the keys j < n visible
 // behind a window; `softcap` c > 0 bends every score to c * tanh(score / c) before the softmax; `sinks` (one float per
-// query head) adds exp(sink) to the softmax's denominator, a term without key or value.
+// query head) adds exp(sink) to the softmax's denominator, a term without key or value. `slopes` (one float per query
+// head) takes slope * (position - j) off the score of key j, behind the cap.
 //
 // Keys are processed in chunks whose boundaries are multiples of the chunk size counted from
 // position 0 of the request, so the order of every sum for a given token is the same however
@@ -15,6 +16,7 @@
 #include "common.h"
 
 #define AS_THREADS 256
+#define AS_CHANNELS 4
 
 template <typename T>
 __global__ void __launch_bounds__(AS_THREADS)
@@ -23,7 +25,8 @@ attn_simple_kernel(const T* __restrict__ q, int64_t q_stride, T* __restrict__ ou
                    const int32_t* __restrict__ block_tables, int bt_stride,
                    const int32_t* __restrict__ seq_of_token, const int32_t* __restrict__ positions,
                    const int32_t* __restrict__ context_lens, int Hq, int Hkv, int D, int page, float scale,
-                   int window, int keep_first, float softcap, const float* __restrict__ sinks) {
+                   int window, int keep_first, float softcap, const float* __restrict__ sinks,
+                   const float* __restrict__ slopes) {
   extern __shared__ float lds[];
   float* qs = lds;                 // D
   float* sc = lds + D;             // AS_THREADS scores / probabilities
@@ -48,8 +51,11 @@ attn_simple_kernel(const T* __restrict__ q, int64_t q_stride, T* __restrict__ ou
   // behind a window the first keep_first keys stay visible: the chunks walk [0, kept) and then [lo, hi)
   const int kept = (window > 0 && keep_first > 0) ? min(min(keep_first, lo), hi) : 0;
   float m = -INFINITY, l = 0.f;
-  // thread d < D owns output channel d (two channels per thread when D > AS_THREADS)
-  float acc0 = 0.f, acc1 = 0.f;
+  // a thread owns the output channels tid, tid + AS_THREADS, ...
+  float acc[AS_CHANNELS];
+#pragma unroll
+  for (int dd = 0; dd < AS_CHANNELS; ++dd) acc[dd] = 0.f;
+  const float slope = slopes != nullptr ? slopes[h] : 0.f;
 
   const int first_c0 = (lo / AS_THREADS) * AS_THREADS;
   for (int c0 = kept > 0 ? 0 : first_c0; c0 < hi; c0 += AS_THREADS) {
@@ -67,6 +73,7 @@ attn_simple_kernel(const T* __restrict__ q, int64_t q_stride, T* __restrict__ ou
         for (int d = 0; d < D; ++d) dot += qs[d] * to_f32<T>(kr[d]);
         s = dot * scale;
         if (softcap > 0.f) s = softcap * tanhf(s / softcap);
+        s -= slope * (float)(pos - j);
       }
     }
     // chunk max
@@ -88,10 +95,9 @@ attn_simple_kernel(const T* __restrict__ q, int64_t q_stride, T* __restrict__ ou
     const float alpha = (m == -INFINITY) ? 0.f : expf(m - m_new);   // m finite implies m_new finite
     l = l * alpha + ps;
     m = m_new;
-    acc0 *= alpha;
-    acc1 *= alpha;
     const int jb = kept > 0 ? c0 : max(c0, lo), je = min(c0 + AS_THREADS, hi);
-    for (int dd = 0; dd < 2; ++dd) {
+#pragma unroll
+    for (int dd = 0; dd < AS_CHANNELS; ++dd) {
       const int d = tid + dd * AS_THREADS;
       if (d < D) {
         float a = 0.f;
@@ -102,7 +108,7 @@ attn_simple_kernel(const T* __restrict__ q, int64_t q_stride, T* __restrict__ ou
           const int off = jj % page;
           a += sc[jj - c0] * to_f32<T>(v_cache[((pg * Hkv + kvh) * (int64_t)D + d) * page + off]);
         }
-        if (dd == 0) acc0 += a; else acc1 += a;
+        acc[dd] = acc[dd] * alpha + a;
       }
     }
     __syncthreads();
@@ -113,22 +119,23 @@ attn_simple_kernel(const T* __restrict__ q, int64_t q_stride, T* __restrict__ ou
     const float m_new = fmaxf(m, sk);
     const float alpha = (m == -INFINITY) ? 0.f : expf(m - m_new);
     l = l * alpha + expf(sk - m_new);
-    acc0 *= alpha;
-    acc1 *= alpha;
+#pragma unroll
+    for (int dd = 0; dd < AS_CHANNELS; ++dd) acc[dd] *= alpha;
   }
   const float inv = l > 0.f ? 1.f / l : 0.f;
-  if (tid < D) out[t * out_stride + (int64_t)h * D + tid] = from_f32<T>(acc0 * inv);
-  if (tid + AS_THREADS < D) out[t * out_stride + (int64_t)h * D + tid + AS_THREADS] = from_f32<T>(acc1 * inv);
+#pragma unroll
+  for (int dd = 0; dd < AS_CHANNELS; ++dd)
+    if (tid + dd * AS_THREADS < D) out[t * out_stride + (int64_t)h * D + tid + dd * AS_THREADS] = from_f32<T>(acc[dd] * inv);
 }
 
 extern "C" int me_attn_simple(const void* q, int64_t q_stride, void* out, int64_t out_stride, int dtype,
                               const void* k_cache, const void* v_cache, const int32_t* block_tables,
                               int bt_stride, const int32_t* seq_of_token, const int32_t* positions,
                               const int32_t* context_lens, int64_t num_tokens, int Hq, int Hkv, int D, int page, float scale, int window,
-                              int keep_first, float softcap, const float* sinks, hipStream_t stream) {
+                              int keep_first, float softcap, const float* sinks, const float* slopes, hipStream_t stream) {
   if (num_tokens == 0) return 0;
   ME_CHECK(Hq >= 1 && Hkv >= 1 && Hq % Hkv == 0, "attention: %d query heads are not a multiple of %d key heads", Hq, Hkv);
-  ME_CHECK(D >= 1 && D <= 2 * AS_THREADS, "attention (float32 path): head_dim %d outside 1..%d", D, 2 * AS_THREADS);
+  ME_CHECK(D >= 1 && D <= AS_CHANNELS * AS_THREADS, "attention (float32 path): head_dim %d outside 1..%d", D, AS_CHANNELS * AS_THREADS);
   ME_CHECK(page >= 1, "attention: bad page size");
   ME_CHECK(keep_first >= 0 && softcap >= 0.f, "attention: keep_first and softcap must not be negative");
   dim3 grid(num_tokens, Hq), block(AS_THREADS);
@@ -136,11 +143,11 @@ extern "C" int me_attn_simple(const void* q, int64_t q_stride, void* out, int64_
   if (dtype == ME_F32)
     attn_simple_kernel<float><<<grid, block, lds, stream>>>(
         (const float*)q, q_stride, (float*)out, out_stride, (const float*)k_cache, (const float*)v_cache,
-        block_tables, bt_stride, seq_of_token, positions, context_lens, Hq, Hkv, D, page, scale, window, keep_first, softcap, sinks);
+        block_tables, bt_stride, seq_of_token, positions, context_lens, Hq, Hkv, D, page, scale, window, keep_first, softcap, sinks, slopes);
   else if (dtype == ME_BF16)
     attn_simple_kernel<bf16_t><<<grid, block, lds, stream>>>(
         (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache,
-        block_tables, bt_stride, seq_of_token, positions, context_lens, Hq, Hkv, D, page, scale, window, keep_first, softcap, sinks);
+        block_tables, bt_stride, seq_of_token, positions, context_lens, Hq, Hkv, D, page, scale, window, keep_first, softcap, sinks, slopes);
   else
     ME_CHECK(false, "attention: bad dtype code %d", dtype);
   ME_LAUNCH_CHECK();
@@ -162,7 +169,7 @@ attn_tail_kernel(const T* __restrict__ q, int64_t q_stride, T* __restrict__ out,
                  const T* __restrict__ k_cache, const T* __restrict__ v_cache, const int32_t* __restrict__ block_tables, int bt_stride,
                  const int32_t* __restrict__ seq_of_token, const int32_t* __restrict__ positions,
                  const int32_t* __restrict__ context_lens, int Hq, int Hkv, int D, int page, float scale, int window,
-                 int keep_first, float softcap, const float* __restrict__ sinks) {
+                 int keep_first, float softcap, const float* __restrict__ sinks, const float* __restrict__ slopes) {
   __shared__ float qs[AT_MAX_D];
   __shared__ float sc[64];
   const int64_t t = blockIdx.x;
@@ -174,6 +181,7 @@ attn_tail_kernel(const T* __restrict__ q, int64_t q_stride, T* __restrict__ out,
   const int hi = min(pos + 1, context_lens[b]);
   const int lo = window > 0 ? max(0, pos - window + 1) : 0;
   const int kept = (window > 0 && keep_first > 0) ? min(min(keep_first, lo), hi) : 0;
+  const float slope = slopes != nullptr ? slopes[h] : 0.f;
   float m2 = -INFINITY, l2 = 0.f;
   float acc[AT_MAX_D / 64];
 #pragma unroll
@@ -198,6 +206,7 @@ attn_tail_kernel(const T* __restrict__ q, int64_t q_stride, T* __restrict__ out,
       if (pg >= 0) {
         s = dot * scale;
         if (softcap > 0.f) s = softcap * tanhf(s / softcap);
+        s -= slope * (float)(pos - j);
       }
       const float m_new = fmaxf(m2, wave_max(s));
       const float p = (s > -INFINITY) ? expf(s - m_new) : 0.f;
@@ -248,7 +257,7 @@ extern "C" int me_attn_tail(const void* q, int64_t q_stride, void* out, int64_t 
                             const void* k_cache, const void* v_cache, const int32_t* block_tables, int bt_stride,
                             const int32_t* seq_of_token, const int32_t* positions, const int32_t* context_lens,
                             int64_t num_tokens, int Hq, int Hkv, int D, int page, float scale, int window, int keep_first,
-                            float softcap, const float* sinks, hipStream_t stream) {
+                            float softcap, const float* sinks, const float* slopes, hipStream_t stream) {
   if (num_tokens == 0) return 0;
   ME_CHECK(Hq >= 1 && Hkv >= 1 && Hq % Hkv == 0 && Hq <= 65535, "attention tail: %d query heads over %d key heads", Hq, Hkv);
   ME_CHECK(D >= 1 && D <= AT_MAX_D && page >= 1 && keep_first >= 0 && softcap >= 0.f, "attention tail: head size 1..%d", AT_MAX_D);
@@ -257,11 +266,11 @@ extern "C" int me_attn_tail(const void* q, int64_t q_stride, void* out, int64_t 
   if (dtype == ME_F32)
     attn_tail_kernel<float><<<grid, block, 0, stream>>>((const float*)q, q_stride, (float*)out, out_stride, lse, (const float*)k_cache,
         (const float*)v_cache, block_tables, bt_stride, seq_of_token, positions, context_lens, Hq, Hkv, D, page, scale, window,
-        keep_first, softcap, sinks);
+        keep_first, softcap, sinks, slopes);
   else
     attn_tail_kernel<bf16_t><<<grid, block, 0, stream>>>((const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, lse, (const bf16_t*)k_cache,
         (const bf16_t*)v_cache, block_tables, bt_stride, seq_of_token, positions, context_lens, Hq, Hkv, D, page, scale, window,
-        keep_first, softcap, sinks);
+        keep_first, softcap, sinks, slopes);
   ME_LAUNCH_CHECK();
   return 0;
 }

@@ -347,7 +347,7 @@ extern "C" int me_rms_norm(const void* x, int x_dtype, int num_partials, int64_t
 // gu: [T, 2I] with gate = first I columns (reference layers/activation.py:6); out: [T, I].
 // VEC: a thread takes 16 bytes of gate and of up at a time (I a multiple of the vector length).
 template <typename T, bool VEC>
-__global__ void silu_and_mul_kernel(const T* __restrict__ gu, T* __restrict__ out, int64_t rows, int inter) {
+__global__ void silu_and_mul_kernel(const T* __restrict__ gu, const float* __restrict__ bias, T* __restrict__ out, int64_t rows, int inter) {
   constexpr int W = VEC ? 16 / sizeof(T) : 1;
   const int per_row = inter / W;
   const int64_t total = rows * (int64_t)per_row;
@@ -365,15 +365,17 @@ __global__ void silu_and_mul_kernel(const T* __restrict__ gu, T* __restrict__ ou
     }
 #pragma unroll
     for (int j = 0; j < W; ++j) {
-      const float gf = to_f32<T>(g[j]);
-      o[j] = from_f32<T>(gf / (1.f + expf(-gf)) * to_f32<T>(u[j]));
+      float gf = to_f32<T>(g[j]), uf = to_f32<T>(u[j]);
+      if (bias) { gf += bias[i + j]; uf += bias[inter + i + j]; }
+      o[j] = from_f32<T>(gf / (1.f + expf(-gf)) * uf);
     }
     if (VEC) *reinterpret_cast<uint4*>(out + t * inter + i) = *reinterpret_cast<const uint4*>(o);
     else out[t * inter + i] = o[0];
   }
 }
 
-extern "C" int me_silu_and_mul(const void* gu, void* out, int dtype, int64_t rows, int inter,
+// bias: float32 [2 I] (the gates', then the ups') that joins gu first, or null
+extern "C" int me_silu_and_mul(const void* gu, const float* bias, void* out, int dtype, int64_t rows, int inter,
                                hipStream_t stream) {
   if (rows == 0) return 0;
   ME_CHECK(inter > 0, "silu_and_mul: intermediate size must be positive");
@@ -385,11 +387,11 @@ extern "C" int me_silu_and_mul(const void* gu, void* out, int dtype, int64_t row
   if (blocks > 65536) blocks = 65536;
   dim3 grid(blocks), block(256);
   if (dtype == ME_BF16) {
-    if (vec) silu_and_mul_kernel<bf16_t, true><<<grid, block, 0, stream>>>((const bf16_t*)gu, (bf16_t*)out, rows, inter);
-    else silu_and_mul_kernel<bf16_t, false><<<grid, block, 0, stream>>>((const bf16_t*)gu, (bf16_t*)out, rows, inter);
+    if (vec) silu_and_mul_kernel<bf16_t, true><<<grid, block, 0, stream>>>((const bf16_t*)gu, bias, (bf16_t*)out, rows, inter);
+    else silu_and_mul_kernel<bf16_t, false><<<grid, block, 0, stream>>>((const bf16_t*)gu, bias, (bf16_t*)out, rows, inter);
   } else {
-    if (vec) silu_and_mul_kernel<float, true><<<grid, block, 0, stream>>>((const float*)gu, (float*)out, rows, inter);
-    else silu_and_mul_kernel<float, false><<<grid, block, 0, stream>>>((const float*)gu, (float*)out, rows, inter);
+    if (vec) silu_and_mul_kernel<float, true><<<grid, block, 0, stream>>>((const float*)gu, bias, (float*)out, rows, inter);
+    else silu_and_mul_kernel<float, false><<<grid, block, 0, stream>>>((const float*)gu, bias, (float*)out, rows, inter);
   }
   ME_LAUNCH_CHECK();
   return 0;

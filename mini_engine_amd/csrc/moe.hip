@@ -8,10 +8,13 @@
 //                  a constant, divided by their sum or not (`RouteRule`)
 //   moe_sort       (token, choice) pairs ordered by expert, cut into tiles of 16, 64 or 128 rows that never span two experts
 //   moe_gate_up    per tile: silu(x W_gate^T) * (x W_up^T) of the tile's expert, token rows gathered through the order;
-//                  or, for experts without a gate, relu(x W_up^T)^2
+//                  or, for experts without a gate, relu(x W_up^T)^2; or g sigmoid(alpha g) (u + 1) with the gate g cut at
+//                  limit from above and u at both sides
 //   moe_down       per tile: the expert's down product, times the pair's weight, into float32 [top, T, hidden]: one
 //                  partial sum per choice, for a consumer that adds them (no atomics: the result does not depend on
-//                  what else is in the batch)
+//                  what else is in the batch). The router may know more experts than there are weights: an expert behind
+//                  the last one with weights hands its input row on (an identity expert), times the pair's weight. The
+//                  pairs of all of them form one class behind the last expert's, whose tiles copy rows
 //   moe_*_simple   the same two products with one wave per output element: the float32 path, and sizes whose rows
 //                  are not whole 16-byte pieces
 //
@@ -269,12 +272,13 @@ extern "C" int me_moe_route(const void* x, int64_t ldx, int dtype, const float* 
 }
 
 // ------------------------------------------------------------------ pairs by expert
-// One workgroup. order[p']: the pair at sorted place p'; offsets[e]: where expert e's pairs begin; tile_expert / tile_row:
-// expert and first sorted place of every tile of up to `tile_rows` pairs (expert -1: a tile nobody needs).
+// One workgroup. E: classes of pairs: the experts with weights, and one more for all pairs of identity experts (ids from
+// E - 1 on) where the router has any. order[p']: the pair at sorted place p'; offsets[e]: where class e's pairs begin;
+// tile_expert / tile_row: expert and first sorted place of every tile of up to `tile_rows` pairs (expert -1: a tile nobody needs).
 // With `logits` (few tokens) the workgroup first makes the choice itself, a wave per token in turn, and writes ids and
 // weights: the launch of `moe_select` is saved.
 __global__ void __launch_bounds__(1024)
-moe_sort_kernel(int32_t* __restrict__ ids, int P, int E, int max_tiles, int tile_rows, int32_t* __restrict__ order,
+moe_sort_kernel(int32_t* __restrict__ ids, int P, int routed, int E, int max_tiles, int tile_rows, int32_t* __restrict__ order,
                 int32_t* __restrict__ offsets, int32_t* __restrict__ tile_expert, int32_t* __restrict__ tile_row,
                 const float* __restrict__ logits, float* __restrict__ weights, RouteRule rule) {
   __shared__ int count[MOE_MAX_EXPERTS], begin[MOE_MAX_EXPERTS + 1], tile_at[MOE_MAX_EXPERTS + 1], cursor[MOE_MAX_EXPERTS];
@@ -282,12 +286,12 @@ moe_sort_kernel(int32_t* __restrict__ ids, int P, int E, int max_tiles, int tile
   for (int e = threadIdx.x; e < E; e += blockDim.x) { count[e] = 0; cursor[e] = 0; }
   if (logits) {
     const int wave = threadIdx.x >> 6, waves = blockDim.x >> 6;
-    float* s = reinterpret_cast<float*>(route_lds) + (size_t)wave * (2 * E + rule.group_count);
-    for (int t = wave; t < P / rule.top; t += waves) select_token(logits, t, E, rule, s, s + E, s + 2 * E, ids, weights);
+    float* s = reinterpret_cast<float*>(route_lds) + (size_t)wave * (2 * routed + rule.group_count);
+    for (int t = wave; t < P / rule.top; t += waves) select_token(logits, t, routed, rule, s, s + routed, s + 2 * routed, ids, weights);
     __threadfence_block();
   }
   __syncthreads();
-  for (int p = threadIdx.x; p < P; p += blockDim.x) atomicAdd(&count[ids[p]], 1);
+  for (int p = threadIdx.x; p < P; p += blockDim.x) atomicAdd(&count[min(ids[p], E - 1)], 1);
   __syncthreads();
   if (threadIdx.x == 0) {
     int at = 0, tiles = 0;
@@ -301,7 +305,7 @@ moe_sort_kernel(int32_t* __restrict__ ids, int P, int E, int max_tiles, int tile
   __syncthreads();
   for (int e = threadIdx.x; e <= E; e += blockDim.x) offsets[e] = begin[e];
   for (int p = threadIdx.x; p < P; p += blockDim.x) {
-    const int e = ids[p];
+    const int e = min(ids[p], E - 1);
     order[begin[e] + atomicAdd(&cursor[e], 1)] = p;
   }
   for (int e = threadIdx.x; e < E; e += blockDim.x)
@@ -312,26 +316,29 @@ moe_sort_kernel(int32_t* __restrict__ ids, int P, int E, int max_tiles, int tile
   for (int i = tile_at[E] + threadIdx.x; i < max_tiles; i += blockDim.x) { tile_expert[i] = -1; tile_row[i] = 0; }
 }
 
-// logits: null, or the router's float32 [T, E] with the choice still to be made (`me_moe_route` with select 0): ids and
+// routed: how many experts the router chooses among, the last `identity` of them without weights.
+// logits: null, or the router's float32 [T, routed] with the choice still to be made (`me_moe_route` with select 0): ids and
 // weights are then written here (`moe_sort_chooses` says when that fits).
-extern "C" int me_moe_sort(int32_t* ids, int64_t P, int E, int max_tiles, int tile_rows, int32_t* order, int32_t* offsets,
+extern "C" int me_moe_sort(int32_t* ids, int64_t P, int routed, int identity, int max_tiles, int tile_rows, int32_t* order, int32_t* offsets,
                            int32_t* tile_expert, int32_t* tile_row, const float* logits, float* weights, int top, int group_count,
                            int group_keep, int group_top, int sigmoid, int normalise, float scale, const float* correction,
                            hipStream_t stream) {
   if (P == 0) return 0;
-  ME_CHECK(E >= 1 && E <= MOE_MAX_EXPERTS && P < (1ll << 30), "moe_sort: %d experts, %lld pairs", E, (long long)P);
+  ME_CHECK(identity >= 0 && identity < routed && routed <= MOE_MAX_EXPERTS && P < (1ll << 30), "moe_sort: %d experts (%d of them without weights), %lld pairs",
+           routed, identity, (long long)P);
+  const int E = routed - identity + (identity > 0 ? 1 : 0);
   ME_CHECK(tile_rows == 16 || tile_rows == 64 || tile_rows == 128, "moe_sort: tiles of 16, 64 or 128 rows");
   ME_CHECK(max_tiles >= P / tile_rows + (P < E ? P : E), "moe_sort: %d tiles cannot hold every expert's last tile", max_tiles);
   size_t lds = 0;
   RouteRule rule;
-  route_rule(rule, E, top, group_count, group_keep, group_top, sigmoid, normalise, scale, correction);
+  route_rule(rule, routed, top, group_count, group_keep, group_top, sigmoid, normalise, scale, correction);
   if (logits) {
-    ME_CHECK(weights && route_rule(rule, E, top, group_count, group_keep, group_top, sigmoid, normalise, scale, correction) && P % top == 0,
+    ME_CHECK(weights && route_rule(rule, routed, top, group_count, group_keep, group_top, sigmoid, normalise, scale, correction) && P % top == 0,
              "moe_sort: bad routing sizes");
-    lds = (size_t)16 * (2 * E + group_count) * 4;
-    ME_CHECK(lds <= 40 * 1024, "moe_sort: %d experts are too many to choose here", E);
+    lds = (size_t)16 * (2 * routed + group_count) * 4;
+    ME_CHECK(lds <= 40 * 1024, "moe_sort: %d experts are too many to choose here", routed);
   }
-  moe_sort_kernel<<<dim3(1), dim3(1024), lds, stream>>>(ids, (int)P, E, max_tiles, tile_rows, order, offsets, tile_expert, tile_row,
+  moe_sort_kernel<<<dim3(1), dim3(1024), lds, stream>>>(ids, (int)P, routed, E, max_tiles, tile_rows, order, offsets, tile_expert, tile_row,
                                                         logits, weights, rule);
   ME_LAUNCH_CHECK();
   return 0;
@@ -342,15 +349,43 @@ extern "C" int me_moe_sort(int32_t* ids, int64_t P, int E, int max_tiles, int ti
 // sub-tiles of TM/2 x TN/2, each MJ x MI matrix-instruction tiles of 16 x 16: 64 x 64 (2 x 2 per wave) for a few
 // hundred rows per expert, 128 x 128 (4 x 4 per wave: twice the products per operand read from LDS) beyond.
 // ACT 1: the tile's weight rows are TN/2 gate rows and the TN/2 up rows that go with them; the result is silu(gate) * up.
+// ACT 3: the same rows under `glu` (`ClampedGate`). Tiles of class `experts` (identity experts) have no weights: ACT 0 copies
+// their token rows from x_in, the others leave.
 // ACT 2: experts without a gate: the tile's TN weight rows are up rows and the result is relu(up)^2. ACT 0: the down product,
 // times the pair's weight, into the pair's partial sum.
 //   x: [T, K] token rows (ACT 1, 2) or [P, K] rows at sorted places (ACT 0); w: [E * rows_per_expert, K]
+struct ClampedGate { float limit, alpha; };      // g = min(gate, limit), u = clamp(up, -limit, limit): g sigmoid(alpha g) (u + 1)
+
+template <int ACT>
+__device__ __forceinline__ float gated_value(float gate, float up, const ClampedGate& glu) {
+  if constexpr (ACT == 3) {
+    const float g = fminf(gate, glu.limit), u = fminf(fmaxf(up, -glu.limit), glu.limit);
+    return g / (1.f + __expf(-glu.alpha * g)) * (u + 1.f);
+  } else {
+    return gate / (1.f + __expf(-gate)) * up;
+  }
+}
+
+// Rows [row0, row0 + rows) of the identity experts' pairs, features [n0, n1): the token's row times the pair's weight.
+__device__ __forceinline__ void copy_identity_rows(const bf16_t* __restrict__ x_in, int64_t ld_in, const int32_t* __restrict__ order,
+                                                   const float* __restrict__ pair_weight, float* __restrict__ out, int64_t T, int top,
+                                                   int N, int row0, int rows, int n0, int n1) {
+  const int width = n1 - n0;
+  for (int i = threadIdx.x; i < rows * width; i += blockDim.x) {
+    const int r = i / width, f = n0 + i - r * width;
+    const int pair = order[row0 + r];
+    const int64_t tok = pair / top, choice = pair - tok * top;
+    out[(choice * T + tok) * N + f] = pair_weight[pair] * static_cast<float>(x_in[tok * ld_in + f]);
+  }
+}
+
 template <int ACT, int TM, int TN>
 __global__ void __launch_bounds__(256)
 moe_tile_kernel(const bf16_t* __restrict__ x, int64_t ldx, const bf16_t* __restrict__ w, int64_t ldw,
                 const int32_t* __restrict__ order, const int32_t* __restrict__ offsets, const int32_t* __restrict__ tile_expert,
                 const int32_t* __restrict__ tile_row, const float* __restrict__ pair_weight, void* __restrict__ out,
-                int64_t T, int top, int N, int K) {
+                int64_t T, int top, int N, int K, int experts, ClampedGate glu, const bf16_t* __restrict__ x_in, int64_t ld_in) {
+  constexpr bool GATED = ACT == 1 || ACT == 3;
   constexpr int ROWS = TM + TN, NQ = ROWS / 32, MI = TN / 32, MJ = TM / 32, STAGE = ROWS * 128;
   extern __shared__ __align__(16) unsigned char lds[];        // [2][STAGE]
   const int e = tile_expert[blockIdx.y];
@@ -359,7 +394,11 @@ moe_tile_kernel(const bf16_t* __restrict__ x, int64_t ldx, const bf16_t* __restr
   const int rows = min(TM, offsets[e + 1] - row0);
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int n = lane & 15, g = lane >> 4;
-  const int n0 = blockIdx.x * (ACT == 1 ? TN / 2 : TN);      // first feature of the tile
+  const int n0 = blockIdx.x * (GATED ? TN / 2 : TN);      // first feature of the tile
+  if (e >= experts) {
+    if constexpr (ACT == 0) copy_identity_rows(x_in, ld_in, order, pair_weight, (float*)out, T, top, N, row0, rows, n0, min(n0 + TN, N));
+    return;
+  }
   // the pieces this thread brings per stage: rows tid / 8 + 32 q, piece tid % 8
   const bf16_t* src[NQ];
   uint32_t dst[NQ];
@@ -374,7 +413,7 @@ moe_tile_kernel(const bf16_t* __restrict__ x, int64_t ldx, const bf16_t* __restr
     } else {
       const int wr = R - TM;
       int64_t row;
-      if (ACT == 1) row = (int64_t)e * 2 * N + (wr < TN / 2 ? min(n0 + wr, N - 1) : N + min(n0 + wr - TN / 2, N - 1));
+      if (GATED) row = (int64_t)e * 2 * N + (wr < TN / 2 ? min(n0 + wr, N - 1) : N + min(n0 + wr - TN / 2, N - 1));
       else row = (int64_t)e * N + min(n0 + wr, N - 1);
       src[q] = w + row * ldw;
     }
@@ -396,7 +435,7 @@ moe_tile_kernel(const bf16_t* __restrict__ x, int64_t ldx, const bf16_t* __restr
   int a_row[MI];
 #pragma unroll
   for (int i = 0; i < MI; ++i)
-    a_row[i] = TM + (ACT == 1 ? (i < MI / 2 ? wn * (TN / 4) + 16 * i : TN / 2 + wn * (TN / 4) + 16 * (i - MI / 2)) : wn * (TN / 2) + 16 * i) + n;
+    a_row[i] = TM + (GATED ? (i < MI / 2 ? wn * (TN / 4) + 16 * i : TN / 2 + wn * (TN / 4) + 16 * (i - MI / 2)) : wn * (TN / 2) + 16 * i) + n;
   f32x4 acc[MI][MJ];
 #pragma unroll
   for (int i = 0; i < MI; ++i)
@@ -450,7 +489,7 @@ moe_tile_kernel(const bf16_t* __restrict__ x, int64_t ldx, const bf16_t* __restr
             if (f + q < N) o[f + q] = r[q];
         }
       }
-    } else if constexpr (ACT == 1) {
+    } else if constexpr (GATED) {
       bf16_t* o = (bf16_t*)out + (int64_t)p * N;
 #pragma unroll
       for (int i = 0; i < MI / 2; ++i) {
@@ -458,8 +497,7 @@ moe_tile_kernel(const bf16_t* __restrict__ x, int64_t ldx, const bf16_t* __restr
         bf16x4 r;
 #pragma unroll
         for (int q = 0; q < 4; ++q) {
-          const float gate = acc[i][j][q];
-          r[q] = from_f32<bf16_t>(gate / (1.f + __expf(-gate)) * acc[i + MI / 2][j][q]);
+          r[q] = from_f32<bf16_t>(gated_value<ACT>(acc[i][j][q], acc[i + MI / 2][j][q], glu));
         }
         if (f + 3 < N && (N & 3) == 0) {
           *reinterpret_cast<bf16x4*>(o + f) = r;          // 4 neighbours, 8 bytes
@@ -492,7 +530,8 @@ moe_tile_kernel(const bf16_t* __restrict__ x, int64_t ldx, const bf16_t* __restr
 template <int ACT, int TM>
 static int launch_moe_tile(const bf16_t* x, int64_t ldx, const bf16_t* w, int64_t ldw, const int32_t* order, const int32_t* offsets,
                            const int32_t* tile_expert, const int32_t* tile_row, const float* pair_weight, void* out, int64_t T,
-                           int top, int N, int K, int max_tiles, hipStream_t stream) {
+                           int top, int N, int K, int max_tiles, int experts, ClampedGate glu, const bf16_t* x_in, int64_t ld_in,
+                           hipStream_t stream) {
   constexpr int TN = TM;
   const size_t lds = 2 * (size_t)(TM + TN) * 128;
   static bool allowed = false;                     // 64 KB of LDS for the large tiles: more than a kernel may have unasked
@@ -501,9 +540,9 @@ static int launch_moe_tile(const bf16_t* x, int64_t ldx, const bf16_t* w, int64_
     ME_CHECK(err == hipSuccess, "routed experts: cannot get %zu bytes of LDS: %s", lds, hipGetErrorString(err));
     allowed = true;
   }
-  const int per = ACT == 1 ? TN / 2 : TN;
+  const int per = ACT == 1 || ACT == 3 ? TN / 2 : TN;
   moe_tile_kernel<ACT, TM, TN><<<dim3((unsigned)((N + per - 1) / per), (unsigned)max_tiles), dim3(256), lds, stream>>>(
-      x, ldx, w, ldw, order, offsets, tile_expert, tile_row, pair_weight, out, T, top, N, K);
+      x, ldx, w, ldw, order, offsets, tile_expert, tile_row, pair_weight, out, T, top, N, K, experts, glu, x_in, ld_in);
   ME_LAUNCH_CHECK();
   return 0;
 }
@@ -517,8 +556,10 @@ template <int ACT>
 __global__ void __launch_bounds__(256)
 moe_skinny_kernel(const bf16_t* __restrict__ x, int64_t ldx, const bf16_t* __restrict__ w, const int32_t* __restrict__ order,
                   const int32_t* __restrict__ offsets, const int32_t* __restrict__ tile_expert, const int32_t* __restrict__ tile_row,
-                  const float* __restrict__ pair_weight, void* __restrict__ out, int64_t T, int top, int N, int K) {
-  __shared__ float part[4][ACT == 1 ? 2 : 1][64][4];
+                  const float* __restrict__ pair_weight, void* __restrict__ out, int64_t T, int top, int N, int K, int experts,
+                  ClampedGate glu, const bf16_t* __restrict__ x_in, int64_t ld_in) {
+  constexpr bool GATED = ACT == 1 || ACT == 3;
+  __shared__ float part[4][GATED ? 2 : 1][64][4];
   const int e = tile_expert[blockIdx.y];
   if (e < 0) return;
   const int row0 = tile_row[blockIdx.y];
@@ -526,11 +567,15 @@ moe_skinny_kernel(const bf16_t* __restrict__ x, int64_t ldx, const bf16_t* __res
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int n = lane & 15, g = lane >> 4;
   const int n0 = blockIdx.x * 16;
+  if (e >= experts) {
+    if constexpr (ACT == 0) copy_identity_rows(x_in, ld_in, order, pair_weight, (float*)out, T, top, N, row0, rows, n0, min(n0 + 16, N));
+    return;
+  }
   const int p = row0 + min(n, rows - 1);
   const bf16_t* xr = x + (ACT ? (int64_t)(order[p] / top) : (int64_t)p) * ldx + 8 * g;
   const int f = min(n0 + n, N - 1);
-  const bf16_t* wr = w + ((int64_t)e * (ACT == 1 ? 2 : 1) * N + f) * K + 8 * g;
-  const bf16_t* ur = wr + (int64_t)N * K;            // ACT 1: the up row of the same feature
+  const bf16_t* wr = w + ((int64_t)e * (GATED ? 2 : 1) * N + f) * K + 8 * g;
+  const bf16_t* ur = wr + (int64_t)N * K;            // gated: the up row of the same feature
   f32x4 acc_g = {0.f, 0.f, 0.f, 0.f}, acc_u = {0.f, 0.f, 0.f, 0.f};
   const bf16x8 zero = {0, 0, 0, 0, 0, 0, 0, 0};
   for (int k0 = wave * 32; k0 < K; k0 += 4 * 128) {
@@ -540,19 +585,19 @@ moe_skinny_kernel(const bf16_t* __restrict__ x, int64_t ldx, const bf16_t* __res
       const int k = k0 + i * 128;
       const bool in = k + 8 * g < K;
       a[i] = in ? *reinterpret_cast<const bf16x8*>(wr + k) : zero;
-      if (ACT == 1) u[i] = in ? *reinterpret_cast<const bf16x8*>(ur + k) : zero;
+      if (GATED) u[i] = in ? *reinterpret_cast<const bf16x8*>(ur + k) : zero;
       b[i] = in ? *reinterpret_cast<const bf16x8*>(xr + k) : zero;
     }
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       acc_g = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[i], b[i], acc_g, 0, 0, 0);
-      if (ACT == 1) acc_u = __builtin_amdgcn_mfma_f32_16x16x32_bf16(u[i], b[i], acc_u, 0, 0, 0);
+      if (GATED) acc_u = __builtin_amdgcn_mfma_f32_16x16x32_bf16(u[i], b[i], acc_u, 0, 0, 0);
     }
   }
 #pragma unroll
   for (int q = 0; q < 4; ++q) {
     part[wave][0][lane][q] = acc_g[q];
-    if constexpr (ACT == 1) part[wave][1][lane][q] = acc_u[q];
+    if constexpr (GATED) part[wave][1][lane][q] = acc_u[q];
   }
   __syncthreads();
   if (wave != 0 || n >= rows) return;
@@ -562,18 +607,18 @@ moe_skinny_kernel(const bf16_t* __restrict__ x, int64_t ldx, const bf16_t* __res
 #pragma unroll
   for (int q = 0; q < 4; ++q) {
     sg[q] = part[0][0][lane][q] + part[1][0][lane][q] + part[2][0][lane][q] + part[3][0][lane][q];
-    if constexpr (ACT == 1) su[q] = part[0][1][lane][q] + part[1][1][lane][q] + part[2][1][lane][q] + part[3][1][lane][q];
+    if constexpr (GATED) su[q] = part[0][1][lane][q] + part[1][1][lane][q] + part[2][1][lane][q] + part[3][1][lane][q];
   }
   if constexpr (ACT == 2) {
     bf16_t* o = (bf16_t*)out + (int64_t)pr * N;
 #pragma unroll
     for (int q = 0; q < 4; ++q)
       if (n0 + 4 * g + q < N) { const float up = fmaxf(sg[q], 0.f); o[n0 + 4 * g + q] = from_f32<bf16_t>(up * up); }
-  } else if constexpr (ACT == 1) {
+  } else if constexpr (GATED) {
     bf16_t* o = (bf16_t*)out + (int64_t)pr * N;
 #pragma unroll
     for (int q = 0; q < 4; ++q)
-      if (n0 + 4 * g + q < N) o[n0 + 4 * g + q] = from_f32<bf16_t>(sg[q] / (1.f + __expf(-sg[q])) * su[q]);
+      if (n0 + 4 * g + q < N) o[n0 + 4 * g + q] = from_f32<bf16_t>(gated_value<ACT>(sg[q], su[q], glu));
   } else {
     const int pair = order[pr];
     const int64_t tok = pair / top, choice = pair - tok * top;
@@ -585,64 +630,67 @@ moe_skinny_kernel(const bf16_t* __restrict__ x, int64_t ldx, const bf16_t* __res
   }
 }
 
-// act: bfloat16 [P, F] at sorted places; gate_up: [E * 2 F, K] (an expert's gate rows, then its up rows), or with `gated` 0
-// [E * F, K] (up rows only: the result is relu(up)^2)
-// tile_rows: 16 (tiles of `moe_sort` with 16 rows: the skinny kernel) or 64
+// act: bfloat16 [P, F] at sorted places; gate_up: [experts * 2 F, K] (an expert's gate rows, then its up rows), or with `gated`
+// 0 [experts * F, K] (up rows only: the result is relu(up)^2). limit > 0: a clamped gate (`ClampedGate`) in place of silu.
+// Tiles of class `experts` (identity experts) write nothing here.
+// tile_rows: 16 (tiles of `moe_sort` with 16 rows: the skinny kernel), 64 or 128
 extern "C" int me_moe_gate_up(const void* x, int64_t ldx, const void* gate_up, const int32_t* order, const int32_t* offsets,
                               const int32_t* tile_expert, const int32_t* tile_row, void* act, int64_t T, int top, int F, int K,
-                              int max_tiles, int tile_rows, int gated, hipStream_t stream) {
+                              int max_tiles, int tile_rows, int gated, int experts, float limit, float alpha, hipStream_t stream) {
   if (T == 0) return 0;
   ME_CHECK(K % 8 == 0 && ldx % 8 == 0 && reinterpret_cast<uintptr_t>(x) % 16 == 0 && reinterpret_cast<uintptr_t>(gate_up) % 16 == 0,
            "moe_gate_up: rows must be whole 16-byte pieces (K = %d)", K);
-  ME_CHECK(max_tiles >= 1 && max_tiles <= 65535 && F >= 1, "moe_gate_up: %d tiles", max_tiles);
-  if (!gated) {
-    if (tile_rows == 16) {
-      moe_skinny_kernel<2><<<dim3((unsigned)((F + 15) / 16), (unsigned)max_tiles), dim3(256), 0, stream>>>(
-          (const bf16_t*)x, ldx, (const bf16_t*)gate_up, order, offsets, tile_expert, tile_row, nullptr, act, T, top, F, K);
-      ME_LAUNCH_CHECK();
-      return 0;
-    }
-    if (tile_rows == 128)
-      return launch_moe_tile<2, 128>((const bf16_t*)x, ldx, (const bf16_t*)gate_up, (int64_t)K, order, offsets, tile_expert, tile_row,
-                                     nullptr, act, T, top, F, K, max_tiles, stream);
-    ME_CHECK(tile_rows == 64, "moe_gate_up: tiles of 16, 64 or 128 rows");
-    return launch_moe_tile<2, 64>((const bf16_t*)x, ldx, (const bf16_t*)gate_up, (int64_t)K, order, offsets, tile_expert, tile_row,
-                                  nullptr, act, T, top, F, K, max_tiles, stream);
-  }
+  ME_CHECK(max_tiles >= 1 && max_tiles <= 65535 && F >= 1 && experts >= 1, "moe_gate_up: %d tiles", max_tiles);
+  ME_CHECK(limit <= 0.f || gated, "moe_gate_up: only a gate can be clamped");
+  const ClampedGate glu{limit, alpha};
+  const int kind = !gated ? 2 : (limit > 0.f ? 3 : 1);
   if (tile_rows == 16) {
-    moe_skinny_kernel<1><<<dim3((unsigned)((F + 15) / 16), (unsigned)max_tiles), dim3(256), 0, stream>>>(
-        (const bf16_t*)x, ldx, (const bf16_t*)gate_up, order, offsets, tile_expert, tile_row, nullptr, act, T, top, F, K);
+    const dim3 grid((unsigned)((F + 15) / 16), (unsigned)max_tiles), block(256);
+#define SKINNY(A) moe_skinny_kernel<A><<<grid, block, 0, stream>>>((const bf16_t*)x, ldx, (const bf16_t*)gate_up, order, offsets, tile_expert, \
+                                                                   tile_row, nullptr, act, T, top, F, K, experts, glu, nullptr, 0)
+    if (kind == 1) SKINNY(1); else if (kind == 2) SKINNY(2); else SKINNY(3);
+#undef SKINNY
     ME_LAUNCH_CHECK();
     return 0;
   }
-  if (tile_rows == 128)
-    return launch_moe_tile<1, 128>((const bf16_t*)x, ldx, (const bf16_t*)gate_up, (int64_t)K, order, offsets, tile_expert, tile_row,
-                                      nullptr, act, T, top, F, K, max_tiles, stream);
-  ME_CHECK(tile_rows == 64, "moe_gate_up: tiles of 16, 64 or 128 rows");
-  return launch_moe_tile<1, 64>((const bf16_t*)x, ldx, (const bf16_t*)gate_up, (int64_t)K, order, offsets, tile_expert, tile_row,
-                                   nullptr, act, T, top, F, K, max_tiles, stream);
+  ME_CHECK(tile_rows == 64 || tile_rows == 128, "moe_gate_up: tiles of 16, 64 or 128 rows");
+#define TILE(A, M) return launch_moe_tile<A, M>((const bf16_t*)x, ldx, (const bf16_t*)gate_up, (int64_t)K, order, offsets, tile_expert, tile_row, \
+                                                nullptr, act, T, top, F, K, max_tiles, experts, glu, nullptr, 0, stream)
+  if (tile_rows == 128) {
+    if (kind == 1) TILE(1, 128);
+    if (kind == 2) TILE(2, 128);
+    TILE(3, 128);
+  }
+  if (kind == 1) TILE(1, 64);
+  if (kind == 2) TILE(2, 64);
+  TILE(3, 64);
+#undef TILE
 }
 
-// out: float32 [top, T, N]; down: [E * N, F]
+// out: float32 [top, T, N]; down: [experts * N, F]; x_in: the token rows [T, N], for the tiles of identity experts (class
+// `experts`; null where there are none)
 extern "C" int me_moe_down(const void* act, const void* down, const int32_t* order, const int32_t* offsets,
                            const int32_t* tile_expert, const int32_t* tile_row, const float* pair_weight, float* out, int64_t T,
-                           int top, int N, int F, int max_tiles, int tile_rows, hipStream_t stream) {
+                           int top, int N, int F, int max_tiles, int tile_rows, int experts, const void* x_in, int64_t ld_in,
+                           hipStream_t stream) {
   if (T == 0) return 0;
   ME_CHECK(F % 8 == 0 && reinterpret_cast<uintptr_t>(act) % 16 == 0 && reinterpret_cast<uintptr_t>(down) % 16 == 0,
            "moe_down: rows must be whole 16-byte pieces (F = %d)", F);
-  ME_CHECK(max_tiles >= 1 && max_tiles <= 65535 && N >= 1, "moe_down: %d tiles", max_tiles);
+  ME_CHECK(max_tiles >= 1 && max_tiles <= 65535 && N >= 1 && experts >= 1, "moe_down: %d tiles", max_tiles);
+  const ClampedGate none{0.f, 0.f};
   if (tile_rows == 16) {
     moe_skinny_kernel<0><<<dim3((unsigned)((N + 15) / 16), (unsigned)max_tiles), dim3(256), 0, stream>>>(
-        (const bf16_t*)act, (int64_t)F, (const bf16_t*)down, order, offsets, tile_expert, tile_row, pair_weight, out, T, top, N, F);
+        (const bf16_t*)act, (int64_t)F, (const bf16_t*)down, order, offsets, tile_expert, tile_row, pair_weight, out, T, top, N, F,
+        experts, none, (const bf16_t*)x_in, ld_in);
     ME_LAUNCH_CHECK();
     return 0;
   }
   if (tile_rows == 128)
     return launch_moe_tile<0, 128>((const bf16_t*)act, (int64_t)F, (const bf16_t*)down, (int64_t)F, order, offsets, tile_expert,
-                                       tile_row, pair_weight, out, T, top, N, F, max_tiles, stream);
+                                       tile_row, pair_weight, out, T, top, N, F, max_tiles, experts, none, (const bf16_t*)x_in, ld_in, stream);
   ME_CHECK(tile_rows == 64, "moe_down: tiles of 16, 64 or 128 rows");
   return launch_moe_tile<0, 64>((const bf16_t*)act, (int64_t)F, (const bf16_t*)down, (int64_t)F, order, offsets, tile_expert,
-                                    tile_row, pair_weight, out, T, top, N, F, max_tiles, stream);
+                                    tile_row, pair_weight, out, T, top, N, F, max_tiles, experts, none, (const bf16_t*)x_in, ld_in, stream);
 }
 
 // ------------------------------------------------------------------ one wave per output element
@@ -650,12 +698,13 @@ extern "C" int me_moe_down(const void* act, const void* down, const int32_t* ord
 template <typename TX, bool GATED>
 __global__ void __launch_bounds__(256)
 moe_gate_up_simple_kernel(const TX* __restrict__ x, int64_t ldx, const TX* __restrict__ gate_up, const int32_t* __restrict__ ids,
-                          TX* __restrict__ act, int64_t P, int top, int F, int K) {
+                          TX* __restrict__ act, int64_t P, int top, int F, int K, int experts, ClampedGate glu) {
   const int lane = threadIdx.x & 63;
   const int64_t at = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (at >= P * F) return;
   const int64_t pair = at / F;
   const int f = (int)(at - pair * F);
+  if (ids[pair] >= experts) return;                    // an identity expert has no weights
   const TX* xr = x + (pair / top) * ldx;
   const TX* gr = gate_up + ((int64_t)ids[pair] * (GATED ? 2 : 1) * F + f) * K;
   const TX* ur = gr + (int64_t)F * K;
@@ -668,48 +717,64 @@ moe_gate_up_simple_kernel(const TX* __restrict__ x, int64_t ldx, const TX* __res
   sg = wave_sum(sg);
   if (GATED) su = wave_sum(su);
   const float up = fmaxf(sg, 0.f);
-  if (lane == 0) act[at] = from_f32<TX>(GATED ? sg / (1.f + expf(-sg)) * su : up * up);
+  float v = up * up;
+  if (GATED) {
+    if (glu.limit > 0.f) {
+      const float g = fminf(sg, glu.limit), u = fminf(fmaxf(su, -glu.limit), glu.limit);
+      v = g / (1.f + expf(-glu.alpha * g)) * (u + 1.f);
+    } else {
+      v = sg / (1.f + expf(-sg)) * su;
+    }
+  }
+  if (lane == 0) act[at] = from_f32<TX>(v);
 }
 
 template <typename TX>
 __global__ void __launch_bounds__(256)
 moe_down_simple_kernel(const TX* __restrict__ act, const TX* __restrict__ down, const int32_t* __restrict__ ids,
-                       const float* __restrict__ pair_weight, float* __restrict__ out, int64_t T, int top, int N, int F) {
+                       const float* __restrict__ pair_weight, float* __restrict__ out, int64_t T, int top, int N, int F, int experts,
+                       const TX* __restrict__ x, int64_t ldx) {
   const int lane = threadIdx.x & 63;
   const int64_t at = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (at >= T * top * N) return;
   const int64_t pair = at / N;
   const int f = (int)(at - pair * N);
+  const int64_t tok = pair / top, choice = pair - tok * top;
+  if (ids[pair] >= experts) {                          // an identity expert hands its input on
+    if (lane == 0) out[(choice * T + tok) * N + f] = to_f32<TX>(x[tok * ldx + f]) * pair_weight[pair];
+    return;
+  }
   const TX* ar = act + pair * F;
   const TX* dr = down + ((int64_t)ids[pair] * N + f) * F;
   float s = 0.f;
   for (int k = lane; k < F; k += 64) s += to_f32<TX>(ar[k]) * to_f32<TX>(dr[k]);
   s = wave_sum(s);
-  const int64_t tok = pair / top, choice = pair - tok * top;
   if (lane == 0) out[(choice * T + tok) * N + f] = s * pair_weight[pair];
 }
 
 extern "C" int me_moe_experts_simple(const void* x, int64_t ldx, int dtype, const void* gate_up, const void* down,
                                      const int32_t* ids, const float* pair_weight, void* act, float* out, int64_t T, int top,
-                                     int N, int F, int K, int gated, hipStream_t stream) {
+                                     int N, int F, int K, int gated, int experts, float limit, float alpha, hipStream_t stream) {
   if (T == 0) return 0;
+  ME_CHECK(experts >= 1 && (limit <= 0.f || gated), "moe_experts_simple: only a gate can be clamped");
+  const ClampedGate glu{limit, alpha};
   const int64_t P = T * top;
   const int64_t g1 = (P * F + 3) / 4, g2 = (P * N + 3) / 4;
   ME_CHECK(g1 < (1ll << 31) && g2 < (1ll << 31), "moe_experts_simple: too many outputs");
   if (dtype == ME_F32) {
     if (gated) moe_gate_up_simple_kernel<float, true><<<dim3((unsigned)g1), dim3(256), 0, stream>>>((const float*)x, ldx, (const float*)gate_up, ids,
-                                                                                                    (float*)act, P, top, F, K);
+                                                                                                    (float*)act, P, top, F, K, experts, glu);
     else moe_gate_up_simple_kernel<float, false><<<dim3((unsigned)g1), dim3(256), 0, stream>>>((const float*)x, ldx, (const float*)gate_up, ids,
-                                                                                               (float*)act, P, top, F, K);
+                                                                                               (float*)act, P, top, F, K, experts, glu);
     moe_down_simple_kernel<float><<<dim3((unsigned)g2), dim3(256), 0, stream>>>((const float*)act, (const float*)down, ids, pair_weight,
-                                                                                out, T, top, N, F);
+                                                                                out, T, top, N, F, experts, (const float*)x, ldx);
   } else {
     if (gated) moe_gate_up_simple_kernel<bf16_t, true><<<dim3((unsigned)g1), dim3(256), 0, stream>>>((const bf16_t*)x, ldx, (const bf16_t*)gate_up, ids,
-                                                                                                     (bf16_t*)act, P, top, F, K);
+                                                                                                     (bf16_t*)act, P, top, F, K, experts, glu);
     else moe_gate_up_simple_kernel<bf16_t, false><<<dim3((unsigned)g1), dim3(256), 0, stream>>>((const bf16_t*)x, ldx, (const bf16_t*)gate_up, ids,
-                                                                                                (bf16_t*)act, P, top, F, K);
+                                                                                                (bf16_t*)act, P, top, F, K, experts, glu);
     moe_down_simple_kernel<bf16_t><<<dim3((unsigned)g2), dim3(256), 0, stream>>>((const bf16_t*)act, (const bf16_t*)down, ids,
-                                                                                 pair_weight, out, T, top, N, F);
+                                                                                 pair_weight, out, T, top, N, F, experts, (const bf16_t*)x, ldx);
   }
   ME_LAUNCH_CHECK();
   return 0;

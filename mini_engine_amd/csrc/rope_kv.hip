@@ -58,7 +58,7 @@ qk_norm_rope_store_kernel(T* __restrict__ qkv, int64_t row_stride, const float* 
                           const float* __restrict__ table,  // [P, D/2, 2] cos,sin or null
                           const int32_t* __restrict__ positions, const int32_t* __restrict__ slots,
                           T* __restrict__ k_cache, T* __restrict__ v_cache, int Hq, int Hkv, int D,
-                          int page, int store, int64_t num_tokens) {
+                          int page, int store, int v_head, int64_t num_tokens) {
   const int64_t t = blockIdx.x;
   const int lane = threadIdx.x & 63;
   const int head = blockIdx.y * 4 + (threadIdx.x >> 6);
@@ -70,7 +70,9 @@ qk_norm_rope_store_kernel(T* __restrict__ qkv, int64_t row_stride, const float* 
   const int half = D >> 1;
 
   if (head >= Hq + Hkv) {  // a value head: copy into the transposed page
-    store_value_head<T>(row, row_stride, t, num_tokens, slots, v_cache, Hkv, head - Hq - Hkv, D, page, lane);
+    const int kvh = head - Hq - Hkv;
+    store_value_head<T>(qkv + t * row_stride + (int64_t)(v_head + kvh) * D, row_stride, t, num_tokens, slots, v_cache, Hkv, kvh, D,
+                        page, lane);
     return;
   }
 
@@ -157,14 +159,14 @@ qk_norm_rope_store_vec_kernel(T* __restrict__ qkv, int64_t row_stride, const flo
                               const float* __restrict__ k_w, float eps, const float* __restrict__ table,
                               const int32_t* __restrict__ positions, const int32_t* __restrict__ slots,
                               T* __restrict__ k_cache, T* __restrict__ v_cache, int Hq, int Hkv, int D, int page,
-                              int store, int64_t num_tokens, int qk_blocks) {
+                              int store, int v_head, int64_t num_tokens, int qk_blocks) {
   constexpr int HPW = 64 / LPH;
   const int64_t t = blockIdx.x;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int half = D >> 1;
   if ((int)blockIdx.y >= qk_blocks) {
     const int kvh = ((int)blockIdx.y - qk_blocks) * 4 + wave;
-    if (kvh < Hkv) store_value_head<T>(qkv + t * row_stride + (int64_t)(Hq + Hkv + kvh) * D, row_stride, t, num_tokens,
+    if (kvh < Hkv) store_value_head<T>(qkv + t * row_stride + (int64_t)(v_head + kvh) * D, row_stride, t, num_tokens,
                                        slots, v_cache, Hkv, kvh, D, page, lane);
     return;
   }
@@ -245,7 +247,7 @@ qk_norm_rope_store_tile_kernel(bf16_t* __restrict__ qkv, int64_t row_stride, con
                                const float* __restrict__ k_w, float eps, const float* __restrict__ table,
                                const int32_t* __restrict__ positions, const int32_t* __restrict__ slots,
                                bf16_t* __restrict__ k_cache, bf16_t* __restrict__ v_cache, int Hq, int Hkv, int D,
-                               int page, int store, int64_t num_tokens, int qk_groups) {
+                               int page, int store, int v_head, int64_t num_tokens, int qk_groups) {
   const int64_t t0 = (int64_t)blockIdx.x * 8;
   const int cnt = (int)min((int64_t)8, num_tokens - t0);
   const int half = D >> 1;
@@ -329,7 +331,7 @@ qk_norm_rope_store_tile_kernel(bf16_t* __restrict__ qkv, int64_t row_stride, con
     const int64_t pg = s0 / page, off = s0 - pg * page;               // page % 8 == 0: a group lies within one page
     for (int unit = threadIdx.x; unit < Hkv * dvecs; unit += 256) {
       const int kvh = unit / dvecs, dv = unit - kvh * dvecs;
-      const bf16_t* src = qkv + t * row_stride + (int64_t)(heads + kvh) * D + 8 * dv;
+      const bf16_t* src = qkv + t * row_stride + (int64_t)(v_head + kvh) * D + 8 * dv;
       bf16_t* dst = v_cache + ((pg * Hkv + kvh) * (int64_t)D + 8 * dv) * page + off;
       if (n == 8) {
         u32x4r tok[8];
@@ -361,19 +363,22 @@ extern "C" int me_qk_norm_rope_store(void* qkv, int dtype, int64_t num_tokens, i
                                      const float* table, int64_t table_positions, int64_t position_bound,
                                      const int32_t* positions, const int32_t* slots, void* k_cache,
                                      void* v_cache, int Hq, int Hkv, int D, int page, int store,
-                                     hipStream_t stream) {
+                                     int values_are_keys, hipStream_t stream) {
   if (num_tokens == 0) return 0;
   ME_CHECK(D >= 2 && D % 2 == 0 && D <= 2 * 64 * ME_MAX_PAIRS,
            "qk_norm_rope_store: head_dim %d must be even and <= %d", D, 2 * 64 * ME_MAX_PAIRS);
   ME_CHECK(Hq >= 1 && Hkv >= 0 && page >= 1, "qk_norm_rope_store: bad head counts or page size");
   ME_CHECK(!store || (Hkv >= 1 && k_cache && v_cache), "qk_norm_rope_store: storing needs kv heads and caches");
-  ME_CHECK(row_stride >= (int64_t)(Hq + (store ? 2 * Hkv : Hkv)) * D, "qk_norm_rope_store: row stride too small");
+  ME_CHECK(row_stride >= (int64_t)(Hq + (store && !values_are_keys ? 2 * Hkv : Hkv)) * D, "qk_norm_rope_store: row stride too small");
   ME_CHECK(!table || table_positions > 0, "qk_norm_rope_store: empty rotary table");
   // position_bound: every position of the step is below it (what the host knows of the step; 0: not told)
   ME_CHECK(!table || position_bound <= table_positions,
            "qk_norm_rope_store: positions up to %lld are beyond the rotation table's %lld", (long long)position_bound - 1,
            (long long)table_positions);
   const int heads = Hq + (store ? 2 * Hkv : Hkv);
+  // where a row's value heads begin; values that are the keys as projected are read from the key heads, which stay as they
+  // are in the row (what is normed and rotated goes to the pages)
+  const int v_head = values_are_keys ? Hq : Hq + Hkv;
   ME_CHECK(dtype == ME_BF16 || dtype == ME_F32, "qk_norm_rope_store: bad dtype code %d", dtype);
   // vectorised form: D/8 lanes per head must be a power of two, rows and caches 16-byte aligned
   const int lph = D / 8;
@@ -394,7 +399,7 @@ extern "C" int me_qk_norm_rope_store(void* qkv, int dtype, int64_t num_tokens, i
 #define LAUNCH_TILE(L)                                                                                     \
   qk_norm_rope_store_tile_kernel<L><<<grid, block, 0, stream>>>((bf16_t*)qkv, row_stride, q_w, k_w, eps, table, \
                                                                 positions, slots, (bf16_t*)k_cache,       \
-                                                                (bf16_t*)v_cache, Hq, Hkv, D, page, store, num_tokens, qk_groups)
+                                                                (bf16_t*)v_cache, Hq, Hkv, D, page, store, v_head, num_tokens, qk_groups)
     switch (lph16) {
       case 1: LAUNCH_TILE(1); break; case 2: LAUNCH_TILE(2); break; case 4: LAUNCH_TILE(4); break;
       case 8: LAUNCH_TILE(8); break; case 16: LAUNCH_TILE(16); break; case 32: LAUNCH_TILE(32); break;
@@ -412,7 +417,7 @@ extern "C" int me_qk_norm_rope_store(void* qkv, int dtype, int64_t num_tokens, i
 #define LAUNCH(TT, L)                                                                                       \
   qk_norm_rope_store_vec_kernel<TT, L><<<grid, block, 0, stream>>>((TT*)qkv, row_stride, q_w, k_w, eps, table, \
                                                                    positions, slots, (TT*)k_cache, (TT*)v_cache, \
-                                                                   Hq, Hkv, D, page, store, num_tokens, qk_blocks)
+                                                                   Hq, Hkv, D, page, store, v_head, num_tokens, qk_blocks)
 #define PICK(TT)                                                                                            \
   do {                                                                                                      \
     if (lph == 1) LAUNCH(TT, 1); else if (lph == 2) LAUNCH(TT, 2); else if (lph == 4) LAUNCH(TT, 4);        \
@@ -428,11 +433,11 @@ extern "C" int me_qk_norm_rope_store(void* qkv, int dtype, int64_t num_tokens, i
   if (dtype == ME_BF16)
     qk_norm_rope_store_kernel<bf16_t><<<grid, block, 0, stream>>>(
         (bf16_t*)qkv, row_stride, q_w, k_w, eps, table, positions, slots, (bf16_t*)k_cache,
-        (bf16_t*)v_cache, Hq, Hkv, D, page, store, num_tokens);
+        (bf16_t*)v_cache, Hq, Hkv, D, page, store, v_head, num_tokens);
   else
     qk_norm_rope_store_kernel<float><<<grid, block, 0, stream>>>(
         (float*)qkv, row_stride, q_w, k_w, eps, table, positions, slots, (float*)k_cache,
-        (float*)v_cache, Hq, Hkv, D, page, store, num_tokens);
+        (float*)v_cache, Hq, Hkv, D, page, store, v_head, num_tokens);
   ME_LAUNCH_CHECK();
   return 0;
 }

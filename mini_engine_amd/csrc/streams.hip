@@ -2,7 +2,7 @@
 //
 //   stream_mix_norm   per token, the streams x_1 .. x_S (float32): every new stream takes a share of every old one and
 //                     of the sublayer's output y that waits to be added,
-//                         x'_t = sum_s mix[s, t] x_s + out[t] y,      y = the sum of up to four terms,
+//                         x'_t = sum_s mix[s, t] x_s + out[t] y,      y = the sum of up to four terms (and a bias),
 //                     then what the next sublayer reads, u = sum_t read[t] x'_t, and a norm of u (a layer norm with
 //                     weight and bias, or an RMS norm) in one pass over the streams. Every part may be absent: without
 //                     mix nothing is mixed (x'_t = x_t, plus y where there are terms), without read u is the plain sum,
@@ -20,6 +20,7 @@ struct StreamArgs {
   const void* in; int in_dtype; int64_t row_stride, stream_stride;
   const int32_t* rows; int64_t in_rows;
   const void* term[HS_MAX_TERMS]; int dtype[HS_MAX_TERMS]; int parts[HS_MAX_TERMS]; int64_t part_stride[HS_MAX_TERMS]; int count;
+  const float* y_bias;                                           // [n] or null: joins the sum of the terms
   const float* mix; const float* out_w; const float* read;      // [S, S] (from, to), [S], [S]
   float* streams_out;                                            // [T, S, n] or null
   const float* w; const float* b; int center; float eps;
@@ -79,6 +80,7 @@ __global__ void __launch_bounds__(1024) stream_mix_norm_kernel(StreamArgs a) {
     float y[W];
 #pragma unroll
     for (int e = 0; e < W; ++e) y[e] = 0.f;
+    if (a.y_bias) load_row<W>(a.y_bias, ME_F32, i, y);
 #pragma unroll
     for (int k = 0; k < HS_MAX_TERMS; ++k)
       if (k < a.count) {
@@ -171,7 +173,7 @@ static void launch_stream_mix(const StreamArgs& a, int64_t R, int threads, hipSt
 // streams share the row). rows: int32 [R] or null (R = in_rows then, row by row). terms: `count` entries [parts, in_rows, n].
 extern "C" int me_stream_mix_norm(const void* in, int in_dtype, int64_t row_stride, int64_t stream_stride, const int32_t* rows,
                                   int64_t in_rows, int count, const void* const* term, const int* term_dtype, const int* term_parts,
-                                  const int64_t* term_stride, const float* mix, const float* out_w, const float* read,
+                                  const int64_t* term_stride, const float* y_bias, const float* mix, const float* out_w, const float* read,
                                   float* streams_out, const float* w, const float* b, int center, float eps, void* y, int out_dtype,
                                   int64_t R, int S, int n, hipStream_t stream) {
   if (R == 0) return 0;
@@ -183,10 +185,10 @@ extern "C" int me_stream_mix_norm(const void* in, int in_dtype, int64_t row_stri
   ME_CHECK(y != nullptr || w == nullptr, "stream_mix_norm: a norm needs a place for its result");
   StreamArgs a;
   a.in = in; a.in_dtype = in_dtype; a.row_stride = row_stride; a.stream_stride = stream_stride; a.rows = rows; a.in_rows = in_rows;
-  a.count = count; a.mix = mix; a.out_w = out_w; a.read = read; a.streams_out = streams_out; a.w = w; a.b = b; a.center = center;
+  a.count = count; a.y_bias = y_bias; a.mix = mix; a.out_w = out_w; a.read = read; a.streams_out = streams_out; a.w = w; a.b = b; a.center = center;
   a.eps = eps; a.y = y; a.S = S; a.n = n;
   uintptr_t bits = reinterpret_cast<uintptr_t>(in) | reinterpret_cast<uintptr_t>(streams_out) | reinterpret_cast<uintptr_t>(y) |
-                   reinterpret_cast<uintptr_t>(w) | reinterpret_cast<uintptr_t>(b);
+                   reinterpret_cast<uintptr_t>(w) | reinterpret_cast<uintptr_t>(b) | reinterpret_cast<uintptr_t>(y_bias);
   bool vec = n % 4 == 0 && row_stride % 4 == 0 && stream_stride % 4 == 0;
   for (int k = 0; k < HS_MAX_TERMS; ++k) {
     const bool on = k < count;

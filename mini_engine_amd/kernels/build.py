@@ -36,6 +36,7 @@ HEADERS = ["common.h", "errors.inc", "sampling.h"]
 # Head sizes that build_all() compiles ahead of use; any other multiple of 16 up to 512 is compiled when a model first needs it.
 DEFAULT_HEAD_DIMS = (16, 32, 48, 64, 80, 128, 256)
 CAPPED_HEAD_DIMS = (32, 64, 128)          # ... of the variant with a cap on the scores
+DISTANCE_HEAD_DIMS = (32, 48, 128)        # ... of the variant with slopes times distances
 
 _locks: dict = {}
 _locks_guard = threading.Lock()
@@ -189,14 +190,14 @@ def core_library(force: bool = False) -> str:
     return _ensure("libme_core.so", CORE_SOURCES, [], force)
 
 
-def attention_library(head_dim: int, force: bool = False, score_cap: bool = False) -> str:
+def attention_library(head_dim: int, force: bool = False, score_cap: bool = False, distance: bool = False) -> str:
     """The matrix-core attention kernels for one head size. `score_cap`: the variant whose softmax bends its scores under
-    a cap first (a library of its own, so that the kernels of models without a cap stay as they are)."""
+    a cap first; `distance`: the one whose scores lose a slope per head times the distance between query and key (libraries
+    of their own, so that the kernels of models without them stay as they are)."""
     if head_dim % 16 or not 16 <= head_dim <= 512:
         raise BuildError(f"the bf16 attention kernels need a head size that is a multiple of 16 in 16..512, got {head_dim}")
-    if score_cap:
-        return _ensure(f"libme_attn_d{head_dim}c.so", [ATTN_SOURCE], [f"-DME_HEAD_DIM={head_dim}", "-DME_ATTN_SOFTCAP=1"], force)
-    return _ensure(f"libme_attn_d{head_dim}.so", [ATTN_SOURCE], [f"-DME_HEAD_DIM={head_dim}"], force)
+    flags = [f"-DME_HEAD_DIM={head_dim}"] + ["-DME_ATTN_SOFTCAP=1"] * score_cap + ["-DME_ATTN_DISTANCE=1"] * distance
+    return _ensure(f"libme_attn_d{head_dim}{'c' * score_cap}{'d' * distance}.so", [ATTN_SOURCE], flags, force)
 
 
 def build_all(head_dims=DEFAULT_HEAD_DIMS, force: bool = True) -> list:
@@ -205,4 +206,5 @@ def build_all(head_dims=DEFAULT_HEAD_DIMS, force: bool = True) -> list:
     with ThreadPoolExecutor(max_workers=4) as pool:
         libs += list(pool.map(lambda d: attention_library(d, force=force), head_dims))
         libs += list(pool.map(lambda d: attention_library(d, force=force, score_cap=True), CAPPED_HEAD_DIMS))
+        libs += list(pool.map(lambda d: attention_library(d, force=force, distance=True), DISTANCE_HEAD_DIMS))
     return libs

@@ -62,11 +62,11 @@ _CORE_PROTOS = {
     "me_gather_rows_scaled": [P, I, P, P, L, L, L, F, P],
     "me_take_tokens": [P, P, P, I, I, P],
     "me_rms_norm": [P, I, I, L, P, P, P, P, I, L, I, F, P],
-    "me_silu_and_mul": [P, P, I, L, I, P],
-    "me_qk_norm_rope_store": [P, I, L, L, P, P, F, P, L, L, P, P, P, P, I, I, I, I, I, P],
+    "me_silu_and_mul": [P, P, P, I, L, I, P],
+    "me_qk_norm_rope_store": [P, I, L, L, P, P, F, P, L, L, P, P, P, P, I, I, I, I, I, I, P],
     "me_store_kv": [P, P, I, L, L, L, P, P, P, I, I, I, P],
-    "me_attn_simple": [P, L, P, L, I, P, P, P, I, P, P, P, L, I, I, I, I, F, I, I, F, P, P],
-    "me_attn_tail": [P, L, P, L, P, I, P, P, P, I, P, P, P, L, I, I, I, I, F, I, I, F, P, P],
+    "me_attn_simple": [P, L, P, L, I, P, P, P, I, P, P, P, L, I, I, I, I, F, I, I, F, P, P, P],
+    "me_attn_tail": [P, L, P, L, P, I, P, P, P, I, P, P, P, L, I, I, I, I, F, I, I, F, P, P, P],
     "me_gemm_tiled": [P, L, P, L, P, L, I, I, I, I, I, P],
     "me_gemm_skinny_bf16": [P, L, P, L, P, L, I, P, I, I, I, I, I, I, I, P],
     "me_gemm_rows_bf16": [P, L, P, L, P, L, I, P, I, I, I, I, I, P],
@@ -82,16 +82,16 @@ _CORE_PROTOS = {
                              P, P, P, P, L, P, P, L, P, P, F, P, L, P],
     "me_soft_gates": [P, P, L, I, P, P, F, P, L, P, P, P, P, P, I, I, P],
     "me_memory_readout": [P, I, L, P, P, F, P, L, I, P, P, L, I, I, F, P, P, L, P, P, F, P, L, P, P],
-    "me_stream_mix_norm": [P, I, L, L, P, L, I, P, P, P, P, P, P, P, P, P, P, I, F, P, I, L, I, I, P],
+    "me_stream_mix_norm": [P, I, L, L, P, L, I, P, P, P, P, P, P, P, P, P, P, P, I, F, P, I, L, I, I, P],
     "me_gated_rms_norm": [P, I, L, P, L, I, P, P, L, I, I, I, F, P],
     "me_scaled_sum_norm": [P, I, I, P, P, P, P, P, F, P, P, P, P, P, I, L, I, F, P],
     "me_softcap": [P, L, L, I, F, P],
     "me_qkv_prepare": [P, L, P, P, P, F, I, I, F, I, P, P, P, P, P, L, I, L, I, I, I, I, I, I, P, P, L, P],
     "me_moe_route": [P, L, I, P, P, L, I, I, I, I, I, P, P, P, I, I, I, I, F, P, P],
-    "me_moe_sort": [P, L, I, I, I, P, P, P, P, P, P, I, I, I, I, I, I, F, P, P],
-    "me_moe_gate_up": [P, L, P, P, P, P, P, P, L, I, I, I, I, I, I, P],
-    "me_moe_down": [P, P, P, P, P, P, P, P, L, I, I, I, I, I, P],
-    "me_moe_experts_simple": [P, L, I, P, P, P, P, P, P, L, I, I, I, I, I, P],
+    "me_moe_sort": [P, L, I, I, I, I, P, P, P, P, P, P, I, I, I, I, I, I, F, P, P],
+    "me_moe_gate_up": [P, L, P, P, P, P, P, P, L, I, I, I, I, I, I, I, F, F, P],
+    "me_moe_down": [P, P, P, P, P, P, P, P, L, I, I, I, I, I, I, P, L, P],
+    "me_moe_experts_simple": [P, L, I, P, P, P, P, P, P, L, I, I, I, I, I, I, F, F, P],
     "me_add_bias": [P, I, I, L, L, P, I, P, I, L, I, P],
     "me_sigmoid_gate": [P, L, P, L, I, L, I, P],
     "me_glu_clamped": [P, L, P, I, L, I, F, F, P],
@@ -104,9 +104,9 @@ _CORE_PROTOS = {
     "me_sample_static": [P, L, P, P, P, I, I, P],
 }
 _ATTN_PROTOS = {
-    "me_attn_prefill": [P, L, P, L, P, P, P, I, P, P, I, L, I, I, I, F, I, I, I, I, I, I, P, P, I, F, P, P],
-    "me_attn_decode": [P, L, P, L, P, P, P, I, P, I, I, I, I, F, I, I, I, P, I, F, P, P],
-    "me_attn_decode_fused": [P, L, P, L, P, P, F, P, I, P, P, P, I, P, I, I, I, I, I, F, I, I, I, P, I, F, P, P],
+    "me_attn_prefill": [P, L, P, L, P, P, P, I, P, P, I, L, I, I, I, F, I, I, I, I, I, I, P, P, I, F, P, P, P, P],
+    "me_attn_decode": [P, L, P, L, P, P, P, I, P, I, I, I, I, F, I, I, I, P, I, F, P, P, P, P],
+    "me_attn_decode_fused": [P, L, P, L, P, P, F, P, I, P, P, P, I, P, I, I, I, I, I, F, I, I, I, P, I, F, P, P, P, I, P],
 }
 
 _core: _Lib | None = None
@@ -127,12 +127,12 @@ def core() -> _Lib:
     return _core
 
 
-def attn_lib(head_dim: int, score_cap: bool = False) -> _Lib:
-    key = (head_dim, bool(score_cap)) if score_cap else head_dim
+def attn_lib(head_dim: int, score_cap: bool = False, distance: bool = False) -> _Lib:
+    key = (head_dim, bool(score_cap), bool(distance)) if score_cap or distance else head_dim
     lib = _attn.get(key)
     if lib is None:
         _require_gpu()
-        lib = _Lib(build.attention_library(head_dim, score_cap=bool(score_cap)), _ATTN_PROTOS)
+        lib = _Lib(build.attention_library(head_dim, score_cap=bool(score_cap), distance=bool(distance)), _ATTN_PROTOS)
         lib.cdll.me_attn_head_dim.restype = c_int
         if lib.cdll.me_attn_head_dim() != head_dim:
             raise KernelError(f"{lib.path} was built for head size {lib.cdll.me_attn_head_dim()}, not {head_dim}")
@@ -357,17 +357,19 @@ class HipBackend:
         return y, res_out
 
     # -- feed-forward activation ---------------------------------------------------------
-    def silu_and_mul(self, gu: torch.Tensor) -> torch.Tensor:
-        """silu(gu[:, :I]) * gu[:, I:] (reference layers/activation.py:5-7)."""
+    def silu_and_mul(self, gu: torch.Tensor, bias: torch.Tensor | None = None) -> torch.Tensor:
+        """silu(gu[:, :I]) * gu[:, I:] (reference layers/activation.py:5-7); `bias` (float32 [2 I]) joins gu first."""
         _check(gu.dim() == 2 and gu.is_contiguous() and gu.shape[1] % 2 == 0, "silu_and_mul: [T, 2I] contiguous")
         inter = gu.shape[1] // 2
         out = torch.empty((gu.shape[0], inter), dtype=gu.dtype, device=gu.device)
-        core().call("me_silu_and_mul", gu.data_ptr(), out.data_ptr(), _code(gu.dtype), gu.shape[0], inter, _stream())
+        _check(bias is None or (bias.dtype == torch.float32 and bias.shape == (2 * inter,) and bias.is_contiguous()), "silu_and_mul: bias float32 [2 I]")
+        core().call("me_silu_and_mul", gu.data_ptr(), _ptr(bias), out.data_ptr(), _code(gu.dtype), gu.shape[0], inter, _stream())
         return out
 
     # -- q/k norm + rotary + cache write -------------------------------------------------
     def qk_norm_rope_store(self, qkv, q_weight, k_weight, eps, table, positions, slots, k_cache, v_cache,
-                           Hq: int, Hkv: int, D: int, page: int, store: bool = True, position_bound: int = 0) -> None:
+                           Hq: int, Hkv: int, D: int, page: int, store: bool = True, position_bound: int = 0,
+                           values_are_keys: bool = False) -> None:
         """In place on packed rows: per-head RMSNorm of q and k (weights float32 [D] or None), then
         rotary by `table` [P, D/2, 2] float32 (or None), q written back. `position_bound`: every position
         of the step is below it (the longest context the step's layout allows; 0: not told); a bound beyond
@@ -375,10 +377,11 @@ class HipBackend:
 
         store=True: rows are [T, (Hq+2Hkv)*D]; k and v are scattered to the pages at `slots`
         (slots < 0 skipped). store=False: rows are [T, (Hq+Hkv)*D] (Hkv may be 0); k is written
-        back in place and nothing is cached. (reference models/qwen3.py:34-36,
+        back in place and nothing is cached. values_are_keys (with store): rows are [T, (Hq+Hkv)*D] and a
+        value is its key as projected, in front of norm and rotation. (reference models/qwen3.py:34-36,
         layers/rotary_embedding.py:20-25, csrc/kv_cache.cu:10-31.)"""
         T = qkv.shape[0]
-        width = (Hq + (2 * Hkv if store else Hkv)) * D
+        width = (Hq + (2 * Hkv if store and not values_are_keys else Hkv)) * D
         _check(qkv.dim() == 2 and qkv.stride(1) == 1 and qkv.shape[1] == width,
                f"qk_norm_rope_store: rows must be [T, {width}] with unit inner stride, got {tuple(qkv.shape)}")
         for w in (q_weight, k_weight):
@@ -398,7 +401,7 @@ class HipBackend:
         core().call("me_qk_norm_rope_store", qkv.data_ptr(), _code(qkv.dtype), T, qkv.stride(0), _ptr(q_weight),
                     _ptr(k_weight), float(eps), _ptr(table), 0 if table is None else table.shape[0], int(position_bound),
                     positions.data_ptr(), _ptr(slots) if store else None, _ptr(k_cache) if store else None,
-                    _ptr(v_cache) if store else None, Hq, Hkv, D, page, int(store), _stream())
+                    _ptr(v_cache) if store else None, Hq, Hkv, D, page, int(store), int(bool(values_are_keys)), _stream())
 
     def store_kv(self, k, v, slots, k_cache, v_cache, page: int) -> None:
         """Scatter k, v [T, Hkv, D] (views with a token stride are fine) into the pages; slots < 0
@@ -418,15 +421,17 @@ class HipBackend:
                         positions, prefill_cu, num_decodes: int, max_decode_context: int, scale: float,
                         window: int | None, Hq: int, Hkv: int, D: int, force_simple: bool = False,
                         max_prefill_context: int = 0, even_contexts: bool = False, decode_as_prefill: bool = False,
-                        chunk: int | None = None, keep_first: int = 0, softcap: float | None = None, sinks=None):
+                        chunk: int | None = None, keep_first: int = 0, softcap: float | None = None, sinks=None, slopes=None):
         """Causal attention of this step's tokens over the paged keys of their requests. `chunk`: a block mask in
         place of a window: the query at position i sees the keys j <= i of its own block, floor(j / chunk) =
         floor(i / chunk) (the kernels take it as a negative window). `keep_first`: behind a window the keys j <
         keep_first stay visible. `softcap` c: every score becomes c * tanh(score / c) before the softmax. `sinks`
-        (float32 [Hq]): exp(sink_h) joins the softmax's denominator of head h, a term without key or value. With any
-        three. On the matrix-core path the cap runs inside the kernels (a library variant of its own), which also leave
-        the logarithm of every softmax denominator; a second kernel (`attn_tail`) then joins the kept keys behind the
-        window and the sink to that softmax. The float32 path and odd sizes take the exact kernel (`attn_simple`) for all of it.
+        (float32 [Hq]): exp(sink_h) joins the softmax's denominator of head h, a term without key or value. `slopes`
+        (float32 [Hq], not negative): behind the cap, the score of the query at position i and the key j loses slope_h * (i - j).
+        On the matrix-core path the cap and the slopes run inside the kernels (library variants of their own), and so do
+        the sinks where a launch forms or merges its last sums. Kept keys behind a window are joined by a second kernel
+        (`attn_tail`, then with the sinks) to a softmax whose denominators' logarithms the first has left.
+        The float32 path and odd sizes take the exact kernel (`attn_simple`) for all of it.
 
         q: [T, Hq*D] (a strided view is fine). Rows are ordered decode requests first (one token
         each, `num_decodes` of them), then the others; `prefill_cu` int32 [B - num_decodes + 1]
@@ -456,16 +461,20 @@ class HipBackend:
         _check(not keep_first or (window and keep_first > 0), "attention: keys are kept behind a window only")
         _check(sinks is None or (sinks.dtype == torch.float32 and sinks.shape == (Hq,) and sinks.is_contiguous()),
                "attention: sinks must be float32 [Hq]")
-        tail = bool(keep_first) or sinks is not None
+        _check(slopes is None or (slopes.dtype == torch.float32 and slopes.shape == (Hq,) and slopes.is_contiguous()),
+               "attention: slopes must be float32 [Hq]")
+        tail = bool(keep_first)
+        extras = tail or softcap or sinks is not None or slopes is not None
         mfma = (q.dtype == torch.bfloat16 and D % 16 == 0 and 16 <= D <= 512 and page >= 8 and page & (page - 1) == 0
-                and not force_simple and (MFMA_WITH_EXTRAS or not (tail or softcap)))
+                and not force_simple and (MFMA_WITH_EXTRAS or not extras))
         if not mfma:
             core().call("me_attn_simple", q.data_ptr(), q.stride(0), out.data_ptr(), out.stride(0), _code(q.dtype),
                         k_cache.data_ptr(), v_cache.data_ptr(), block_tables.data_ptr(), block_tables.stride(0),
                         seq_of_token.data_ptr(), positions.data_ptr(), context_lens.data_ptr(), T, Hq, Hkv, D, page,
-                        float(scale), win, int(keep_first or 0), float(softcap or 0.0), _ptr(sinks), _stream())
+                        float(scale), win, int(keep_first or 0), float(softcap or 0.0), _ptr(sinks), _ptr(slopes), _stream())
             return out
-        lib = attn_lib(D, score_cap=bool(softcap))
+        lib = attn_lib(D, score_cap=bool(softcap), distance=slopes is not None)
+        inner = None if tail else _ptr(sinks)
         cap = float(softcap or 0.0)
         lse = torch.empty((T, Hq), dtype=torch.float32, device=q.device) if tail else None
         es = q.element_size()
@@ -482,7 +491,7 @@ class HipBackend:
             lib.call("me_attn_decode", q.data_ptr(), q.stride(0), out.data_ptr(), out.stride(0), k_cache.data_ptr(),
                      v_cache.data_ptr(), block_tables.data_ptr(), block_tables.stride(0), context_lens.data_ptr(),
                      num_decodes, Hq, Hkv, page, float(scale), win, part_size, num_parts, _ptr(scratch),
-                     0 if even_contexts else 1, cap, _ptr(lse), _stream())
+                     0 if even_contexts else 1, cap, inner, _ptr(slopes), _ptr(lse), _stream())
         if T > num_decodes:
             _check(prefill_cu is not None and _is_i32(prefill_cu, B - num_decodes + 1), "attention: prefill_cu must be int32 [B-Dn+1]")
             Tp = T - num_decodes
@@ -497,30 +506,36 @@ class HipBackend:
                      v_cache.data_ptr(), block_tables.data_ptr() + num_decodes * block_tables.stride(0) * 4,
                      block_tables.stride(0), context_lens.data_ptr() + num_decodes * 4, prefill_cu.data_ptr(),
                      B - num_decodes, Tp, Hq, Hkv, page, float(scale), win, col_tiles, PREFILL_THROUGH_LDS, waves, seg_keys, max_segs,
-                     _ptr(pf), seq_of_token.data_ptr() + num_decodes * 4, num_decodes, cap,
+                     _ptr(pf), seq_of_token.data_ptr() + num_decodes * 4, num_decodes, cap, inner, _ptr(slopes),
                      None if lse is None else lse.data_ptr() + num_decodes * Hq * 4, _stream())
         if tail:
             core().call("me_attn_tail", q.data_ptr(), q.stride(0), out.data_ptr(), out.stride(0), lse.data_ptr(), _code(q.dtype),
                         k_cache.data_ptr(), v_cache.data_ptr(), block_tables.data_ptr(), block_tables.stride(0),
                         seq_of_token.data_ptr(), positions.data_ptr(), context_lens.data_ptr(), T, Hq, Hkv, D, page, float(scale),
-                        win, int(keep_first or 0), cap, _ptr(sinks), _stream())
+                        win, int(keep_first or 0), cap, _ptr(sinks), _ptr(slopes), _stream())
         return out
 
     def decode_step_attention(self, qkv, q_weight, k_weight, eps, table, k_cache, v_cache, page: int, block_tables,
                               context_lens, max_context: int, scale: float, window: int | None, Hq: int, Hkv: int,
-                              D: int, even_contexts: bool = False, chunk: int | None = None):
+                              D: int, even_contexts: bool = False, chunk: int | None = None, sinks=None, slopes=None,
+                              values_are_keys: bool = False):
         """A pure decode step's `qk_norm_rope_store` and `paged_attention` as one launch: rows [B, (Hq+2Hkv)*D]
         as the packed product left them (row r is request r's one new token, at position context_lens[r] - 1).
         The kernel norms and rotates q and the new key in float32, rounds them to bfloat16 as the separate
         kernel leaves them in the rows, writes the new key and value to the page the block table names for
         that position and attends over the pages. The rows stay as they were. Takes what `decode_step_fuses`
-        admits. Returns [B, Hq*D]. (reference models/qwen3.py:34-38, layers/attention.py:63-70: the same
+        admits; `sinks`, `slopes` as in `paged_attention`; values_are_keys: rows [B, (Hq+Hkv)*D], a value is its key as
+        projected, in front of norm and rotation. Returns [B, Hq*D]. (reference models/qwen3.py:34-38, layers/attention.py:63-70: the same
         four calls one after the other.)"""
         B = qkv.shape[0]
         _check(decode_step_fuses(qkv.dtype, D, page), "decode_step_attention: bfloat16 rows, head sizes in steps of 16 "
                "up to 512 and pages of a power of two from 8 on")
-        _check(qkv.dim() == 2 and qkv.stride(1) == 1 and qkv.shape[1] == (Hq + 2 * Hkv) * D,
-               f"decode_step_attention: rows must be [B, {(Hq + 2 * Hkv) * D}] with unit inner stride")
+        width = (Hq + (1 if values_are_keys else 2) * Hkv) * D
+        _check(qkv.dim() == 2 and qkv.stride(1) == 1 and qkv.shape[1] == width,
+               f"decode_step_attention: rows must be [B, {width}] with unit inner stride")
+        for per_head in (sinks, slopes):
+            _check(per_head is None or (per_head.dtype == torch.float32 and per_head.shape == (Hq,) and per_head.is_contiguous()),
+                   "decode_step_attention: sinks and slopes must be float32 [Hq]")
         for w in (q_weight, k_weight):
             _check(w is None or (w.dtype == torch.float32 and w.shape == (D,) and w.is_contiguous()),
                    "decode_step_attention: norm weights must be float32 [D]")
@@ -538,12 +553,13 @@ class HipBackend:
         out = torch.empty((B, Hq * D), dtype=qkv.dtype, device=qkv.device)
         part_size, num_parts = decode_partitions(B, Hq, Hkv, max_context, even_contexts)
         scratch = _scratch(B * Hq * num_parts * (D + 2), qkv.device) if num_parts > 1 else None
-        attn_lib(D).call("me_attn_decode_fused", qkv.data_ptr(), qkv.stride(0), out.data_ptr(), out.stride(0),
+        attn_lib(D, distance=slopes is not None).call("me_attn_decode_fused", qkv.data_ptr(), qkv.stride(0), out.data_ptr(), out.stride(0),
                          _ptr(q_weight), _ptr(k_weight), float(eps), _ptr(table), 0 if table is None else table.shape[0],
                          k_cache.data_ptr(), v_cache.data_ptr(), block_tables.data_ptr(), block_tables.stride(0),
                          context_lens.data_ptr(), int(max_context), B, Hq, Hkv, page, float(scale),
                          -int(chunk) if chunk else int(window or 0),
-                         part_size, num_parts, _ptr(scratch), 0 if even_contexts else 1, 0.0, None, _stream())
+                         part_size, num_parts, _ptr(scratch), 0 if even_contexts else 1, 0.0, _ptr(sinks), _ptr(slopes), None,
+                         int(bool(values_are_keys)), _stream())
         return out
 
     # -- matrix products -----------------------------------------------------------------
@@ -843,10 +859,11 @@ class HipBackend:
         return out
 
     # -- several residual streams ----------------------------------------------------------------
-    def stream_mix_norm(self, streams, count: int, terms, mix, out_weights, read, norm, out_dtype: torch.dtype, rows=None, keep: bool = True):
+    def stream_mix_norm(self, streams, count: int, terms, mix, out_weights, read, norm, out_dtype: torch.dtype, rows=None, keep: bool = True,
+                        bias=None):
         """Several residual streams x_1 .. x_S (S = `count`), float32 [T, S, n], or rows [T, n] (any dtype) that all streams
         share. x'_t = sum_s mix[s, t] x_s + out_weights[t] y, y the sum of up to four `terms` (rows [T, n] or float32 partial
-        sums [P, T, n]); without mix x'_t = x_t + y. u = sum_t read[t] x'_t (read None: the plain sum). `norm`: (weight float32
+        sums [P, T, n]), to which `bias` (float32 [n]) is added; without mix x'_t = x_t + y. u = sum_t read[t] x'_t (read None: the plain sum). `norm`: (weight float32
         [n], bias float32 [n] or None, eps, centred): a layer norm (centred: the mean is taken off, the variance is that of the
         deviations) or an RMS norm of u; None: u itself comes out. `rows` (int32 [R]): only these rows, one result each, in
         order. `keep`: the new streams are wanted. Returns (x' float32 [R, S, n] or None, the result [R, n] in out_dtype). Where
@@ -861,7 +878,7 @@ class HipBackend:
                "stream_mix_norm: mix float32 [S, S] with weights [S], read float32 [S]")
         _check(rows is None or (_is_i32(rows) and rows.dim() == 1), "stream_mix_norm: rows int32 [R]")
         w, b, eps, centred = norm if norm is not None else (None, None, 0.0, False)
-        _check(f32(w, (n,)) and f32(b, (n,)), "stream_mix_norm: norm weight and bias float32 [n]")
+        _check(f32(w, (n,)) and f32(b, (n,)) and f32(bias, (n,)), "stream_mix_norm: norm weight and biases float32 [n]")
         k = len(terms)
         ptrs, dts, parts, strides = (c_void_p * 4)(), (c_int * 4)(), (c_int * 4)(), (c_int64 * 4)()
         for i, t in enumerate(terms):
@@ -869,11 +886,11 @@ class HipBackend:
                    "stream_mix_norm: a term is rows [T, n] or float32 partial sums [P, T, n]")
             ptrs[i], dts[i], parts[i], strides[i] = t.data_ptr(), _code(t.dtype), (t.shape[0] if t.dim() == 3 else 1), T * n
         R = T if rows is None else rows.numel()
-        as_they_are = k == 0 and mix is None and not shared and rows is None and streams.dtype == torch.float32
+        as_they_are = k == 0 and bias is None and mix is None and not shared and rows is None and streams.dtype == torch.float32
         new = torch.empty((R, S, n), dtype=torch.float32, device=streams.device) if keep and not as_they_are else None
         y = torch.empty((R, n), dtype=out_dtype, device=streams.device)
         core().call("me_stream_mix_norm", streams.data_ptr(), _code(streams.dtype), n if shared else S * n, 0 if shared else n, _ptr(rows), T,
-                    k, ptrs, dts, parts, strides, _ptr(mix), _ptr(out_weights), _ptr(read), _ptr(new), _ptr(w), _ptr(b), int(bool(centred)),
+                    k, ptrs, dts, parts, strides, _ptr(bias), _ptr(mix), _ptr(out_weights), _ptr(read), _ptr(new), _ptr(w), _ptr(b), int(bool(centred)),
                     float(eps), y.data_ptr(), _code(out_dtype), R, S, n, _stream())
         return (streams if as_they_are and keep else new), y
 
@@ -1119,8 +1136,9 @@ class HipBackend:
         return ids, weights
 
     def route_and_run_experts(self, x, router, top: int, group_count: int, group_keep: int, gate_up, down,
-                              rule: "RouteRule | None" = None, gated: bool = True) -> torch.Tensor:
-        """`moe_route` and `routed_experts` behind it: float32 [top, T, hidden]. For the few tokens `moe_sort_chooses` admits,
+                              rule: "RouteRule | None" = None, gated: bool = True, clamp: tuple | None = None) -> torch.Tensor:
+        """`moe_route` and `routed_experts` behind it: float32 [top, T, hidden]. The router may know more experts than there
+        are weights; those behind the last one with weights are identity experts. For the few tokens `moe_sort_chooses` admits,
         the kernel that orders the pairs by expert makes the choice itself from the router's logits: one launch less in a
         decode step's chain."""
         T, n = x.shape
@@ -1130,7 +1148,7 @@ class HipBackend:
         if not (moe_sort_chooses(T, E, group_count) and x.dtype == torch.bfloat16 and n % 8 == 0 and F % 8 == 0 and x.stride(0) % 8 == 0
                 and x.data_ptr() % 16 == 0):
             ids, weights = self.moe_route(x, router, top, group_count, group_keep, rule)
-            return self.routed_experts(x, ids, weights, gate_up, down, gated=gated)
+            return self.routed_experts(x, ids, weights, gate_up, down, gated=gated, clamp=clamp, routed=E)
         _check(x.stride(1) == 1 and router.dtype == torch.float32 and router.shape == (E, n) and router.is_contiguous(),
                "moe_route: rows [T, n], router float32 [E, n]")
         rule.check(E)
@@ -1139,14 +1157,18 @@ class HipBackend:
         logits = torch.empty((T, E), dtype=torch.float32, device=x.device)
         core().call("me_moe_route", x.data_ptr(), x.stride(0), _code(x.dtype), router.data_ptr(), _ptr(rule.bias), T, n, E, int(top), int(group_count),
                     int(group_keep), logits.data_ptr(), ids.data_ptr(), weights.data_ptr(), 0, *rule.args(), _stream())
-        return self.routed_experts(x, ids, weights, gate_up, down, choose_from=(logits, group_count, group_keep, rule), gated=gated)
+        return self.routed_experts(x, ids, weights, gate_up, down, choose_from=(logits, group_count, group_keep, rule), gated=gated,
+                                   clamp=clamp, routed=E)
 
     def routed_experts(self, x, ids, weights, gate_up, down, force_simple: bool = False, tile_rows: int | None = None,
-                       choose_from=None, gated: bool = True) -> torch.Tensor:
+                       choose_from=None, gated: bool = True, clamp: tuple | None = None, routed: int | None = None) -> torch.Tensor:
         """Every token through its chosen experts: out[j, t] = weights[t, j] * W_down[e] (silu(W_gate[e] x_t) * (W_up[e] x_t)),
         e = ids[t, j]: float32 [top, T, hidden], one partial sum per choice for a consumer that adds them. x: [T, K];
         gate_up: [E, 2 F, K] (an expert's gate rows, then its up rows); down: [E, hidden, F]. With `gated` False the experts
-        have no gate: gate_up is [E, F, K] (up rows only) and an expert is W_down[e] relu(W_up[e] x_t)^2. bfloat16 with K and F in
+        have no gate: gate_up is [E, F, K] (up rows only) and an expert is W_down[e] relu(W_up[e] x_t)^2. `clamp` (limit,
+        alpha): with g = min(W_gate[e] x_t, limit) and u = clamp(W_up[e] x_t, -limit, limit) an expert is W_down[e] (g sigmoid(alpha
+        g) (u + 1)). `routed` (more than E): ids run up to it, and those from E on name identity experts, whose output is x_t
+        itself (hidden = K then). bfloat16 with K and F in
         whole steps of 8: the (token, choice) pairs are ordered by expert and cut into tiles that never span two experts, of
         64 rows (a workgroup's 64 x 64 tile of the matrix-core kernel) or, while an expert gets few rows (`expert_tile_rows`;
         `tile_rows` forces it), of 16 rows for the kernel that streams the chosen experts' weights with K cut over a
@@ -1159,29 +1181,34 @@ class HipBackend:
                and down.shape == (E, N, F) and gate_up.dtype == x.dtype and down.dtype == x.dtype, "routed_experts: operand shapes")
         _check(ids.dtype == torch.int32 and ids.is_contiguous() and weights.dtype == torch.float32 and weights.is_contiguous()
                and ids.shape == (T, top) and weights.shape == (T, top), "routed_experts: ids int32 [T, top], weights float32 [T, top]")
+        routed = int(routed or E)
+        _check(routed >= E and (routed == E or N == K), "routed_experts: an identity expert's output is as wide as its input")
+        _check(clamp is None or (gated and clamp[0] > 0), "routed_experts: only a gate can be clamped, at a positive limit")
+        limit, alpha = (0.0, 0.0) if clamp is None else (float(clamp[0]), float(clamp[1]))
+        classes = E + (1 if routed > E else 0)        # the pairs of all identity experts form one class behind the experts'
         out = torch.empty((top, T, N), dtype=torch.float32, device=x.device)
         Pn = T * top
         act = torch.empty((Pn, F), dtype=x.dtype, device=x.device)
-        rows = tile_rows or expert_tile_rows(T, top, E)
+        rows = tile_rows or expert_tile_rows(T, top, routed)
         tiled = (x.dtype == torch.bfloat16 and K % 8 == 0 and F % 8 == 0 and x.stride(0) % 8 == 0 and x.data_ptr() % 16 == 0
-                 and not force_simple and Pn // rows + min(E, Pn) <= 65535)
+                 and not force_simple and Pn // rows + min(classes, Pn) <= 65535)
         if not tiled:
             core().call("me_moe_experts_simple", x.data_ptr(), x.stride(0), _code(x.dtype), gate_up.data_ptr(), down.data_ptr(),
-                        ids.data_ptr(), weights.data_ptr(), act.data_ptr(), out.data_ptr(), T, top, N, F, K, int(gated), _stream())
+                        ids.data_ptr(), weights.data_ptr(), act.data_ptr(), out.data_ptr(), T, top, N, F, K, int(gated), E, limit, alpha, _stream())
             return out
-        max_tiles = Pn // rows + min(E, Pn)
-        meta = torch.empty((Pn + E + 1 + 2 * max_tiles,), dtype=torch.int32, device=x.device)
-        order, offsets = meta[:Pn], meta[Pn:Pn + E + 1]
-        tile_expert, tile_row = meta[Pn + E + 1:Pn + E + 1 + max_tiles], meta[Pn + E + 1 + max_tiles:]
+        max_tiles = Pn // rows + min(classes, Pn)
+        at = Pn + classes + 1
+        meta = torch.empty((at + 2 * max_tiles,), dtype=torch.int32, device=x.device)
+        order, offsets, tile_expert, tile_row = meta[:Pn], meta[Pn:at], meta[at:at + max_tiles], meta[at + max_tiles:]
         # choose_from (logits, group_count, group_keep, rule): ids and weights are still empty and the sort kernel fills them
         logits, gc, gk, rule = choose_from if choose_from is not None else (None, 1, 1, RouteRule())
         _check(choose_from is None or tiled, "routed_experts: the choice inside the sort kernel needs the tiled path")
-        core().call("me_moe_sort", ids.data_ptr(), Pn, E, max_tiles, rows, order.data_ptr(), offsets.data_ptr(), tile_expert.data_ptr(),
+        core().call("me_moe_sort", ids.data_ptr(), Pn, routed, routed - E, max_tiles, rows, order.data_ptr(), offsets.data_ptr(), tile_expert.data_ptr(),
                     tile_row.data_ptr(), _ptr(logits), weights.data_ptr(), top, int(gc), int(gk), *rule.args(), _stream())
         core().call("me_moe_gate_up", x.data_ptr(), x.stride(0), gate_up.data_ptr(), order.data_ptr(), offsets.data_ptr(),
-                    tile_expert.data_ptr(), tile_row.data_ptr(), act.data_ptr(), T, top, F, K, max_tiles, rows, int(gated), _stream())
+                    tile_expert.data_ptr(), tile_row.data_ptr(), act.data_ptr(), T, top, F, K, max_tiles, rows, int(gated), E, limit, alpha, _stream())
         core().call("me_moe_down", act.data_ptr(), down.data_ptr(), order.data_ptr(), offsets.data_ptr(), tile_expert.data_ptr(),
-                    tile_row.data_ptr(), weights.data_ptr(), out.data_ptr(), T, top, N, F, max_tiles, rows, _stream())
+                    tile_row.data_ptr(), weights.data_ptr(), out.data_ptr(), T, top, N, F, max_tiles, rows, E, x.data_ptr(), x.stride(0), _stream())
         return out
 
     # -- attention over a latent that all heads share ------------------------------------------

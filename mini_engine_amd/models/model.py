@@ -11,8 +11,8 @@ from dataclasses import dataclass, replace
 import torch
 
 from ..kernels import ops
-from ..parts.base import CacheNeed, LayerCall, Part, Settled, StateNeed, StreamSum
-from ..parts.block import norm_of, settled
+from ..parts.base import CacheNeed, LayerCall, Part, Settled, StateNeed, StreamSum, TermSum
+from ..parts.block import norm_of, settled, with_start
 
 
 @dataclass
@@ -108,9 +108,11 @@ class DecoderModel(Part):
         """token_ids int32 [T] -> (last layer output, residual): both go to `logits`.
 
         caches[i] / states[i]: the CacheView / state tensor of run-order entry i (or None)."""
-        h = self.embedding.forward(token_ids)
+        h = start = self.embedding.forward(token_ids)
         residual = None
         for i, call in enumerate(self.order):
+            if call.add_start:
+                h, residual = with_start(h, residual, start)
             h, residual = self.layers[call.layer].forward(h, residual, step, caches[i], states[i])
         return h, residual
 
@@ -118,7 +120,7 @@ class DecoderModel(Part):
         """Final norm of (h + residual), then the rows that want logits, then the head: float32
         [len(rows), vocab] (reference models/qwen3.py:91,116-117; layers/embed_head.py:19-23).
         `out`: where the head puts them (`parts.Head.forward(x, out)`)."""
-        if isinstance(h, StreamSum):        # the last layer's streams: mixed, summed and normed at the wanted rows only
+        if isinstance(h, (StreamSum, TermSum)):        # what the last layer left: summed (its streams mixed) and normed at the wanted rows only
             x = h.normed_rows(residual, self.final_norm, rows)
             if x is not None:
                 return self.head.forward(x, out=out)

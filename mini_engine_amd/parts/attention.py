@@ -7,7 +7,7 @@ import math
 import torch
 
 from ..kernels import ops
-from .base import CacheNeed, Mixer, ParamSpec, PositionEncoding, register_part
+from .base import Biased, CacheNeed, Mixer, ParamSpec, PositionEncoding, register_part
 from .linear import Linear
 
 
@@ -53,7 +53,12 @@ class Attention(Mixer):
     output product), and `qkv_bias` together with per-head norms or a position encoding (the biases are then added to
     the packed product's unrounded sums by a kernel of their own in front of the per-head norm and rotation).
     `qk_norm_weights=False`: the per-head norm of q and k has no learned weights (every head is brought to unit root mean
-    square and that is all). Such a norm may stand in front of the rotation or behind it: a rotation changes no pair's
+    square and that is all). `values_are_keys`: there is no value projection, a head's values are its keys as projected (in front
+    of norm and rotation). `slopes` (one number per query head): a score loses slope_h times the distance between query and
+    key. `sink_score`: the same number for every head in place of learned `sinks`. `kernel_dim`: the head size of the kernels
+    without a position encoding (slots behind `head_dim` are zero).
+
+    A norm without weights may stand in front of the rotation or behind it: a rotation changes no pair's
     length, so the head's mean square, and with it the result, is the same either way.
     """
 
@@ -65,8 +70,20 @@ class Attention(Mixer):
                  chunk: int | None = None, head_gate: bool = False, qkv_bias: bool = False, qk_norm_over: str = "head",
                  q_temperature: tuple | None = None, value_mix: str | None = None, value_mix_key: str = "v_first",
                  keep_first: int = 0, score_cap: float | None = None, sinks: bool = False, output_gate: bool = False,
-                 out_bias: bool = False, qk_norm_weights: bool = True):
+                 out_bias: bool = False, qk_norm_weights: bool = True, values_are_keys: bool = False, slopes=None,
+                 sink_score: float | None = None, kernel_dim: int | None = None):
         super().__init__()
+        self.values_are_keys = bool(values_are_keys)
+        if self.values_are_keys and (not own_kv or qkv_bias or (value_dim is not None and value_dim != head_dim)):
+            raise ValueError("values that are the keys come with keys of the layer's own, of the keys' size, and without biases")
+        if sink_score is not None and sinks:
+            raise ValueError("a sink is learned per head or one given number, not both")
+        if slopes is not None and len(slopes) != num_heads:
+            raise ValueError(f"{len(slopes)} slopes for {num_heads} query heads")
+        self.slope_list = None if slopes is None else [float(s) for s in slopes]
+        if self.slope_list is not None and min(self.slope_list) < 0:
+            raise ValueError("slopes must not be negative")
+        self.sink_score, self.slopes = (None if sink_score is None else float(sink_score)), None
         if qk_norm_over not in ("head", "projection") or value_mix not in (None, "first", "blend"):
             raise ValueError("qk_norm_over is 'head' or 'projection', value_mix None, 'first' or 'blend'")
         self.qkv_bias_on = bool(qkv_bias)
@@ -84,6 +101,8 @@ class Attention(Mixer):
         per_head_path = (position is not None or not own_kv or head_gate or output_gate
                          or (qk_norm_eps is not None and qk_norm_over == "head"))
         self.prologue = bool(qk_norm_over == "projection" or q_temperature is not None or value_mix or (qkv_bias and not per_head_path))
+        if self.prologue and (self.values_are_keys or slopes is not None or sink_score is not None):
+            raise ValueError("values that are the keys, slopes and sinks are not part of the path with biases and whole-projection norms")
         if self.prologue and per_head_path:
             raise ValueError("biases, whole-projection norms, query temperatures and value mixing come without a position "
                              "encoding, head gates or per-head norms, on keys and values of the layer's own")
@@ -105,6 +124,8 @@ class Attention(Mixer):
         self.value_dim = head_dim if value_dim is None else int(value_dim)
         order = position.head_order() if position is not None and hasattr(position, "head_order") else None
         slots = getattr(position, "head_dim", head_dim) if position is not None else head_dim
+        if position is None and kernel_dim is not None:
+            slots = max(head_dim, int(kernel_dim))
         if self.value_dim != head_dim or slots != head_dim:
             # one head size for the kernels: the larger of the two, in whole steps of 16
             head_dim = self.head_dim = max(slots, -(-max(head_dim, self.value_dim) // 16) * 16)
@@ -116,16 +137,18 @@ class Attention(Mixer):
         stored_q, stored_k, stored_v = num_heads * self.stored_dim, num_kv_heads * self.stored_dim, num_kv_heads * self.value_dim
         blocks = {"q": stored_q}
         if own_kv:
-            blocks.update(k=stored_k, v=stored_v)
+            blocks["k"] = stored_k
+            if not self.values_are_keys:
+                blocks["v"] = stored_v
         if head_gate:
             blocks["g"] = num_heads
         if output_gate:
             blocks["g"] = num_heads * self.value_dim
         self.add_child("qkv", Linear(hidden_size, sum(blocks.values()), parts=blocks))
         self.add_child("o", Linear(num_heads * self.value_dim, hidden_size))
-        rows = self.q_size + (2 * self.kv_size if own_kv else 0) + (num_heads if head_gate else 0) + (self.q_size if output_gate else 0)
+        self.gate_at = self.q_size + ((1 if self.values_are_keys else 2) * self.kv_size if own_kv else 0)      # first gate column of the kernels' rows
+        rows = self.gate_at + (num_heads if head_gate else 0) + (self.q_size if output_gate else 0)
         self._relayout = self._relayout or rows % 8 != 0
-        self.gate_at = self.q_size + (2 * self.kv_size if own_kv else 0)      # first gate column of the kernels' rows
         self._laid_out = False
         self.qk_norm_weights = bool(qk_norm_weights)
         if qk_norm_eps is not None and not self.qk_norm_weights:
@@ -167,6 +190,10 @@ class Attention(Mixer):
         if self.norm_eps is not None and not self.qk_norm_weights and not self._laid_out:
             self.q_norm_weight = torch.ones(self.stored_dim, dtype=torch.float32, device=device)
             self.k_norm_weight = torch.ones(self.stored_dim, dtype=torch.float32, device=device) if self.own_kv else None
+        if self.slope_list is not None:
+            self.slopes = torch.tensor(self.slope_list, dtype=torch.float32, device=device)
+        if self.sink_score is not None:
+            self.sinks = torch.full((self.num_heads,), self.sink_score, dtype=torch.float32, device=device)
         if not self._relayout or self._laid_out:
             return
         H, G, D, n, nv = self.num_heads, self.num_kv_heads, self.head_dim, self.stored_dim, self.value_dim
@@ -185,8 +212,11 @@ class Attention(Mixer):
         at = stored_q
         if self.own_kv:
             keep = torch.tensor(list(range(nv)) + [-1] * (D - nv), dtype=torch.long)
-            parts += [heads(w[at:at + stored_k], G, n, take), heads(w[at + stored_k:at + stored_k + G * nv], G, nv, keep)]
-            at += stored_k + G * nv
+            parts.append(heads(w[at:at + stored_k], G, n, take))
+            at += stored_k
+            if not self.values_are_keys:
+                parts.append(heads(w[at:at + G * nv], G, nv, keep))
+                at += G * nv
         if self.head_gate:
             parts.append(w[at:at + H])
         if self.output_gate:                 # the gates take the slots of the values they multiply
@@ -256,8 +286,10 @@ class Attention(Mixer):
         else:
             packed = self.qkv.forward(x)
         gated = self.head_gate
-        extras = dict(keep_first=self.keep_first, softcap=self.score_cap, sinks=self.sinks)
-        plain_scores = not self.keep_first and self.score_cap is None and self.sinks is None
+        extras = dict(keep_first=self.keep_first, softcap=self.score_cap)
+        per_head = dict(sinks=self.sinks, slopes=self.slopes)
+        same = dict(values_are_keys=True) if self.values_are_keys else {}
+        plain_scores = not self.keep_first and self.score_cap is None
         # the kernels' rows end where the gate columns (and the padding to whole steps of 8) begin
         qkv = packed if packed.shape[1] == self.gate_at else packed[:, : self.gate_at]
         store = self.own_kv and cache.write
@@ -270,7 +302,7 @@ class Attention(Mixer):
             # only single tokens: norm, rotary, cache write and attention in one launch
             o = ops.decode_step_attention(qkv, qw, kw, eps, table, cache.k, cache.v, cache.page_size, grp.block_tables,
                                           step.context_lens, step.max_decode_context, self.scale, self.window,
-                                          Hq, Hkv, D, even_contexts=step.decode_contexts_even, chunk=self.chunk)
+                                          Hq, Hkv, D, even_contexts=step.decode_contexts_even, chunk=self.chunk, **per_head, **same)
             if gated:
                 ops.head_gate(o, packed[:, self.gate_at:self.gate_at + Hq], Hq, D)
             return self._project(o, packed)
@@ -279,12 +311,14 @@ class Attention(Mixer):
             bound = max(step.max_decode_context, step.max_prefill_context)
             if store:
                 ops.qk_norm_rope_store(qkv, qw, kw, eps, table, step.positions, grp.slot_mapping,
-                                       cache.k, cache.v, Hq, Hkv, D, cache.page_size, store=True, position_bound=bound)
+                                       cache.k, cache.v, Hq, Hkv, D, cache.page_size, store=True, position_bound=bound, **same)
             else:
                 rows = qkv[:, : self.q_size]
                 ops.qk_norm_rope_store(rows, qw, kw, eps, table, step.positions, None, None, None,
                                        Hq, 0, D, cache.page_size, store=False, position_bound=bound)
         else:
+            if self.values_are_keys:
+                raise NotImplementedError("values that are the keys need a position encoding with a table, or none")
             # another position encoding: norm in place, the encoding's own apply, then the cache write
             nk = Hkv if self.own_kv else 0
             ops.qk_norm_rope_store(qkv[:, : self.q_size + nk * D], qw, kw, eps, None, step.positions, None, None,
@@ -301,7 +335,7 @@ class Attention(Mixer):
                                 step.seq_of_token, step.positions, step.prefill_cu, step.num_decodes,
                                 step.max_decode_context, self.scale, self.window, Hq, Hkv, D,
                                 max_prefill_context=step.max_prefill_context,
-                                even_contexts=step.decode_contexts_even, chunk=self.chunk, **extras)
+                                even_contexts=step.decode_contexts_even, chunk=self.chunk, **extras, **per_head)
         if gated:
             ops.head_gate(o, packed[:, self.gate_at:self.gate_at + Hq], Hq, D)
         return self._project(o, packed)
@@ -313,7 +347,6 @@ class Attention(Mixer):
         y = self.o.forward(o, allow_partials=True)
         if self.out_bias_on:
             if getattr(self, "defer_bias", False):       # the caller adds it where it adds the output itself
-                from .hybrid import Biased
                 return Biased(y, self.o_bias)
             y = ops.add_bias(y, self.o_bias, self.o.weight.dtype)
         return y

@@ -189,6 +189,7 @@ class Norm(Part):
         """
         raise NotImplementedError
 
+    # Optional: forward_terms(terms: TermSum, stream) -> (normalised x, new residual) of stream + the terms, all in one pass.
     # Optional: row_norm() -> (float32 weight, float32 bias or None, eps, whether the mean is taken off): what a kernel needs
     # to run the norm inside its own pass over the rows (`ops.stream_mix_norm`).
     # Optional: linear_behind(x, residual, weight, out_dtype, gated=False) -> (forward(x, residual)[0] . weight^T,
@@ -200,16 +201,24 @@ class PendingNorm:
     """A norm that has not run yet, in place of its output. A block hands one to a mixer or feed-forward
     that declares `takes_pending_norm = True`; such a part passes it to its first `Linear`, which may run
     norm and product as one kernel (`Norm.linear_behind`), or asks `value()` for the normed rows as a
-    tensor. Whichever happens first also yields the new residual, which the block reads afterwards."""
+    tensor. Whichever happens first also yields the new residual, which the block reads afterwards. x may
+    be a `TermSum`."""
 
-    def __init__(self, norm: "Norm", x: torch.Tensor, residual: torch.Tensor | None):
+    def __init__(self, norm: "Norm", x, residual: torch.Tensor | None):
         self.norm, self.x, self.residual = norm, x, residual
         self._y = None
         self._new_residual = None
 
+    def rows(self) -> int:
+        x = self.x.terms[0] if isinstance(self.x, TermSum) else self.x
+        return x.shape[-2]
+
     def value(self) -> torch.Tensor:
         if self._y is None:
             x = self.x
+            if isinstance(x, TermSum):
+                self._y, self._new_residual = x.normed(self.norm, self.residual)
+                return self._y
             if x.dim() == 3 and not getattr(self.norm, "accepts_partials", False):
                 x = x.sum(0)
             self._y, self._new_residual = self.norm.forward(x, self.residual)
@@ -219,7 +228,7 @@ class PendingNorm:
         """The product of the normed rows with `weight` ([out, in]) if the norm can run inside it, else None.
         gated: `weight` is a packed gate/up weight and the product is silu(gate) * up."""
         behind = getattr(self.norm, "linear_behind", None)
-        if self._y is not None or behind is None:
+        if self._y is not None or behind is None or isinstance(self.x, TermSum):
             return None
         got = behind(self.x, self.residual, weight, out_dtype, gated) if gated else behind(self.x, self.residual, weight, out_dtype)
         if got is None:
@@ -256,6 +265,62 @@ class ScaledSum:
         """The new stream, float32 [T, n]."""
         from ..kernels import ops
         return ops.scaled_sum_norm(stream, self.terms, self.mult, None, None, 0.0, torch.float32)[0]
+
+
+class Biased:
+    """A sublayer's output whose bias is still to be added: (rows or float32 partial sums, float32 bias [n]). A mixer or
+    feed-forward returns one only to a caller that asked for it (`defer_bias`) and adds it where it adds the output."""
+
+    def __init__(self, rows: torch.Tensor, bias: torch.Tensor):
+        self.rows, self.bias = rows, bias
+
+
+class TermSum:
+    """What a layer returns in place of its output when several terms still have to be added to the residual stream, each as it
+    is: rows [T, n], float32 partial sums [P, T, n], or a `Biased` of either. Whoever runs next forms the sum: a norm with
+    `forward_terms` in its own pass, the model's final norm at the wanted rows only (`normed_rows`), anyone else through
+    `settle`."""
+
+    MOST = 4                   # terms that one pass adds (`ops.stream_mix_norm`)
+
+    def __init__(self, terms: list):
+        self.terms, self.bias = [], None
+        for t in terms:
+            if isinstance(t, Biased):
+                self.bias = t.bias if self.bias is None else self.bias + t.bias
+                t = t.rows
+            self.terms.append(t)
+
+    def with_term(self, rows: torch.Tensor) -> "TermSum":
+        out = TermSum(self.terms + [rows])
+        out.bias = self.bias
+        return out
+
+    def _mix(self, stream, norm, out_dtype, rows=None, keep=True):
+        from ..kernels import ops
+        if stream is None:                    # the terms are the whole stream
+            stream = torch.zeros(self.terms[0].shape[-2:], dtype=torch.float32, device=self.terms[0].device)
+        terms = list(self.terms)
+        while len(terms) > self.MOST:
+            stream = ops.stream_mix_norm(stream, 1, terms[:self.MOST], None, None, None, None, torch.float32, keep=False)[1]
+            terms = terms[self.MOST:]
+        return ops.stream_mix_norm(stream.view(stream.shape[0], 1, -1), 1, terms, None, None, None, norm, out_dtype, rows=rows, keep=keep,
+                                   bias=self.bias)
+
+    def settle(self, stream: torch.Tensor | None) -> torch.Tensor:
+        """The new stream, float32 [T, n]."""
+        return self._mix(stream, None, torch.float32, keep=False)[1]
+
+    def normed(self, norm: "Norm", stream: torch.Tensor | None):
+        """(the norm of the new stream, the new stream)."""
+        forward_terms = getattr(norm, "forward_terms", None)
+        return forward_terms(self, stream) if forward_terms is not None else norm.forward(self.settle(stream), None)
+
+    def normed_rows(self, stream: torch.Tensor, norm: "Norm", rows: torch.Tensor):
+        """The norm of the new stream at `rows`, or None for a norm that no kernel can run inside."""
+        if not hasattr(norm, "row_norm"):
+            return None
+        return self._mix(stream, norm.row_norm(), norm.out_dtype, rows=rows, keep=False)[1]
 
 
 class StreamSum:
@@ -357,7 +422,8 @@ class Mixer(Part):
 class FeedForward(Part):
     def forward(self, x: torch.Tensor) -> torch.Tensor:
         """[T, hidden] -> [T, hidden], or float32 partial sums [P, T, hidden], or a tuple of such tensors whose sum is
-        the output (a routed part beside one that every token passes)."""
+        the output (a routed part beside one that every token passes); with `defer_bias` set by the caller, a `Biased` of
+        either of the first two."""
         raise NotImplementedError
 
 
@@ -386,10 +452,13 @@ class LayerCall:
     entries: its weights are then shared, each entry has a cache of its own).
     ``cache_of``: index of an *earlier entry* whose cache this entry reads
     instead of owning one; it then writes nothing.
+    ``add_start``: right before this entry the embedding's output (the stream as it was before the
+    first entry) is added to the stream once more.
     """
 
     layer: int
     cache_of: int | None = None
+    add_start: bool = False
 
 
 @dataclass

@@ -4,8 +4,8 @@ from __future__ import annotations
 import torch
 
 from ..kernels import ops
-from .base import (FeedForward, Mixer, Norm, ParamSpec, Part, PendingNorm, ScaledSum, Settled, StreamSum, few_tokens, register_part,
-                   side_branch)
+from .base import (Biased, FeedForward, Mixer, Norm, ParamSpec, Part, PendingNorm, ScaledSum, Settled, StreamSum, TermSum, few_tokens,
+                   register_part, side_branch)
 
 
 def one_tensor(x):
@@ -20,15 +20,28 @@ def one_tensor(x):
 
 
 def settled(h, residual):
-    """(h, residual) with a `ScaledSum` or `StreamSum` in place of h turned into a `Settled` stream."""
-    if isinstance(h, (ScaledSum, StreamSum)):
+    """(h, residual) with a `ScaledSum`, `StreamSum` or `TermSum` in place of h turned into a `Settled` stream."""
+    if isinstance(h, (ScaledSum, StreamSum, TermSum)):
         return Settled(None), h.settle(residual)
     return h, residual
 
 
+def with_start(h, residual, start):
+    """(h, residual) of a layer, with `start` added to the stream: (a `TermSum`, residual)."""
+    if isinstance(h, (ScaledSum, StreamSum)):
+        h, residual = settled(h, residual)
+    if isinstance(h, Settled):
+        return TermSum([start]), residual
+    if isinstance(h, TermSum):
+        return h.with_term(start), residual
+    return TermSum((list(h) if isinstance(h, (tuple, list)) else [h]) + [start]), residual
+
+
 def norm_of(norm: Norm, x, residual):
-    """Run a norm on x, which may be float32 partial sums [P, T, n] of a split product; a norm
-    that does not declare `accepts_partials` gets their sum."""
+    """Run a norm on x, which may be float32 partial sums [P, T, n] of a split product (a norm
+    that does not declare `accepts_partials` gets their sum) or a `TermSum`."""
+    if isinstance(x, TermSum):
+        return x.normed(norm, residual)
     x = one_tensor(x)
     if x.dim() == 3 and not getattr(norm, "accepts_partials", False):
         x = x.sum(0)
@@ -42,7 +55,8 @@ class PreNormBlock(Part):
 
     The layer's output is added to the residual by whoever runs next: the next block's first
     norm or the model's final norm (reference models/qwen3.py:65-74: the add lives inside the
-    norm call). The residual stream is float32.
+    norm call). The residual stream is float32. A feed-forward that returns several terms, or rows with a
+    bias to be added, leaves them as a `TermSum`: the norm that runs next adds them in its own pass.
     """
 
     def __init__(self, norm1: Norm, mixer: Mixer, norm2: Norm | None, feed_forward: FeedForward | None):
@@ -55,6 +69,7 @@ class PreNormBlock(Part):
         if feed_forward is not None:
             self.add_child("norm2", norm2)
             self.add_child("feed_forward", feed_forward)
+            feed_forward.defer_bias = True
         else:
             self.norm2 = self.feed_forward = None
 
@@ -65,7 +80,8 @@ class PreNormBlock(Part):
         return self.mixer.state_need()
 
     def forward(self, h, residual, step, cache, state):
-        h, residual = settled(h, residual)
+        if not isinstance(h, TermSum):
+            h, residual = settled(h, residual)
         if isinstance(h, Settled):          # the layer before has added its output already: the stream starts anew here
             h, residual = residual, None
         # a part that takes it gets the norm before it as a `PendingNorm` and may run it inside its first product
@@ -81,9 +97,15 @@ class PreNormBlock(Part):
         if getattr(self.feed_forward, "takes_pending_norm", False):
             x = PendingNorm(self.norm2, a, residual)
             out = self.feed_forward.forward(x)
-            return one_tensor(out), x.new_residual()
+            return _left_to_add(out), x.new_residual()
         x, residual = norm_of(self.norm2, a, residual)
-        return one_tensor(self.feed_forward.forward(x)), residual
+        return _left_to_add(self.feed_forward.forward(x)), residual
+
+
+def _left_to_add(out):
+    if isinstance(out, (tuple, list, Biased)):
+        return TermSum(list(out) if isinstance(out, (tuple, list)) else [out])
+    return out
 
 
 @register_part("block", "output_norm")
@@ -181,6 +203,8 @@ class ParallelBlock(Part):
         return self.mixer.state_need()
 
     def forward(self, h, residual, step, cache, state):
+        if isinstance(h, TermSum):
+            h, residual = settled(h, residual)
         if isinstance(h, ScaledSum):
             stream, terms, mult = residual, h.terms, h.mult
         elif isinstance(h, Settled):

@@ -4,7 +4,7 @@ from __future__ import annotations
 import torch
 
 from ..kernels import ops
-from .base import FeedForward, ParamSpec, PendingNorm, register_part
+from .base import Biased, FeedForward, ParamSpec, PendingNorm, register_part
 from .linear import Linear
 
 
@@ -23,20 +23,29 @@ class TokenGated:
 @register_part("feed_forward", "swiglu")
 class SwiGLU(FeedForward):
     """down(silu(gate(x)) * up(x)); gate and up are one packed product with gate's rows first
-    (reference layers/linear.py:29-45, layers/activation.py:5-7)."""
+    (reference layers/linear.py:29-45, layers/activation.py:5-7). `bias`: all three projections have biases; gate's and
+    up's join inside the activation's kernel, down's where the output is added to the stream."""
 
     takes_pending_norm = True      # x goes to the packed product and nowhere else
+    defer_bias = False             # the caller adds the output's bias itself (`Biased`)
 
-    def __init__(self, hidden_size: int, intermediate_size: int):
+    def __init__(self, hidden_size: int, intermediate_size: int, bias: bool = False):
         super().__init__()
         self.hidden_size = hidden_size
         self.intermediate_size = intermediate_size
+        self.biased = bool(bias)
+        if self.biased:
+            self.add_param("gate_up_bias", ParamSpec((2 * intermediate_size,), init="matrix", dtype="float32"))
+            self.add_param("down_bias", ParamSpec((hidden_size,), init="matrix", dtype="float32"))
         self.add_child("gate_up", Linear(hidden_size, 2 * intermediate_size,
                                          parts={"gate": intermediate_size, "up": intermediate_size}))
         self.add_child("down", Linear(intermediate_size, hidden_size))
 
     def forward(self, x):
-        rows = x.x.shape[-2] if isinstance(x, PendingNorm) else x.shape[0]
+        if self.biased:
+            y = self.down.forward(ops.silu_and_mul(self.gate_up.forward(x), bias=self.gate_up_bias), allow_partials=True)
+            return Biased(y, self.down_bias) if self.defer_bias else ops.add_bias(y, self.down_bias, self.down.weight.dtype)
+        rows = x.rows() if isinstance(x, PendingNorm) else x.shape[0]
         if ops.gated_linear_rows(rows, self.gate_up.weight):
             # few rows (or a few hundred over a small weight): the gating in the gate/up product's epilogue (every gate formed
             # once), a plain down product

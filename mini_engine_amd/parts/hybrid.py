@@ -13,7 +13,7 @@ import math
 import torch
 
 from ..kernels import ops
-from .base import Mixer, ParamSpec, StateNeed, few_tokens, register_part, side_branch
+from .base import Biased, Mixer, ParamSpec, StateNeed, few_tokens, register_part, side_branch
 from .linear import Linear
 
 
@@ -70,14 +70,6 @@ class SideBySide(Mixer):
             b = self.right.forward(x, step, *give(1))
         out = ScaledTerms([_term(a, self.left_scale), _term(b, self.right_scale)])
         return out if terms else out.value()
-
-
-class Biased:
-    """A mixer's output whose bias is still to be added: (rows or float32 partial sums, float32 bias [n]). A mixer returns
-    one only to a caller that asked for it (`defer_bias`); `SideBySide` does, and adds the bias inside its weighted sum."""
-
-    def __init__(self, rows: torch.Tensor, bias: torch.Tensor):
-        self.rows, self.bias = rows, bias
 
 
 def _term(y, scale: float) -> tuple:

@@ -26,8 +26,10 @@ class LatentAttention(Mixer):
     place in the packed product, its norm runs in the kernel that norms the cached latent). `sinks`: a learned number per
     head whose exponential joins the softmax's denominator without a key or a value.
 
-    `position`: a rotary encoding over `rot_dim` dimensions in adjacent pairs (its table is read as it stands; any scaling
-    of the positions lives there). q, the latent's rows and the gate are one packed product."""
+    `position`: a rotary encoding over `rot_dim` dimensions (its table is read as it stands; any scaling of the positions lives
+    there). The kernels turn adjacent pairs; where the stored pairs lie half the rotating part apart, `finalize` moves their rows
+    beside each other once, in the queries' projection and the shared key part's alike. q, the latent's rows and the gate are one
+    packed product."""
 
     takes_pending_norm = True      # x goes to the packed product and nowhere else
 
@@ -37,8 +39,8 @@ class LatentAttention(Mixer):
         super().__init__()
         if rot_dim % 2 or (rot_dim and position is None):
             raise ValueError("the rotating part has an even size and needs a position encoding")
-        if position is not None and (position.head_dim != rot_dim or position.rotary_dims != rot_dim or not position.interleaved):
-            raise ValueError("the position encoding must turn all of the rotating part, in adjacent pairs")
+        if position is not None and (position.head_dim != rot_dim or position.rotary_dims != rot_dim):
+            raise ValueError("the position encoding must turn all of the rotating part")
         self.hidden_size, self.num_heads, self.nope_dim, self.rot_dim = hidden_size, num_heads, nope_dim, rot_dim
         self.value_dim, self.rank, self.scale, self.norm_eps = value_dim, rank, float(scale), float(norm_eps)
         self.window, self.own_kv, self.output_gate = window, bool(own_kv), bool(output_gate)
@@ -73,6 +75,7 @@ class LatentAttention(Mixer):
         else:
             self.position = None
         self._uk_t = None
+        self._paired: dict = {}               # projections whose rotating rows lie in adjacent pairs already
 
     def cache_need(self):
         return CacheNeed.keys_and_values(1, self.head_dim, self.window)
@@ -84,9 +87,29 @@ class LatentAttention(Mixer):
     def finalize(self, device, dtype, max_positions):
         # W_uk[h]^T, [heads, rank, nope_dim]: the matrix that carries a head's unrotated query part into the latent's space
         self._uk_t = self.uk.view(self.num_heads, self.nope_dim, self.rank).transpose(1, 2).contiguous()
+        if self.position is not None and not self.position.interleaved:
+            if self.query_rank is None:
+                self._pair_rows(self.in_proj, True, self.kv_at)
+            else:
+                self._pair_rows(self.in_proj, False, self.kv_at)
+                self._pair_rows(self.uq, True, None)
         w = self.in_proj.weight
         if w.shape[0] % 8:                  # the packed rows in whole steps of 8: views of them keep 16-byte row strides
             self.in_proj.weight = torch.cat((w, w.new_zeros(8 - w.shape[0] % 8, w.shape[1])), 0).contiguous()
+            if self.in_proj in self._paired:
+                self._paired[self.in_proj] = self.in_proj.weight
+
+    def _pair_rows(self, linear, queries: bool, kv_at: int | None):
+        """The rotating rows of the query heads (from row 0 on) and of the shared key part reordered: i and i + rot_dim / 2 side by side."""
+        if self._paired.get(linear) is linear.weight:
+            return
+        H, dn, dr = self.num_heads, self.nope_dim, self.rot_dim
+        order = torch.arange(linear.weight.shape[0])
+        pairs = torch.stack((torch.arange(dr // 2), torch.arange(dr // 2) + dr // 2), 1).reshape(-1)
+        for at in ([h * (dn + dr) + dn for h in range(H)] if queries else []) + ([] if kv_at is None else [kv_at + self.rank]):
+            order[at:at + dr] = at + pairs
+        linear.weight = linear.weight[order.to(linear.weight.device)].contiguous()
+        self._paired[linear] = linear.weight
 
     def forward(self, x, step, cache, state):
         H, dn, dr, R, D, nv = self.num_heads, self.nope_dim, self.rot_dim, self.rank, self.head_dim, self.value_dim

@@ -9,7 +9,9 @@ from .base import FeedForward, ParamSpec, few_tokens, register_part, side_branch
 class RoutedExperts(FeedForward):
     """out = sum over the token's chosen experts e of weight_e * expert_e(x), plus, if there is one, a feed-forward that
     every token passes (`shared`, any `FeedForward`). An expert is W_down[e] (silu(W_gate[e] x) * (W_up[e] x)), or with
-    `gated=False` W_down[e] relu(W_up[e] x)^2.
+    `gated=False` W_down[e] relu(W_up[e] x)^2, or with `clamp` (limit, alpha) W_down[e] (g sigmoid(alpha g) (u + 1)) with the gate
+    g cut at limit from above and u = W_up[e] x at both sides (`ClampedGLU`'s form). `identity`: the router knows so many experts
+    more, behind the others, whose output is x itself; they have no weights.
 
     The router is float32. `scoring` "softmax": scores = softmax(W_router x) over all experts; "sigmoid": a sigmoid
     each; "chosen": the choice goes by the logits themselves and the weights are their softmax over the chosen experts alone.
@@ -32,30 +34,34 @@ class RoutedExperts(FeedForward):
     def __init__(self, hidden_size: int, intermediate_size: int, num_experts: int, top: int, group_count: int = 1,
                  group_keep: int = 1, shared: FeedForward | None = None, gated: bool = True, scoring: str = "softmax",
                  correction: bool = False, group_top: int = 1, normalise: bool = True, route_scale: float = 1.0,
-                 sum_outputs: bool = False, router_bias: bool = False):
+                 sum_outputs: bool = False, router_bias: bool = False, identity: int = 0, clamp: tuple | None = None):
         super().__init__()
-        if not 1 <= top <= num_experts:
-            raise ValueError(f"top {top} of {num_experts} experts")
-        if group_count < 1 or num_experts % group_count or not 1 <= group_keep <= group_count:
-            raise ValueError(f"{num_experts} experts do not form {group_count} equal groups of which {group_keep} are kept")
-        if group_keep * (num_experts // group_count) < top:
+        routed = num_experts + int(identity)
+        if num_experts < 1 or identity < 0 or not 1 <= top <= routed:
+            raise ValueError(f"top {top} of {num_experts} experts and {identity} identity experts")
+        if group_count < 1 or routed % group_count or not 1 <= group_keep <= group_count:
+            raise ValueError(f"{routed} experts do not form {group_count} equal groups of which {group_keep} are kept")
+        if group_keep * (routed // group_count) < top:
             raise ValueError("the kept groups hold fewer experts than a token uses")
         if scoring not in ops.RouteRule.SCORINGS or group_top < 1:
             raise ValueError(f"scoring is one of {sorted(ops.RouteRule.SCORINGS)}, group_top positive")
         self.hidden_size, self.intermediate_size = hidden_size, intermediate_size
         self.num_experts, self.top, self.group_count, self.group_keep = num_experts, top, group_count, group_keep
         self.gated, self.scoring, self.group_top = bool(gated), scoring, int(group_top)
+        self.identity, self.clamp = int(identity), (None if clamp is None else (float(clamp[0]), float(clamp[1])))
+        if self.clamp is not None and (not self.gated or not self.clamp[0] > 0):
+            raise ValueError("only a gate can be clamped, at a positive limit")
         self.normalise, self.route_scale, self.sum_outputs = bool(normalise), float(route_scale), bool(sum_outputs)
         rows = (2 if self.gated else 1) * intermediate_size
-        self.add_param("router", ParamSpec((num_experts, hidden_size), init="matrix", dtype="float32"))
+        self.add_param("router", ParamSpec((routed, hidden_size), init="matrix", dtype="float32"))
         self.add_param("gate_up", ParamSpec((num_experts * rows, hidden_size), init="matrix", dtype="compute"))
         self.add_param("down", ParamSpec((num_experts * hidden_size, intermediate_size), init="matrix", dtype="compute"))
         if router_bias:
-            self.add_param("router_bias", ParamSpec((num_experts,), init="matrix", dtype="float32"))
+            self.add_param("router_bias", ParamSpec((routed,), init="matrix", dtype="float32"))
         else:
             self.router_bias = None
         if correction:
-            self.add_param("correction", ParamSpec((num_experts,), init="matrix", dtype="float32"))
+            self.add_param("correction", ParamSpec((routed,), init="matrix", dtype="float32"))
         else:
             self.correction = None
         if shared is not None:
@@ -76,9 +82,10 @@ class RoutedExperts(FeedForward):
 
     def forward(self, x):
         E, F, h = self.num_experts, self.intermediate_size, self.hidden_size
+        clamp = {} if self.clamp is None else {"clamp": self.clamp}
         run = lambda: ops.route_and_run_experts(x, self.router, self.top, self.group_count, self.group_keep,
                                                 self.gate_up.view(E, (2 if self.gated else 1) * F, h), self.down.view(E, h, F),
-                                                rule=self.rule(), gated=self.gated)
+                                                rule=self.rule(), gated=self.gated, **clamp)
         if not self.sum_outputs:
             routed = run()
             return routed if self.shared is None else (routed, self.shared.forward(x))

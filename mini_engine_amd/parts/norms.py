@@ -11,6 +11,12 @@ def _around_zero(shape, generator, device):
     return torch.rand(shape, generator=generator, dtype=torch.float32, device=device) * 0.2 - 0.1
 
 
+def _norm_of_terms(norm, terms, stream):
+    """stream + the terms of a `TermSum`, and that sum's norm, in one pass."""
+    new, y = terms._mix(stream, norm.row_norm(), norm.out_dtype)
+    return y, new.view(new.shape[0], -1)
+
+
 @register_part("norm", "rms")
 class RMSNorm(Norm):
     """y = weight * r / sqrt(mean(r^2) + eps), r = x + residual.
@@ -55,6 +61,9 @@ class RMSNorm(Norm):
     def row_norm(self):
         return self.weight, None, self.eps, False
 
+    def forward_terms(self, terms, stream):
+        return _norm_of_terms(self, terms, stream)
+
     def forward(self, x, residual, want_residual: bool = True):
         return ops.rms_norm(x, self.weight, self.eps, residual, self.out_dtype, want_residual)
 
@@ -66,15 +75,19 @@ class RMSNorm(Norm):
 
 @register_part("norm", "layer")
 class LayerNorm(Norm):
-    """y = weight * (r - mean(r)) / sqrt(mean((r - mean(r))^2) + eps) + bias, r = x + residual, all in float32."""
+    """y = weight * (r - mean(r)) / sqrt(mean((r - mean(r))^2) + eps) + bias, r = x + residual, all in float32. `bias` False:
+    the design has none."""
 
     accepts_partials = True
 
-    def __init__(self, size: int, eps: float):
+    def __init__(self, size: int, eps: float, bias: bool = True):
         super().__init__()
         self.size, self.eps = size, eps
         self.add_param("weight", ParamSpec((size,), init="norm", dtype="float32"))
-        self.add_param("bias", ParamSpec((size,), init=_around_zero, dtype="float32"))
+        if bias:
+            self.add_param("bias", ParamSpec((size,), init=_around_zero, dtype="float32"))
+        else:
+            self.bias = None
         self.out_dtype = torch.float32
 
     def finalize(self, device, dtype, max_positions):
@@ -83,10 +96,13 @@ class LayerNorm(Norm):
     def row_norm(self):
         return self.weight, self.bias, self.eps, True
 
+    def forward_terms(self, terms, stream):
+        return _norm_of_terms(self, terms, stream)
+
     def forward(self, x, residual):
         if residual is None:
             x = x.sum(0) if x.dim() == 3 else x
-            stream, terms = x, []
+            stream, terms = (x.view(x.shape[0], 1, -1) if x.dtype == torch.float32 else x), []
         else:
             stream, terms = residual.view(residual.shape[0], 1, -1), [x]
         new, y = ops.stream_mix_norm(stream, 1, terms, None, None, None, self.row_norm(), self.out_dtype)

@@ -34,9 +34,10 @@ def rms_norm(x, weight, eps, residual, out_dtype, want_residual=True):
     return y.to(out_dtype), (r if want_residual else None)
 
 
-def silu_and_mul(gu):
+def silu_and_mul(gu, bias=None):
     inter = gu.shape[1] // 2
-    g, u = gu[:, :inter].float(), gu[:, inter:].float()
+    r = gu.float() if bias is None else gu.float() + bias
+    g, u = r[:, :inter], r[:, inter:]
     return (g * torch.sigmoid(g) * u).to(gu.dtype)
 
 
@@ -63,7 +64,7 @@ def write_pages(k, v, slots, k_cache, v_cache, page):
 
 
 def qk_norm_rope_store(qkv, q_weight, k_weight, eps, table, positions, slots, k_cache, v_cache,
-                       Hq, Hkv, D, page, store=True, position_bound=0):
+                       Hq, Hkv, D, page, store=True, position_bound=0, values_are_keys=False):
     T = qkv.shape[0]
     if table is not None:
         # what the kernel's launcher refuses, and what it could not see: a position beyond the table
@@ -74,7 +75,7 @@ def qk_norm_rope_store(qkv, q_weight, k_weight, eps, table, positions, slots, k_
         k = _norm_rope(qkv[:, Hq * D:(Hq + Hkv) * D].float().clone().view(T, Hkv, D), k_weight, eps, table, positions)
     qkv[:, :Hq * D] = q.reshape(T, Hq * D).to(qkv.dtype)
     if store:
-        v = qkv[:, (Hq + Hkv) * D:].view(T, Hkv, D)
+        v = qkv[:, Hq * D if values_are_keys else (Hq + Hkv) * D:].view(T, Hkv, D)
         write_pages(k.to(qkv.dtype), v, slots, k_cache, v_cache, page)
     elif Hkv:
         qkv[:, Hq * D:(Hq + Hkv) * D] = k.reshape(T, Hkv * D).to(qkv.dtype)
@@ -87,7 +88,7 @@ def store_kv(k, v, slots, k_cache, v_cache, page):
 def paged_attention(q, k_cache, v_cache, page, block_tables, context_lens, seq_of_token, positions,
                     prefill_cu, num_decodes, max_decode_context, scale, window, Hq, Hkv, D,
                     force_simple=False, max_prefill_context=0, even_contexts=False, compute_dtype=torch.float32,
-                    chunk=None, decode_as_prefill=False, keep_first=0, softcap=None, sinks=None):
+                    chunk=None, decode_as_prefill=False, keep_first=0, softcap=None, sinks=None, slopes=None):
     """Token by token: gather the keys this token may see through its request's block table
     and nothing else (so unowned pages are never read), softmax, weighted sum."""
     T = q.shape[0]
@@ -115,6 +116,8 @@ def paged_attention(q, k_cache, v_cache, page, block_tables, context_lens, seq_o
         s = torch.einsum("nkd,kgd->kgn", k, qt) * scale
         if softcap:
             s = softcap * torch.tanh(s / softcap)
+        if slopes is not None:                             # what a head takes off per token of distance
+            s = s - slopes.to(compute_dtype).view(Hkv, G, 1) * (pos - js).to(compute_dtype)
         if sinks is not None:                              # one more term in the denominator, no key, no value
             s = torch.cat((s, sinks.to(compute_dtype).view(Hkv, G, 1)), dim=-1)
             p = torch.softmax(s, dim=-1)[..., :-1]
@@ -126,7 +129,7 @@ def paged_attention(q, k_cache, v_cache, page, block_tables, context_lens, seq_o
 
 def decode_step_attention(qkv, q_weight, k_weight, eps, table, k_cache, v_cache, page, block_tables, context_lens,
                           max_context, scale, window, Hq, Hkv, D, even_contexts=False, compute_dtype=torch.float32,
-                          chunk=None):
+                          chunk=None, sinks=None, slopes=None, values_are_keys=False):
     """The two twins above, one after the other, on a copy of the rows: row r is request r's new token at
     position context_lens[r] - 1, its slot is what the block table names for that position (a row with
     context 0 is padding: nothing is written for it and it sees nothing)."""
@@ -137,10 +140,11 @@ def decode_step_attention(qkv, q_weight, k_weight, eps, table, k_cache, v_cache,
     pages = block_tables[torch.arange(B, device=qkv.device), (positions // page).long()].long()
     slots = torch.where((ctx > 0) & (pages >= 0), pages * page + positions.long() % page, torch.full_like(pages, -1)).to(torch.int32)
     rows = qkv.clone()
-    qk_norm_rope_store(rows, q_weight, k_weight, eps, table, positions, slots, k_cache, v_cache, Hq, Hkv, D, page, store=True)
+    qk_norm_rope_store(rows, q_weight, k_weight, eps, table, positions, slots, k_cache, v_cache, Hq, Hkv, D, page, store=True,
+                       values_are_keys=values_are_keys)
     seq = torch.arange(B, dtype=torch.int32, device=qkv.device)
     return paged_attention(rows[:, :Hq * D], k_cache, v_cache, page, block_tables, context_lens, seq, positions, None, B,
-                           max_context, scale, window, Hq, Hkv, D, compute_dtype=compute_dtype, chunk=chunk)
+                           max_context, scale, window, Hq, Hkv, D, compute_dtype=compute_dtype, chunk=chunk, sinks=sinks, slopes=slopes)
 
 
 def linear(x, w, out_dtype=None, allow_partials=False, out=None):
@@ -275,12 +279,14 @@ def memory_readout(reads, gate, weight, eps, heads, q_scale, out_dtype):
     return (o * weight * torch.sigmoid(gate.float())).to(out_dtype)
 
 
-def stream_mix_norm(streams, count, terms, mix, out_weights, read, norm, out_dtype, rows=None, keep=True):
+def stream_mix_norm(streams, count, terms, mix, out_weights, read, norm, out_dtype, rows=None, keep=True, bias=None):
     """Streams [T, S, n] (or rows that all share): mixed, the terms added, read, normed; all in float32."""
     x = streams.float()
     if x.dim() == 2:
         x = x[:, None, :].expand(-1, count, -1)
     y = sum((t.float().sum(0) if t.dim() == 3 else t.float()) for t in terms) if terms else None
+    if bias is not None:
+        y = bias[None, :] + (0 if y is None else y)
     if mix is not None:
         x = torch.einsum("st,bsn->btn", mix, x) + (0 if y is None else out_weights[None, :, None] * y[:, None, :])
     elif y is not None:
@@ -482,12 +488,13 @@ def moe_route(x, router, top, group_count=1, group_keep=1, rule=None):
     return ids.to(torch.int32), (w * (1.0 if rule is None else rule.scale)).float()
 
 
-def route_and_run_experts(x, router, top, group_count, group_keep, gate_up, down, rule=None, gated=True):
+def route_and_run_experts(x, router, top, group_count, group_keep, gate_up, down, rule=None, gated=True, clamp=None):
     ids, weights = moe_route(x, router, top, group_count, group_keep, rule)
-    return routed_experts(x, ids, weights, gate_up, down, gated=gated)
+    return routed_experts(x, ids, weights, gate_up, down, gated=gated, clamp=clamp, routed=router.shape[0])
 
 
-def routed_experts(x, ids, weights, gate_up, down, force_simple=False, tile_rows=None, choose_from=None, gated=True):
+def routed_experts(x, ids, weights, gate_up, down, force_simple=False, tile_rows=None, choose_from=None, gated=True, clamp=None,
+                   routed=None):
     T, K = x.shape
     top = ids.shape[1]
     F = gate_up.shape[1] // 2 if gated else gate_up.shape[1]
@@ -496,8 +503,14 @@ def routed_experts(x, ids, weights, gate_up, down, force_simple=False, tile_rows
     for j in range(top):
         for e in ids[:, j].unique().tolist():
             rows = (ids[:, j] == e).nonzero().flatten()
+            if e >= gate_up.shape[0]:                      # an identity expert
+                out[j, rows] = xf[rows] * weights[rows, j][:, None]
+                continue
             gu = xf[rows] @ gate_up[e].float().t()
-            act = gu[:, :F] * torch.sigmoid(gu[:, :F]) * gu[:, F:] if gated else torch.relu(gu) ** 2
+            if clamp is not None:
+                act = glu_clamped(gu, *clamp)
+            else:
+                act = gu[:, :F] * torch.sigmoid(gu[:, :F]) * gu[:, F:] if gated else torch.relu(gu) ** 2
             out[j, rows] = (act.to(x.dtype).float() @ down[e].float().t()) * weights[rows, j][:, None]
     return out
 
