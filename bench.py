@@ -83,9 +83,10 @@ def _matrix_params(model) -> tuple:
 
 def _routed_share(part, local: str, tokens: int) -> float:
     """The share of a parameter that a step of `tokens` tokens reads: 1, or for the packed expert matrices of a routed
-    feed-forward the expected share of experts that some token chooses (choices taken as uniform over the experts; one
-    token: top / experts)."""
+    feed-forward the expected share of experts that some token chooses (choices taken as uniform over the experts,
+    identity experts included; one token: top / experts)."""
     experts, top = getattr(part, "num_experts", None), getattr(part, "top", None)
+    experts = experts and experts + getattr(part, "identity", 0)
     if not experts or local not in ("gate_up", "down"):
         return 1.0
     return 1.0 - (1.0 - top / experts) ** tokens
@@ -99,11 +100,13 @@ def cache_bytes_per_token(model, page: int, dtype) -> list:
 
 
 def decode_bytes(model, item: int, contexts: list, page: int, dtype) -> int:
-    """Bytes one decode step has to read: every parameter it uses once (the embedding matrix only where it is the
-    head's matrix as well: a step gathers a row per request from it), and what the cache holds of the live requests
-    (a windowed group at most its window)."""
+    """Bytes one decode step has to read: every parameter it uses once, a layer's once per run (the embedding matrix only
+    where it is the head's matrix as well: a step gathers a row per request from it), and what the cache holds of the live
+    requests (a windowed group at most its window)."""
     tied = getattr(model.head, "tied_to", None) is model.embedding
-    weights = sum(_spec_bytes(spec, item) * _routed_share(part, local, len(contexts)) for name, part, local, spec in model.named_specs()
+    runs = _used_per_call(model)
+    times = lambda name: runs.get(int(name.split(".")[1]), 0) if name.startswith("layers.") else 1
+    weights = sum(_spec_bytes(spec, item) * times(name) * _routed_share(part, local, len(contexts)) for name, part, local, spec in model.named_specs()
                   if tied or not name.startswith("embedding."))
     kv = 0.0
     for per_token, window in cache_bytes_per_token(model, page, dtype):

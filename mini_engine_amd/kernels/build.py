@@ -36,7 +36,7 @@ HEADERS = ["common.h", "errors.inc", "sampling.h"]
 # Head sizes that build_all() compiles ahead of use; any other multiple of 16 up to 512 is compiled when a model first needs it.
 DEFAULT_HEAD_DIMS = (16, 32, 48, 64, 80, 128, 256)
 CAPPED_HEAD_DIMS = (32, 64, 128)          # ... of the variant with a cap on the scores
-DISTANCE_HEAD_DIMS = (32, 48, 128)        # ... of the variant with slopes times distances
+DISTANCE_HEAD_DIMS = (16, 32, 48, 64, 128)          # ... of the variant with slopes times distances
 
 _locks: dict = {}
 _locks_guard = threading.Lock()

@@ -51,6 +51,23 @@ def test_a_window_bounds_what_a_decode_step_reads_and_what_a_prompt_computes():
     assert linear > 0 and abs(linear - bench.prefill_flops(model, 50) + 2 * full + 2 * windowed) < 1e-6
 
 
+def test_layers_that_run_twice_and_experts_without_weights():
+    from mini_engine_amd.config.model_config import VenezenConfig
+    from mini_engine_amd.registry import build_model
+    moe = {"kind": "moe", "expert": {"ff": 8, "limit": 1.0}, "router": {"experts": 6, "identity": 2, "top": 2, "scale": 1.0}}
+    raw = {"architecture": "Venezen", "vocab": 64, "width": 16, "norm": {"eps": 1e-5}, "embedding": {"scale": 1.0}, "layers": [
+        {"type": "attention", "mlp": moe, "mixer": {"heads": 2, "kv_heads": 1, "dim": 16, "vdim": 16, "scale": 0.25, "mask": {"size": 9}}}]}
+    once, twice = build_model(VenezenConfig.from_dict(raw)), build_model(VenezenConfig.from_dict(dict(raw, loop={"start": 0, "stop": 1, "times": 2})))
+    fixed = (64 * 16) * 2 + 16 * 4                                            # the tied table and the final norm
+    layer = ((3 * 16 * 16) + 16 * 32) * 2 + (2 * 16 + 8 * 16 + 8) * 4         # q and k, o; norms, router and correction
+    expert = 3 * 8 * 16 * 2
+    cache = 2 * 16 * 2 * 9                                                    # keys and values of one head under the window
+    assert bench.decode_bytes(once, 2, [20], 16, torch.bfloat16) == fixed + layer + 6 * expert * 2 // 8 + cache
+    assert bench.decode_bytes(twice, 2, [20], 16, torch.bfloat16) == fixed + 2 * (layer + 6 * expert * 2 // 8 + cache)
+    flops = lambda m: bench.prefill_flops(m, 1) - 2.0 * 64 * 16
+    assert flops(twice) == 2 * flops(once)
+
+
 def test_more_than_one_gpu_is_refused_with_one_line(capsys):
     assert bench.main(["--gpus", "2"]) == 2
     out = capsys.readouterr().out.strip().splitlines()

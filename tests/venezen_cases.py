@@ -241,12 +241,22 @@ def real_sizes(env_f32, env_bf16, name="real", every_row=True):
 
 def window_edges(env, name, window_layer, at=90):
     """A query just inside and just outside a window: the token whose key lies exactly at the edge is changed, in a prompt and with
-    the query decoded alone. In a model of that one layer, run once, the logits move inside the window and stay outside."""
+    the query decoded alone. In a model of that one layer, run once, the logits move inside the window and stay outside. Of all
+    tokens that may stand at the edge, the pair whose keys matter most to the query at the edge is taken."""
     window = CONFIGS[name]["layers"][window_layer]["mixer"]["mask"]["size"]
     V = CONFIGS[name]["vocab"]
     ids = random_ids(at + window + 2, V, 640)
+    folder, edge = env.folders(name), at + window - 1
+    rows = []
+    for token in range(V):
+        ids[at] = token
+        rows.append(plain_logits(folder, ids[:edge + 1])[edge])
+    apart = (torch.stack(rows)[:, None] - torch.stack(rows)[None]).abs().amax(-1)
+    one, two = divmod(int(apart.argmax()), V)
     other = list(ids)
-    other[at] = (other[at] + 1) % V
+    ids[at], other[at] = one, two
+    shows = float(apart.max() / torch.stack(rows).abs().max())
+    assert shows > 1e-2, "no key at the edge matters"
     out = {}
     for key, tokens in (("a", ids), ("b", other)):
         runner, manager, folder = env.runner(name, 2 * -(-len(ids) // PAGE[name]), 2)
@@ -261,5 +271,5 @@ def window_edges(env, name, window_layer, at=90):
             CUTS.check(env, folder, tokens, got, f"{name} window edge")
     for a, b in zip(out["a"], out["b"]):
         moved = (a - b).abs().amax(-1) / a.abs().max()
-        assert float(moved[at + window - 1]) > 0, "the last query that sees the key"
-        assert float(moved[at + window]) == 0, "the first query that does not"
+        assert float(moved[edge]) > 0.3 * shows, "the last query that sees the key"
+        assert float(moved[edge + 1]) == 0, "the first query that does not"
