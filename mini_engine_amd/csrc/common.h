@@ -67,3 +67,20 @@ __device__ __forceinline__ float block_sum(float v, float* scratch) {
   for (int w = 0; w < nwaves; ++w) total += scratch[w];
   return total;
 }
+
+// What a gated feed-forward makes of a gate and its up value: silu(gate) * up, or with limit > 0 and g = min(gate, limit),
+// u = clamp(up, -limit, limit): g sigmoid(alpha g) (u + 1). bias: float32 [2 I] (the gates', then the ups') that joins both
+// first, or null.
+struct GateForm { float limit, alpha; const float* bias; };
+// FAST: the hardware's exponential (for results that are rounded to bfloat16).
+template <bool FAST>
+__device__ __forceinline__ float gate_value(float gate, float up, const GateForm& form) {
+  float alpha = 1.f;
+  if (form.limit > 0.f) {
+    gate = fminf(gate, form.limit);
+    up = fminf(fmaxf(up, -form.limit), form.limit) + 1.f;
+    alpha = form.alpha;
+  }
+  const float e = FAST ? __expf(-alpha * gate) : expf(-alpha * gate);
+  return gate / (1.f + e) * up;
+}

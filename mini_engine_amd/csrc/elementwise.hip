@@ -344,10 +344,11 @@ extern "C" int me_rms_norm(const void* x, int x_dtype, int num_partials, int64_t
 }
 
 // ------------------------------------------------------------------ SiLU(gate) * up
-// gu: [T, 2I] with gate = first I columns (reference layers/activation.py:6); out: [T, I].
-// VEC: a thread takes 16 bytes of gate and of up at a time (I a multiple of the vector length).
-template <typename T, bool VEC>
-__global__ void silu_and_mul_kernel(const T* __restrict__ gu, const float* __restrict__ bias, T* __restrict__ out, int64_t rows, int inter) {
+// gu: [T, 2I] with gate = first I columns (reference layers/activation.py:6), rows gu_stride apart; out: [T, I].
+// VEC: a thread takes 16 bytes of gate and of up at a time (I a multiple of the vector length). PLAIN: silu(gate) * up, known to the
+// compiler (5.7 against 5.1 TB/s with the form asked for at run time).
+template <typename T, bool VEC, bool PLAIN>
+__global__ void gate_mul_kernel(const T* __restrict__ gu, int64_t gu_stride, GateForm form, T* __restrict__ out, int64_t rows, int inter) {
   constexpr int W = VEC ? 16 / sizeof(T) : 1;
   const int per_row = inter / W;
   const int64_t total = rows * (int64_t)per_row;
@@ -357,42 +358,80 @@ __global__ void silu_and_mul_kernel(const T* __restrict__ gu, const float* __res
     const int i = (int)(e - t * per_row) * W;
     alignas(16) T g[W], u[W], o[W];
     if (VEC) {
-      *reinterpret_cast<uint4*>(g) = *reinterpret_cast<const uint4*>(gu + t * 2 * inter + i);
-      *reinterpret_cast<uint4*>(u) = *reinterpret_cast<const uint4*>(gu + t * 2 * inter + inter + i);
+      *reinterpret_cast<uint4*>(g) = *reinterpret_cast<const uint4*>(gu + t * gu_stride + i);
+      *reinterpret_cast<uint4*>(u) = *reinterpret_cast<const uint4*>(gu + t * gu_stride + inter + i);
     } else {
-      g[0] = gu[t * 2 * inter + i];
-      u[0] = gu[t * 2 * inter + inter + i];
+      g[0] = gu[t * gu_stride + i];
+      u[0] = gu[t * gu_stride + inter + i];
     }
 #pragma unroll
     for (int j = 0; j < W; ++j) {
       float gf = to_f32<T>(g[j]), uf = to_f32<T>(u[j]);
-      if (bias) { gf += bias[i + j]; uf += bias[inter + i + j]; }
-      o[j] = from_f32<T>(gf / (1.f + expf(-gf)) * uf);
+      if (PLAIN) {
+        o[j] = from_f32<T>(gf / (1.f + expf(-gf)) * uf);
+      } else {
+        if (!VEC && form.bias) { gf += form.bias[i]; uf += form.bias[inter + i]; }
+        o[j] = from_f32<T>(gate_value<false>(gf, uf, form));
+      }
     }
     if (VEC) *reinterpret_cast<uint4*>(out + t * inter + i) = *reinterpret_cast<const uint4*>(o);
     else out[t * inter + i] = o[0];
   }
 }
 
-// bias: float32 [2 I] (the gates', then the ups') that joins gu first, or null
-extern "C" int me_silu_and_mul(const void* gu, const float* bias, void* out, int dtype, int64_t rows, int inter,
-                               hipStream_t stream) {
-  if (rows == 0) return 0;
-  ME_CHECK(inter > 0, "silu_and_mul: intermediate size must be positive");
-  ME_CHECK(dtype == ME_BF16 || dtype == ME_F32, "silu_and_mul: bad dtype code %d", dtype);
-  const int w = dtype == ME_BF16 ? 8 : 4;
-  const bool vec = inter % w == 0 && reinterpret_cast<uintptr_t>(gu) % 16 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0;
-  const int64_t total = rows * (int64_t)(vec ? inter / w : inter);
+// The same with biases: a thread keeps its columns' biases and walks down the rows.
+template <typename T>
+__global__ void __launch_bounds__(256)
+gate_mul_rows_kernel(const T* __restrict__ gu, int64_t gu_stride, GateForm form, T* __restrict__ out, int64_t rows, int inter) {
+  constexpr int W = 16 / sizeof(T);
+  const int i = (blockIdx.x * blockDim.x + threadIdx.x) * W;
+  if (i >= inter) return;
+  float bg[W], bu[W];
+#pragma unroll
+  for (int j = 0; j < W; ++j) { bg[j] = form.bias[i + j]; bu[j] = form.bias[inter + i + j]; }
+  for (int64_t t = blockIdx.y; t < rows; t += gridDim.y) {
+    alignas(16) T g[W], u[W], o[W];
+    *reinterpret_cast<uint4*>(g) = *reinterpret_cast<const uint4*>(gu + t * gu_stride + i);
+    *reinterpret_cast<uint4*>(u) = *reinterpret_cast<const uint4*>(gu + t * gu_stride + inter + i);
+#pragma unroll
+    for (int j = 0; j < W; ++j) o[j] = from_f32<T>(gate_value<false>(to_f32<T>(g[j]) + bg[j], to_f32<T>(u[j]) + bu[j], form));
+    *reinterpret_cast<uint4*>(out + t * inter + i) = *reinterpret_cast<const uint4*>(o);
+  }
+}
+
+template <typename T>
+static void launch_gate_mul(const T* gu, int64_t gu_stride, const GateForm& form, T* out, int64_t rows, int inter, hipStream_t stream) {
+  constexpr int W = 16 / sizeof(T);
+  const bool vec = inter % W == 0 && gu_stride % W == 0 && reinterpret_cast<uintptr_t>(gu) % 16 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0;
+  if (vec && form.bias) {
+    const int columns = inter / W;
+    const int threads = columns >= 256 ? 256 : (columns + 63) / 64 * 64;
+    const int64_t gx = (columns + threads - 1) / threads;
+    int64_t gy = 8192 / gx;                        // a few rows to a workgroup once there are many
+    if (gy > rows) gy = rows;
+    gate_mul_rows_kernel<T><<<dim3((unsigned)gx, (unsigned)(gy < 1 ? 1 : gy)), dim3(threads), 0, stream>>>(gu, gu_stride, form, out, rows, inter);
+    return;
+  }
+  const int64_t total = rows * (int64_t)(vec ? inter / W : inter);
   int64_t blocks = (total + 255) / 256;
   if (blocks > 65536) blocks = 65536;
-  dim3 grid(blocks), block(256);
-  if (dtype == ME_BF16) {
-    if (vec) silu_and_mul_kernel<bf16_t, true><<<grid, block, 0, stream>>>((const bf16_t*)gu, bias, (bf16_t*)out, rows, inter);
-    else silu_and_mul_kernel<bf16_t, false><<<grid, block, 0, stream>>>((const bf16_t*)gu, bias, (bf16_t*)out, rows, inter);
-  } else {
-    if (vec) silu_and_mul_kernel<float, true><<<grid, block, 0, stream>>>((const float*)gu, bias, (float*)out, rows, inter);
-    else silu_and_mul_kernel<float, false><<<grid, block, 0, stream>>>((const float*)gu, bias, (float*)out, rows, inter);
-  }
+#define GM(V, PL) gate_mul_kernel<T, V, PL><<<dim3((unsigned)blocks), dim3(256), 0, stream>>>(gu, gu_stride, form, out, rows, inter)
+  const bool plain = form.bias == nullptr && form.limit == 0.f;
+  if (vec) { if (plain) GM(true, true); else GM(true, false); }
+  else { if (plain) GM(false, true); else GM(false, false); }
+#undef GM
+}
+
+// bias: float32 [2 I] (the gates', then the ups') that joins gu first, or null; limit, alpha: see `GateForm` (limit 0: silu)
+extern "C" int me_gate_mul(const void* gu, int64_t gu_stride, const float* bias, float limit, float alpha, void* out, int dtype, int64_t rows,
+                           int inter, hipStream_t stream) {
+  if (rows == 0) return 0;
+  ME_CHECK(inter > 0 && gu_stride >= 2 * (int64_t)inter, "gate_mul: rows of a positive intermediate size's gates and ups");
+  ME_CHECK(limit >= 0.f, "gate_mul: the limit must not be negative");
+  ME_CHECK(dtype == ME_BF16 || dtype == ME_F32, "gate_mul: bad dtype code %d", dtype);
+  const GateForm form{limit, alpha, bias};
+  if (dtype == ME_BF16) launch_gate_mul<bf16_t>((const bf16_t*)gu, gu_stride, form, (bf16_t*)out, rows, inter, stream);
+  else launch_gate_mul<float>((const float*)gu, gu_stride, form, (float*)out, rows, inter, stream);
   ME_LAUNCH_CHECK();
   return 0;
 }

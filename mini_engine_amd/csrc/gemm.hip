@@ -163,7 +163,7 @@ template <int MT, typename TO, bool GATED, bool EXACT_K, bool ACT = false, bool 
 __global__ void __launch_bounds__(256, WIDE ? 5 : 1)
 gemm_skinny_kernel(const bf16_t* __restrict__ x, int64_t ldx, const bf16_t* __restrict__ w, int64_t ldw,
                    TO* __restrict__ y, int64_t ldy, float* __restrict__ partials, int M, int N, int K,
-                   int steps_per_split) {
+                   int steps_per_split, GateForm form) {
   static_assert(!WIDE || (MT == 1 && !GATED && EXACT_K), "the wide loads are built for one tile of tokens and whole steps");
   __shared__ float red[4][MT][256];
   __shared__ __align__(16) unsigned char wtile[WIDE ? 4 : 1][WIDE ? WIDE_TILE_BYTES : 16];
@@ -280,9 +280,10 @@ gemm_skinny_kernel(const bf16_t* __restrict__ x, int64_t ldx, const bf16_t* __re
     const int idx = threadIdx.x, m = idx >> 3, f = idx & 7;
     if (idx < 128 && m0 + m < M && n0 + f < half) {
       const int ig = m * 16 + f, iu = ig + 8;
-      const float gate = red[0][0][ig] + red[1][0][ig] + red[2][0][ig] + red[3][0][ig];
-      const float up = red[0][0][iu] + red[1][0][iu] + red[2][0][iu] + red[3][0][iu];
-      y[(int64_t)(m0 + m) * ldy + n0 + f] = from_f32<TO>(gate / (1.f + expf(-gate)) * up);
+      float gate = red[0][0][ig] + red[1][0][ig] + red[2][0][ig] + red[3][0][ig];
+      float up = red[0][0][iu] + red[1][0][iu] + red[2][0][iu] + red[3][0][iu];
+      if (form.bias) { gate += form.bias[n0 + f]; up += form.bias[half + n0 + f]; }
+      y[(int64_t)(m0 + m) * ldy + n0 + f] = from_f32<TO>(gate_value<false>(gate, up, form));
     }
     return;
   }
@@ -461,11 +462,14 @@ extern "C" int me_gemm_rows_bf16(const void* x, int64_t ldx, const void* w, int6
 
 // y: bf16 or float32 [M, N]; or, when ksplit > 1, `partials` float32 [ksplit, M, N] (y unused).
 // gated: x is [M, 2K] and silu(x[:, :K]) * x[:, K:] is what is multiplied. act: w is a packed gate/up weight and y
-// is silu(gate) * up, [M, N / 2] (at most 16 rows, K not split, not together with gated).
+// is silu(gate) * up, [M, N / 2] (at most 16 rows, K not split, not together with gated); limit, alpha, bias: another
+// `GateForm` than that.
 extern "C" int me_gemm_skinny_bf16(const void* x, int64_t ldx, const void* w, int64_t ldw, void* y,
                                    int64_t ldy, int out_dtype, float* partials, int ksplit, int M, int N,
-                                   int K, int gated, int act, int wide, hipStream_t stream) {
+                                   int K, int gated, int act, int wide, float limit, float alpha, const float* bias, hipStream_t stream) {
   if (M == 0 || N == 0) return 0;
+  ME_CHECK(act || (limit == 0.f && bias == nullptr), "skinny gemm: limits and biases belong to the gating epilogue");
+  const GateForm form{limit, alpha, bias};
   // wide: the caller asks for the wide loads (large weights); they apply to one tile of tokens, K in whole steps of
   // 128, an ungated input and a weight under 2 GB, and are left out otherwise
   const bool wide_ok = wide && M <= 16 && !gated && K % 128 == 0 && (int64_t)(N - 1) * ldw + K <= (int64_t)0x3fffffff;
@@ -480,10 +484,10 @@ extern "C" int me_gemm_skinny_bf16(const void* x, int64_t ldx, const void* w, in
     dim3 grid((N / 2 + 7) / 8, 1, 1), block(256);
 #define LAUNCH_ACT(TO, E)                                                                                    \
   gemm_skinny_kernel<1, TO, false, E, true><<<grid, block, 0, stream>>>((const bf16_t*)x, ldx, (const bf16_t*)w, ldw, \
-                                                                        (TO*)y, ldy, nullptr, M, N, K, steps)
+                                                                        (TO*)y, ldy, nullptr, M, N, K, steps, form)
     if (out_dtype == ME_BF16 && wide_ok) {
       gemm_skinny_kernel<1, bf16_t, false, true, true, true><<<grid, block, 0, stream>>>(
-          (const bf16_t*)x, ldx, (const bf16_t*)w, ldw, (bf16_t*)y, ldy, nullptr, M, N, K, steps);
+          (const bf16_t*)x, ldx, (const bf16_t*)w, ldw, (bf16_t*)y, ldy, nullptr, M, N, K, steps, form);
     } else if (out_dtype == ME_BF16) { if (K % 128 == 0) LAUNCH_ACT(bf16_t, true); else LAUNCH_ACT(bf16_t, false); }
     else if (out_dtype == ME_F32) { if (K % 128 == 0) LAUNCH_ACT(float, true); else LAUNCH_ACT(float, false); }
     else ME_CHECK(false, "skinny gemm: bad output dtype code %d", out_dtype);
@@ -506,7 +510,7 @@ extern "C" int me_gemm_skinny_bf16(const void* x, int64_t ldx, const void* w, in
   const bool exact = K % 128 == 0;
 #define LAUNCH1(MTV, TO, G, E)                                                                               \
   gemm_skinny_kernel<MTV, TO, G, E><<<grid, block, 0, stream>>>((const bf16_t*)x, ldx, (const bf16_t*)w, ldw, \
-                                                                (TO*)y, ldy, partials, M, N, K, steps_per_split)
+                                                                (TO*)y, ldy, partials, M, N, K, steps_per_split, form)
 #define LAUNCH(MTV, TO)                                                                                      \
   do {                                                                                                       \
     if (exact) LAUNCH1(MTV, TO, false, true); else LAUNCH1(MTV, TO, false, false);                           \
@@ -519,10 +523,10 @@ extern "C" int me_gemm_skinny_bf16(const void* x, int64_t ldx, const void* w, in
   if (wide_ok && (out_dtype == ME_F32 || out_dtype == ME_BF16 || partials)) {
     if (out_dtype == ME_F32 || partials)
       gemm_skinny_kernel<1, float, false, true, false, true><<<grid, block, 0, stream>>>(
-          (const bf16_t*)x, ldx, (const bf16_t*)w, ldw, (float*)y, ldy, partials, M, N, K, steps_per_split);
+          (const bf16_t*)x, ldx, (const bf16_t*)w, ldw, (float*)y, ldy, partials, M, N, K, steps_per_split, form);
     else
       gemm_skinny_kernel<1, bf16_t, false, true, false, true><<<grid, block, 0, stream>>>(
-          (const bf16_t*)x, ldx, (const bf16_t*)w, ldw, (bf16_t*)y, ldy, partials, M, N, K, steps_per_split);
+          (const bf16_t*)x, ldx, (const bf16_t*)w, ldw, (bf16_t*)y, ldy, partials, M, N, K, steps_per_split, form);
   } else if (out_dtype == ME_F32 || partials) {
     if (gated) LAUNCH_GATED(float); else if (mt == 4) LAUNCH(4, float); else if (mt == 2) LAUNCH(2, float); else LAUNCH(1, float);
   } else if (out_dtype == ME_BF16) {

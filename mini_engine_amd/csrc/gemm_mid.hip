@@ -41,7 +41,7 @@ __device__ __forceinline__ void mid_barrier() { asm volatile("s_waitcnt lgkmcnt(
 template <typename TO, bool PARTIAL, bool ACT, int MID_BK>
 __global__ void __launch_bounds__(256)
 gemm_mid_kernel(const bf16_t* __restrict__ x, int64_t ldx, const bf16_t* __restrict__ w, int64_t ldw,
-                TO* __restrict__ y, int64_t ldy, int M, int N, int K, int steps_per_split, int m_tiles, int n_tiles) {
+                TO* __restrict__ y, int64_t ldy, int M, int N, int K, int steps_per_split, int m_tiles, int n_tiles, GateForm form) {
   extern __shared__ __align__(16) unsigned char mid_lds[];   // [MID_NB][MID_STAGE]
   static_assert(MID_BK == 64 || MID_BK == 128, "a row of a stage is 128 or 256 bytes");
   constexpr int ROW = 2 * MID_BK;                                    // bytes of a row in LDS
@@ -144,8 +144,9 @@ gemm_mid_kernel(const bf16_t* __restrict__ x, int64_t ldx, const bf16_t* __restr
         out4 r;
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
-          const float gate = acc[0][j][e];
-          r[e] = from_f32<TO>(gate / (1.f + __expf(-gate)) * acc[1][j][e]);
+          float gate = acc[0][j][e], up = acc[1][j][e];
+          if (form.bias) { gate += form.bias[f + e]; up += form.bias[I + f + e]; }
+          r[e] = from_f32<TO>(gate_value<true>(gate, up, form));
         }
         *reinterpret_cast<out4*>(out + (int64_t)t * ldy + f) = r;
       }
@@ -170,10 +171,14 @@ gemm_mid_kernel(const bf16_t* __restrict__ x, int64_t ldx, const bf16_t* __restr
 }
 
 // y: [M, N] of out_dtype (ksplit 1), or float32 partial sums [ksplit, M, N] with ldy = N; act: w is a packed
-// gate/up weight [N = 2 I, K] and y is silu(gate) * up [M, I] (bfloat16, ksplit 1).
+// gate/up weight [N = 2 I, K] and y is silu(gate) * up [M, I] (bfloat16, ksplit 1); limit, alpha, bias: another `GateForm`
+// than that.
 extern "C" int me_gemm_mid_bf16(const void* x, int64_t ldx, const void* w, int64_t ldw, void* y, int64_t ldy,
-                                int out_dtype, int ksplit, int M, int N, int K, int act, hipStream_t stream) {
+                                int out_dtype, int ksplit, int M, int N, int K, int act, float limit, float alpha, const float* bias,
+                                hipStream_t stream) {
   if (M == 0 || N == 0) return 0;
+  ME_CHECK(act || (limit == 0.f && bias == nullptr), "mid gemm: limits and biases belong to the gating epilogue");
+  const GateForm form{limit, alpha, bias};
   ME_CHECK(K >= 64 && K % 64 == 0, "mid gemm: K=%d must be a multiple of 64", K);
   ME_CHECK(N % 4 == 0 && ldy % 4 == 0 && ldx % 8 == 0 && ldw % 8 == 0, "mid gemm: N=%d and the row strides must keep 16-byte pieces whole", N);
   ME_CHECK((reinterpret_cast<uintptr_t>(x) % 16 == 0) && (reinterpret_cast<uintptr_t>(w) % 16 == 0) &&
@@ -195,7 +200,7 @@ extern "C" int me_gemm_mid_bf16(const void* x, int64_t ldx, const void* w, int64
   const size_t lds = (size_t)MID_NB * (MID_TM + MID_TN) * 2 * bk;
 #define MID_LAUNCH1(TO, P, A, BK)                                                                                        \
   gemm_mid_kernel<TO, P, A, BK><<<grid, block, lds, stream>>>((const bf16_t*)x, ldx, (const bf16_t*)w, ldw, (TO*)y, ldy, \
-                                                             M, N, K, steps_per_split, m_tiles, n_tiles)
+                                                             M, N, K, steps_per_split, m_tiles, n_tiles, form)
 #define MID_LAUNCH(TO, P, A)                                                                                       \
   do {                                                                                                             \
     if (wide_steps) {                                                                                              \

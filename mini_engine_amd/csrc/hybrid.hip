@@ -1,7 +1,7 @@
 // Kernels of mixers that run two token mixers side by side, one of them a recurrence whose state rows decay each at
 // a rate of their own: the mix of a token's input with the previous token's, the recurrence itself under two update
 // rules, the weighted sum of the two mixers' outputs, and the small elementwise steps around them (a bias on a
-// projection's rows, an elementwise sigmoid gate, a clamped gated activation). Everything that the recurrence reads
+// projection's rows, an elementwise sigmoid gate). Everything that the recurrence reads
 // besides the projections is formed here in float32: decays and their exponentials, softplus, write strengths, unit
 // lengths.
 #include "common.h"
@@ -59,31 +59,6 @@ extern "C" int me_sigmoid_gate(void* o, int64_t o_stride, const void* g, int64_t
   const dim3 grid((unsigned)((total + 255) / 256 < 65535 ? (total + 255) / 256 : 65535)), block(256);
   if (dtype == ME_F32) sigmoid_gate_kernel<float><<<grid, block, 0, stream>>>((float*)o, o_stride, (const float*)g, g_stride, T, n);
   else sigmoid_gate_kernel<bf16_t><<<grid, block, 0, stream>>>((bf16_t*)o, o_stride, (const bf16_t*)g, g_stride, T, n);
-  ME_LAUNCH_CHECK();
-  return 0;
-}
-
-// ------------------------------------------------------------------ clamped gated activation
-// g = min(gu[t, i], limit), u = clamp(gu[t, I + i], -limit, limit); out = g * sigmoid(alpha * g) * (u + 1).
-template <typename TX>
-__global__ void glu_clamped_kernel(const TX* __restrict__ gu, int64_t gu_stride, TX* __restrict__ out, int64_t T, int I, float limit, float alpha) {
-  const int64_t total = T * I;
-  for (int64_t i = blockIdx.x * (int64_t)blockDim.x + threadIdx.x; i < total; i += (int64_t)gridDim.x * blockDim.x) {
-    const int64_t t = i / I;
-    const int c = (int)(i - t * I);
-    const float g = fminf(to_f32<TX>(gu[t * gu_stride + c]), limit);
-    const float u = fminf(fmaxf(to_f32<TX>(gu[t * gu_stride + I + c]), -limit), limit);
-    out[i] = from_f32<TX>(g * hy_sigmoid(alpha * g) * (u + 1.0f));
-  }
-}
-
-extern "C" int me_glu_clamped(const void* gu, int64_t gu_stride, void* out, int dtype, int64_t T, int I, float limit, float alpha, hipStream_t stream) {
-  if (T == 0 || I == 0) return 0;
-  ME_CHECK(limit > 0.f, "glu_clamped: the limit must be positive");
-  const int64_t total = T * I;
-  const dim3 grid((unsigned)((total + 255) / 256 < 65535 ? (total + 255) / 256 : 65535)), block(256);
-  if (dtype == ME_F32) glu_clamped_kernel<float><<<grid, block, 0, stream>>>((const float*)gu, gu_stride, (float*)out, T, I, limit, alpha);
-  else glu_clamped_kernel<bf16_t><<<grid, block, 0, stream>>>((const bf16_t*)gu, gu_stride, (bf16_t*)out, T, I, limit, alpha);
   ME_LAUNCH_CHECK();
   return 0;
 }

@@ -272,6 +272,22 @@ extern "C" int me_moe_route(const void* x, int64_t ldx, int dtype, const float* 
 }
 
 // ------------------------------------------------------------------ pairs by expert
+// One more in counter[e], and what it held before. Class `common` may have many of a wave's lanes at once: they share one
+// atomic (-1: there is no such class).
+__device__ __forceinline__ int count_one(int* counter, int e, int common) {
+  if (common >= 0) {
+    const unsigned long long lanes = __ballot(e == common);
+    if (e == common) {
+      const int lane = threadIdx.x & 63;
+      const int rank = __popcll(lanes & ((1ull << lane) - 1ull));
+      int base = 0;
+      if (rank == 0) base = atomicAdd(&counter[e], (int)__popcll(lanes));
+      return __shfl(base, __ffsll(lanes) - 1, ME_WAVE) + rank;
+    }
+  }
+  return atomicAdd(&counter[e], 1);
+}
+
 // One workgroup. E: classes of pairs: the experts with weights, and one more for all pairs of identity experts (ids from
 // E - 1 on) where the router has any. order[p']: the pair at sorted place p'; offsets[e]: where class e's pairs begin;
 // tile_expert / tile_row: expert and first sorted place of every tile of up to `tile_rows` pairs (expert -1: a tile nobody needs).
@@ -291,7 +307,8 @@ moe_sort_kernel(int32_t* __restrict__ ids, int P, int routed, int E, int max_til
     __threadfence_block();
   }
   __syncthreads();
-  for (int p = threadIdx.x; p < P; p += blockDim.x) atomicAdd(&count[min(ids[p], E - 1)], 1);
+  const int common = E < routed ? E - 1 : -1;       // identity experts share a class
+  for (int p = threadIdx.x; p < P; p += blockDim.x) count_one(count, min(ids[p], E - 1), common);
   __syncthreads();
   if (threadIdx.x == 0) {
     int at = 0, tiles = 0;
@@ -306,7 +323,7 @@ moe_sort_kernel(int32_t* __restrict__ ids, int P, int routed, int E, int max_til
   for (int e = threadIdx.x; e <= E; e += blockDim.x) offsets[e] = begin[e];
   for (int p = threadIdx.x; p < P; p += blockDim.x) {
     const int e = min(ids[p], E - 1);
-    order[begin[e] + atomicAdd(&cursor[e], 1)] = p;
+    order[begin[e] + count_one(cursor, e, common)] = p;
   }
   for (int e = threadIdx.x; e < E; e += blockDim.x)
     for (int i = tile_at[e]; i < tile_at[e + 1] && i < max_tiles; ++i) {
@@ -348,29 +365,34 @@ extern "C" int me_moe_sort(int32_t* ids, int64_t P, int routed, int identity, in
 // A stage in LDS: TM B rows (pairs) then TN A rows (weights), 128 bytes each. A workgroup's 4 waves are 2 x 2
 // sub-tiles of TM/2 x TN/2, each MJ x MI matrix-instruction tiles of 16 x 16: 64 x 64 (2 x 2 per wave) for a few
 // hundred rows per expert, 128 x 128 (4 x 4 per wave: twice the products per operand read from LDS) beyond.
-// ACT 1: the tile's weight rows are TN/2 gate rows and the TN/2 up rows that go with them; the result is silu(gate) * up.
-// ACT 3: the same rows under `glu` (`ClampedGate`). Tiles of class `experts` (identity experts) have no weights: ACT 0 copies
+// ACT 1: the tile's weight rows are TN/2 gate rows and the TN/2 up rows that go with them; the result is silu(gate) * up, or
+// another `GateForm`. Tiles of class `experts` (identity experts) have no weights: ACT 0 copies
 // their token rows from x_in, the others leave.
 // ACT 2: experts without a gate: the tile's TN weight rows are up rows and the result is relu(up)^2. ACT 0: the down product,
 // times the pair's weight, into the pair's partial sum.
 //   x: [T, K] token rows (ACT 1, 2) or [P, K] rows at sorted places (ACT 0); w: [E * rows_per_expert, K]
-struct ClampedGate { float limit, alpha; };      // g = min(gate, limit), u = clamp(up, -limit, limit): g sigmoid(alpha g) (u + 1)
-
-template <int ACT>
-__device__ __forceinline__ float gated_value(float gate, float up, const ClampedGate& glu) {
-  if constexpr (ACT == 3) {
-    const float g = fminf(gate, glu.limit), u = fminf(fmaxf(up, -glu.limit), glu.limit);
-    return g / (1.f + __expf(-glu.alpha * g)) * (u + 1.f);
-  } else {
-    return gate / (1.f + __expf(-gate)) * up;
-  }
-}
-
 // Rows [row0, row0 + rows) of the identity experts' pairs, features [n0, n1): the token's row times the pair's weight.
 __device__ __forceinline__ void copy_identity_rows(const bf16_t* __restrict__ x_in, int64_t ld_in, const int32_t* __restrict__ order,
                                                    const float* __restrict__ pair_weight, float* __restrict__ out, int64_t T, int top,
                                                    int N, int row0, int rows, int n0, int n1) {
   const int width = n1 - n0;
+  if (width % 8 == 0 && N % 8 == 0 && ld_in % 8 == 0 && reinterpret_cast<uintptr_t>(x_in) % 16 == 0) {
+    const int groups = width / 8;
+#pragma unroll 4
+    for (int i = threadIdx.x; i < rows * groups; i += blockDim.x) {
+      const int r = i / groups, f = n0 + 8 * (i - r * groups);
+      const int pair = order[row0 + r];
+      const int64_t tok = pair / top, choice = pair - tok * top;
+      const float pw = pair_weight[pair];
+      const bf16x8 v = *reinterpret_cast<const bf16x8*>(x_in + tok * ld_in + f);
+      float* o = out + (choice * T + tok) * N + f;
+#pragma unroll
+      for (int q = 0; q < 8; q += 4)
+        *reinterpret_cast<float4*>(o + q) = make_float4(pw * static_cast<float>(v[q]), pw * static_cast<float>(v[q + 1]), pw * static_cast<float>(v[q + 2]),
+                                                        pw * static_cast<float>(v[q + 3]));
+    }
+    return;
+  }
   for (int i = threadIdx.x; i < rows * width; i += blockDim.x) {
     const int r = i / width, f = n0 + i - r * width;
     const int pair = order[row0 + r];
@@ -384,8 +406,8 @@ __global__ void __launch_bounds__(256)
 moe_tile_kernel(const bf16_t* __restrict__ x, int64_t ldx, const bf16_t* __restrict__ w, int64_t ldw,
                 const int32_t* __restrict__ order, const int32_t* __restrict__ offsets, const int32_t* __restrict__ tile_expert,
                 const int32_t* __restrict__ tile_row, const float* __restrict__ pair_weight, void* __restrict__ out,
-                int64_t T, int top, int N, int K, int experts, ClampedGate glu, const bf16_t* __restrict__ x_in, int64_t ld_in) {
-  constexpr bool GATED = ACT == 1 || ACT == 3;
+                int64_t T, int top, int N, int K, int experts, GateForm glu, const bf16_t* __restrict__ x_in, int64_t ld_in) {
+  constexpr bool GATED = ACT == 1;
   constexpr int ROWS = TM + TN, NQ = ROWS / 32, MI = TN / 32, MJ = TM / 32, STAGE = ROWS * 128;
   extern __shared__ __align__(16) unsigned char lds[];        // [2][STAGE]
   const int e = tile_expert[blockIdx.y];
@@ -497,7 +519,7 @@ moe_tile_kernel(const bf16_t* __restrict__ x, int64_t ldx, const bf16_t* __restr
         bf16x4 r;
 #pragma unroll
         for (int q = 0; q < 4; ++q) {
-          r[q] = from_f32<bf16_t>(gated_value<ACT>(acc[i][j][q], acc[i + MI / 2][j][q], glu));
+          r[q] = from_f32<bf16_t>(gate_value<true>(acc[i][j][q], acc[i + MI / 2][j][q], glu));
         }
         if (f + 3 < N && (N & 3) == 0) {
           *reinterpret_cast<bf16x4*>(o + f) = r;          // 4 neighbours, 8 bytes
@@ -530,7 +552,7 @@ moe_tile_kernel(const bf16_t* __restrict__ x, int64_t ldx, const bf16_t* __restr
 template <int ACT, int TM>
 static int launch_moe_tile(const bf16_t* x, int64_t ldx, const bf16_t* w, int64_t ldw, const int32_t* order, const int32_t* offsets,
                            const int32_t* tile_expert, const int32_t* tile_row, const float* pair_weight, void* out, int64_t T,
-                           int top, int N, int K, int max_tiles, int experts, ClampedGate glu, const bf16_t* x_in, int64_t ld_in,
+                           int top, int N, int K, int max_tiles, int experts, GateForm glu, const bf16_t* x_in, int64_t ld_in,
                            hipStream_t stream) {
   constexpr int TN = TM;
   const size_t lds = 2 * (size_t)(TM + TN) * 128;
@@ -540,7 +562,7 @@ static int launch_moe_tile(const bf16_t* x, int64_t ldx, const bf16_t* w, int64_
     ME_CHECK(err == hipSuccess, "routed experts: cannot get %zu bytes of LDS: %s", lds, hipGetErrorString(err));
     allowed = true;
   }
-  const int per = ACT == 1 || ACT == 3 ? TN / 2 : TN;
+  const int per = ACT == 1 ? TN / 2 : TN;
   moe_tile_kernel<ACT, TM, TN><<<dim3((unsigned)((N + per - 1) / per), (unsigned)max_tiles), dim3(256), lds, stream>>>(
       x, ldx, w, ldw, order, offsets, tile_expert, tile_row, pair_weight, out, T, top, N, K, experts, glu, x_in, ld_in);
   ME_LAUNCH_CHECK();
@@ -557,8 +579,8 @@ __global__ void __launch_bounds__(256)
 moe_skinny_kernel(const bf16_t* __restrict__ x, int64_t ldx, const bf16_t* __restrict__ w, const int32_t* __restrict__ order,
                   const int32_t* __restrict__ offsets, const int32_t* __restrict__ tile_expert, const int32_t* __restrict__ tile_row,
                   const float* __restrict__ pair_weight, void* __restrict__ out, int64_t T, int top, int N, int K, int experts,
-                  ClampedGate glu, const bf16_t* __restrict__ x_in, int64_t ld_in) {
-  constexpr bool GATED = ACT == 1 || ACT == 3;
+                  GateForm glu, const bf16_t* __restrict__ x_in, int64_t ld_in) {
+  constexpr bool GATED = ACT == 1;
   __shared__ float part[4][GATED ? 2 : 1][64][4];
   const int e = tile_expert[blockIdx.y];
   if (e < 0) return;
@@ -618,7 +640,7 @@ moe_skinny_kernel(const bf16_t* __restrict__ x, int64_t ldx, const bf16_t* __res
     bf16_t* o = (bf16_t*)out + (int64_t)pr * N;
 #pragma unroll
     for (int q = 0; q < 4; ++q)
-      if (n0 + 4 * g + q < N) o[n0 + 4 * g + q] = from_f32<bf16_t>(gated_value<ACT>(sg[q], su[q], glu));
+      if (n0 + 4 * g + q < N) o[n0 + 4 * g + q] = from_f32<bf16_t>(gate_value<true>(sg[q], su[q], glu));
   } else {
     const int pair = order[pr];
     const int64_t tok = pair / top, choice = pair - tok * top;
@@ -631,7 +653,7 @@ moe_skinny_kernel(const bf16_t* __restrict__ x, int64_t ldx, const bf16_t* __res
 }
 
 // act: bfloat16 [P, F] at sorted places; gate_up: [experts * 2 F, K] (an expert's gate rows, then its up rows), or with `gated`
-// 0 [experts * F, K] (up rows only: the result is relu(up)^2). limit > 0: a clamped gate (`ClampedGate`) in place of silu.
+// 0 [experts * F, K] (up rows only: the result is relu(up)^2). limit, alpha: another `GateForm` than silu (limit 0).
 // Tiles of class `experts` (identity experts) write nothing here.
 // tile_rows: 16 (tiles of `moe_sort` with 16 rows: the skinny kernel), 64 or 128
 extern "C" int me_moe_gate_up(const void* x, int64_t ldx, const void* gate_up, const int32_t* order, const int32_t* offsets,
@@ -642,13 +664,12 @@ extern "C" int me_moe_gate_up(const void* x, int64_t ldx, const void* gate_up, c
            "moe_gate_up: rows must be whole 16-byte pieces (K = %d)", K);
   ME_CHECK(max_tiles >= 1 && max_tiles <= 65535 && F >= 1 && experts >= 1, "moe_gate_up: %d tiles", max_tiles);
   ME_CHECK(limit <= 0.f || gated, "moe_gate_up: only a gate can be clamped");
-  const ClampedGate glu{limit, alpha};
-  const int kind = !gated ? 2 : (limit > 0.f ? 3 : 1);
+  const GateForm glu{limit, alpha, nullptr};
   if (tile_rows == 16) {
     const dim3 grid((unsigned)((F + 15) / 16), (unsigned)max_tiles), block(256);
 #define SKINNY(A) moe_skinny_kernel<A><<<grid, block, 0, stream>>>((const bf16_t*)x, ldx, (const bf16_t*)gate_up, order, offsets, tile_expert, \
                                                                    tile_row, nullptr, act, T, top, F, K, experts, glu, nullptr, 0)
-    if (kind == 1) SKINNY(1); else if (kind == 2) SKINNY(2); else SKINNY(3);
+    if (gated) SKINNY(1); else SKINNY(2);
 #undef SKINNY
     ME_LAUNCH_CHECK();
     return 0;
@@ -657,13 +678,11 @@ extern "C" int me_moe_gate_up(const void* x, int64_t ldx, const void* gate_up, c
 #define TILE(A, M) return launch_moe_tile<A, M>((const bf16_t*)x, ldx, (const bf16_t*)gate_up, (int64_t)K, order, offsets, tile_expert, tile_row, \
                                                 nullptr, act, T, top, F, K, max_tiles, experts, glu, nullptr, 0, stream)
   if (tile_rows == 128) {
-    if (kind == 1) TILE(1, 128);
-    if (kind == 2) TILE(2, 128);
-    TILE(3, 128);
+    if (gated) TILE(1, 128);
+    TILE(2, 128);
   }
-  if (kind == 1) TILE(1, 64);
-  if (kind == 2) TILE(2, 64);
-  TILE(3, 64);
+  if (gated) TILE(1, 64);
+  TILE(2, 64);
 #undef TILE
 }
 
@@ -677,7 +696,7 @@ extern "C" int me_moe_down(const void* act, const void* down, const int32_t* ord
   ME_CHECK(F % 8 == 0 && reinterpret_cast<uintptr_t>(act) % 16 == 0 && reinterpret_cast<uintptr_t>(down) % 16 == 0,
            "moe_down: rows must be whole 16-byte pieces (F = %d)", F);
   ME_CHECK(max_tiles >= 1 && max_tiles <= 65535 && N >= 1 && experts >= 1, "moe_down: %d tiles", max_tiles);
-  const ClampedGate none{0.f, 0.f};
+  const GateForm none{0.f, 0.f, nullptr};
   if (tile_rows == 16) {
     moe_skinny_kernel<0><<<dim3((unsigned)((N + 15) / 16), (unsigned)max_tiles), dim3(256), 0, stream>>>(
         (const bf16_t*)act, (int64_t)F, (const bf16_t*)down, order, offsets, tile_expert, tile_row, pair_weight, out, T, top, N, F,
@@ -698,7 +717,7 @@ extern "C" int me_moe_down(const void* act, const void* down, const int32_t* ord
 template <typename TX, bool GATED>
 __global__ void __launch_bounds__(256)
 moe_gate_up_simple_kernel(const TX* __restrict__ x, int64_t ldx, const TX* __restrict__ gate_up, const int32_t* __restrict__ ids,
-                          TX* __restrict__ act, int64_t P, int top, int F, int K, int experts, ClampedGate glu) {
+                          TX* __restrict__ act, int64_t P, int top, int F, int K, int experts, GateForm glu) {
   const int lane = threadIdx.x & 63;
   const int64_t at = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (at >= P * F) return;
@@ -717,16 +736,7 @@ moe_gate_up_simple_kernel(const TX* __restrict__ x, int64_t ldx, const TX* __res
   sg = wave_sum(sg);
   if (GATED) su = wave_sum(su);
   const float up = fmaxf(sg, 0.f);
-  float v = up * up;
-  if (GATED) {
-    if (glu.limit > 0.f) {
-      const float g = fminf(sg, glu.limit), u = fminf(fmaxf(su, -glu.limit), glu.limit);
-      v = g / (1.f + expf(-glu.alpha * g)) * (u + 1.f);
-    } else {
-      v = sg / (1.f + expf(-sg)) * su;
-    }
-  }
-  if (lane == 0) act[at] = from_f32<TX>(v);
+  if (lane == 0) act[at] = from_f32<TX>(GATED ? gate_value<false>(sg, su, glu) : up * up);
 }
 
 template <typename TX>
@@ -757,7 +767,7 @@ extern "C" int me_moe_experts_simple(const void* x, int64_t ldx, int dtype, cons
                                      int N, int F, int K, int gated, int experts, float limit, float alpha, hipStream_t stream) {
   if (T == 0) return 0;
   ME_CHECK(experts >= 1 && (limit <= 0.f || gated), "moe_experts_simple: only a gate can be clamped");
-  const ClampedGate glu{limit, alpha};
+  const GateForm glu{limit, alpha, nullptr};
   const int64_t P = T * top;
   const int64_t g1 = (P * F + 3) / 4, g2 = (P * N + 3) / 4;
   ME_CHECK(g1 < (1ll << 31) && g2 < (1ll << 31), "moe_experts_simple: too many outputs");

@@ -62,16 +62,16 @@ _CORE_PROTOS = {
     "me_gather_rows_scaled": [P, I, P, P, L, L, L, F, P],
     "me_take_tokens": [P, P, P, I, I, P],
     "me_rms_norm": [P, I, I, L, P, P, P, P, I, L, I, F, P],
-    "me_silu_and_mul": [P, P, P, I, L, I, P],
+    "me_gate_mul": [P, L, P, F, F, P, I, L, I, P],
     "me_qk_norm_rope_store": [P, I, L, L, P, P, F, P, L, L, P, P, P, P, I, I, I, I, I, I, P],
     "me_store_kv": [P, P, I, L, L, L, P, P, P, I, I, I, P],
     "me_attn_simple": [P, L, P, L, I, P, P, P, I, P, P, P, L, I, I, I, I, F, I, I, F, P, P, P],
     "me_attn_tail": [P, L, P, L, P, I, P, P, P, I, P, P, P, L, I, I, I, I, F, I, I, F, P, P, P],
     "me_gemm_tiled": [P, L, P, L, P, L, I, I, I, I, I, P],
-    "me_gemm_skinny_bf16": [P, L, P, L, P, L, I, P, I, I, I, I, I, I, I, P],
+    "me_gemm_skinny_bf16": [P, L, P, L, P, L, I, P, I, I, I, I, I, I, I, F, F, P, P],
     "me_gemm_rows_bf16": [P, L, P, L, P, L, I, P, I, I, I, I, I, P],
     "me_gemm_skinny_norm_bf16": [P, I, I, P, P, P, F, P, L, P, L, I, I, I, I, I, P],
-    "me_gemm_mid_bf16": [P, L, P, L, P, L, I, I, I, I, I, I, P],
+    "me_gemm_mid_bf16": [P, L, P, L, P, L, I, I, I, I, I, I, F, F, P, P],
     "me_gemm_library_bf16": [P, L, P, L, P, L, I, P, ctypes.c_size_t, I, I, I, I, P],
     "me_add_rms_norm": [P, I, I, L, P, P, P, P, L, I, F, P],
     "me_add_rms_norm_partials": [P, I, L, P, P, P, P, L, I, F, P],
@@ -94,7 +94,6 @@ _CORE_PROTOS = {
     "me_moe_experts_simple": [P, L, I, P, P, P, P, P, P, L, I, I, I, I, I, I, F, F, P],
     "me_add_bias": [P, I, I, L, L, P, I, P, I, L, I, P],
     "me_sigmoid_gate": [P, L, P, L, I, L, I, P],
-    "me_glu_clamped": [P, L, P, I, L, I, F, F, P],
     "me_weighted_sum": [I, P, P, P, P, P, P, P, P, F, P, P, P, I, L, I, P, P, P, P],
     "me_latent_prepare": [P, L, I, I, I, I, I, I, I, I, P, F, P, L, P, P, P, L, P, P, I, I, I, P, P, L, P],
     "me_heads_linear": [P, L, L, P, P, L, L, I, L, I, I, I, P],
@@ -363,7 +362,7 @@ class HipBackend:
         inter = gu.shape[1] // 2
         out = torch.empty((gu.shape[0], inter), dtype=gu.dtype, device=gu.device)
         _check(bias is None or (bias.dtype == torch.float32 and bias.shape == (2 * inter,) and bias.is_contiguous()), "silu_and_mul: bias float32 [2 I]")
-        core().call("me_silu_and_mul", gu.data_ptr(), _ptr(bias), out.data_ptr(), _code(gu.dtype), gu.shape[0], inter, _stream())
+        core().call("me_gate_mul", gu.data_ptr(), gu.stride(0), _ptr(bias), 0.0, 1.0, out.data_ptr(), _code(gu.dtype), gu.shape[0], inter, _stream())
         return out
 
     # -- q/k norm + rotary + cache write -------------------------------------------------
@@ -604,7 +603,7 @@ class HipBackend:
         if mid_parts > 1:
             parts = torch.empty((mid_parts, M, N), dtype=torch.float32, device=x.device)
             core().call("me_gemm_mid_bf16", x.data_ptr(), x.stride(0), w.data_ptr(), w.stride(0), parts.data_ptr(), N,
-                        ME_F32, mid_parts, M, N, K, 0, _stream())
+                        ME_F32, mid_parts, M, N, K, 0, 0.0, 1.0, None, _stream())
             return parts
         splits = library_splits(M, N, K) if (allow_partials and out_dtype == x.dtype) else 1
         if splits > 1:
@@ -623,37 +622,41 @@ class HipBackend:
         if ksplit > 1:
             parts = torch.empty((ksplit, M, N), dtype=torch.float32, device=x.device)
             core().call("me_gemm_skinny_bf16", x.data_ptr(), x.stride(0), w.data_ptr(), w.stride(0), None, N,
-                        ME_F32, parts.data_ptr(), ksplit, M, N, K, 0, 0, skinny_wide(N, K), _stream())
+                        ME_F32, parts.data_ptr(), ksplit, M, N, K, 0, 0, skinny_wide(N, K), 0.0, 1.0, None, _stream())
             return parts
         if skinny_takes(M, N, K):
             y = new()
             core().call("me_gemm_skinny_bf16", x.data_ptr(), x.stride(0), w.data_ptr(), w.stride(0), y.data_ptr(), N,
-                        _code(out_dtype), None, 1, M, N, K, 0, 0, skinny_wide(N, K), _stream())
+                        _code(out_dtype), None, 1, M, N, K, 0, 0, skinny_wide(N, K), 0.0, 1.0, None, _stream())
             return y
         if mid_takes(M, N, K, False) == 1:
             y = new()
             core().call("me_gemm_mid_bf16", x.data_ptr(), x.stride(0), w.data_ptr(), w.stride(0), y.data_ptr(), N,
-                        _code(out_dtype), 1, M, N, K, 0, _stream())
+                        _code(out_dtype), 1, M, N, K, 0, 0.0, 1.0, None, _stream())
             return y
         # many rows, or the head over a large vocabulary: the library product (float32 accumulation; the
         # float32 output form keeps the logits unrounded)
         return library_product(x, w, out_dtype, out=out)
 
-    def gated_linear(self, x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    def gated_linear(self, x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None = None, clamp: tuple | None = None) -> torch.Tensor:
         """silu(x . w[:I]^T) * (x . w[I:]^T) for a packed gate/up weight w [2 I, K] (gate rows first), as one
         launch: the product's workgroups pair each gate feature with its up feature when they merge their waves,
         from the unrounded sums (the separate kernels round the product to bfloat16 first). For the row counts
-        `gated_linear_fuses` admits. Returns [M, I]. (reference layers/linear.py:29-45, layers/activation.py:5-7.)"""
+        `gated_linear_fuses` admits. `bias` (float32 [2 I]) joins the sums first; `clamp` (limit, alpha): the form of
+        `glu_clamped` in place of silu(gate) * up. Returns [M, I]. (reference layers/linear.py:29-45, layers/activation.py:5-7.)"""
         _check(gated_linear_fuses(x, w), "gated_linear: bfloat16, few rows, see gated_linear_fuses")
         M, K = x.shape
         N = w.shape[0]
         y = torch.empty((M, N // 2), dtype=x.dtype, device=x.device)
+        _check(bias is None or (bias.dtype == torch.float32 and bias.shape == (N,) and bias.is_contiguous()), "gated_linear: bias float32 [2 I]")
+        _check(clamp is None or clamp[0] > 0, "gated_linear: the limit must be positive")
+        form = (0.0, 1.0) if clamp is None else (float(clamp[0]), float(clamp[1]))
         if M > GATED_EPILOGUE_MAX_M:        # a few hundred rows over a small weight: the gating in that kernel's epilogue
             core().call("me_gemm_mid_bf16", x.data_ptr(), x.stride(0), w.data_ptr(), w.stride(0), y.data_ptr(), N // 2,
-                        ME_BF16, 1, M, N, K, 1, _stream())
+                        ME_BF16, 1, M, N, K, 1, *form, _ptr(bias), _stream())
             return y
         core().call("me_gemm_skinny_bf16", x.data_ptr(), x.stride(0), w.data_ptr(), w.stride(0), y.data_ptr(), N // 2,
-                    ME_BF16, None, 1, M, N, K, 0, 1, skinny_wide(N, K), _stream())
+                    ME_BF16, None, 1, M, N, K, 0, 1, skinny_wide(N, K), *form, _ptr(bias), _stream())
         return y
 
     def norm_linear(self, x: torch.Tensor, residual: torch.Tensor | None, norm_weight: torch.Tensor, eps: float,
@@ -704,11 +707,11 @@ class HipBackend:
         if ksplit > 1:
             parts = torch.empty((ksplit, M, N), dtype=torch.float32, device=gu.device)
             core().call("me_gemm_skinny_bf16", gu.data_ptr(), gu.stride(0), w.data_ptr(), w.stride(0), None, N,
-                        ME_F32, parts.data_ptr(), ksplit, M, N, inter, 1, 0, 0, _stream())
+                        ME_F32, parts.data_ptr(), ksplit, M, N, inter, 1, 0, 0, 0.0, 1.0, None, _stream())
             return parts
         y = torch.empty((M, N), dtype=gu.dtype, device=gu.device)
         core().call("me_gemm_skinny_bf16", gu.data_ptr(), gu.stride(0), w.data_ptr(), w.stride(0), y.data_ptr(), N,
-                    ME_BF16, None, 1, M, N, inter, 1, 0, 0, _stream())
+                    ME_BF16, None, 1, M, N, inter, 1, 0, 0, 0.0, 1.0, None, _stream())
         return y
 
     # -- norms on a sublayer's output, activations, gates ----------------------------------
@@ -1013,7 +1016,7 @@ class HipBackend:
         _check(gu.dim() == 2 and gu.stride(1) == 1 and gu.shape[1] % 2 == 0, "glu_clamped: rows [T, 2 I]")
         T, inter = gu.shape[0], gu.shape[1] // 2
         out = torch.empty((T, inter), dtype=gu.dtype, device=gu.device)
-        core().call("me_glu_clamped", gu.data_ptr(), gu.stride(0), out.data_ptr(), _code(gu.dtype), T, inter, float(limit), float(alpha), _stream())
+        core().call("me_gate_mul", gu.data_ptr(), gu.stride(0), None, float(limit), float(alpha), out.data_ptr(), _code(gu.dtype), T, inter, _stream())
         return out
 
     def weighted_sum(self, terms, norm_weight=None, eps: float = 0.0, stream=None, out_dtype: torch.dtype | None = None):

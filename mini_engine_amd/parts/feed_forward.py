@@ -43,7 +43,7 @@ class SwiGLU(FeedForward):
 
     def forward(self, x):
         if self.biased:
-            y = self.down.forward(ops.silu_and_mul(self.gate_up.forward(x), bias=self.gate_up_bias), allow_partials=True)
+            y = self.down.forward(self.gate_up.forward(x, gated=True, bias=self.gate_up_bias), allow_partials=True)
             return Biased(y, self.down_bias) if self.defer_bias else ops.add_bias(y, self.down_bias, self.down.weight.dtype)
         rows = x.rows() if isinstance(x, PendingNorm) else x.shape[0]
         if ops.gated_linear_rows(rows, self.gate_up.weight):
@@ -94,7 +94,7 @@ class ActivatedMLP(FeedForward):
 @register_part("feed_forward", "clamped_glu")
 class ClampedGLU(FeedForward):
     """g = min(gate(x), limit), u = clamp(up(x), -limit, limit); down(g * sigmoid(alpha * g) * (u + 1)). Gate and up are
-    one packed product with gate's rows first."""
+    one packed product with gate's rows first, the activation in its epilogue where there is a kernel for that."""
 
     def __init__(self, hidden_size: int, intermediate_size: int, limit: float, alpha: float = 1.702):
         super().__init__()
@@ -107,4 +107,4 @@ class ClampedGLU(FeedForward):
         self.add_child("down", Linear(intermediate_size, hidden_size))
 
     def forward(self, x):
-        return self.down.forward(ops.glu_clamped(self.gate_up.forward(x), self.limit, self.alpha), allow_partials=True)
+        return self.down.forward(self.gate_up.forward(x, gated=True, clamp=(self.limit, self.alpha)), allow_partials=True)

@@ -161,8 +161,11 @@ def _gate(y):
     return y[:, :inter] * torch.sigmoid(y[:, :inter]) * y[:, inter:]
 
 
-def gated_linear(x, w, compute_dtype=torch.float32):
-    return _gate(x.to(compute_dtype) @ w.to(compute_dtype).t()).to(x.dtype)
+def gated_linear(x, w, bias=None, clamp=None, compute_dtype=torch.float32):
+    y = x.to(compute_dtype) @ w.to(compute_dtype).t()
+    if bias is not None:
+        y = y + bias
+    return (glu_clamped(y, *clamp) if clamp is not None else _gate(y)).to(x.dtype)
 
 
 def norm_linear(x, residual, norm_weight, eps, w, out_dtype=None, want_residual=True, gated=False, compute_dtype=torch.float32):

@@ -207,13 +207,31 @@ def test_experts_with_a_clamped_gate_and_identity_experts(dtype, T, n, F, E, Z, 
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("T,F", [(1, 256), (37, 24), (5, 13), (700, 100), (64, 3072)])
+@pytest.mark.parametrize("T,F", [(1, 256), (37, 24), (5, 13), (700, 100), (64, 3072), (9000, 40), (20, 6000)])
 def test_silu_and_mul_with_biases(dtype, T, F):
     torch.manual_seed(T + F)
     gu, bias = torch.randn(T, 2 * F, device=DEV).to(dtype), torch.randn(2 * F, device=DEV)
     tol = 1e-2 if dtype == torch.bfloat16 else 1e-5
+    wide = torch.randn(T, 2 * F + 24, device=DEV).to(dtype)
+    for at in (8, 3):                              # rows inside wider ones, at whole pieces and not
+        close(hip().glu_clamped(wide[:, at:at + 2 * F], 0.8, 1.3), twin.glu_clamped(wide.cpu()[:, at:at + 2 * F], 0.8, 1.3), tol)
     close(hip().silu_and_mul(gu, bias=bias), twin.silu_and_mul(gu.cpu(), bias.cpu()), tol)
     close(hip().silu_and_mul(gu), twin.silu_and_mul(gu.cpu()), tol)
+
+
+@pytest.mark.parametrize("M,F,K", [(1, 1536, 1024), (8, 3072, 1024), (16, 96, 40), (3, 12, 136), (24, 512, 1024), (40, 3072, 1024), (200, 512, 256), (128, 1536, 1024)])
+def test_gate_and_up_with_biases_or_a_clamp_in_the_products_epilogue(M, F, K):
+    """Both products that gate in their epilogue, against the twin, and against the product with the activation behind it."""
+    torch.manual_seed(M + F)
+    x, w = torch.randn(M, K, device=DEV).to(torch.bfloat16), (torch.randn(2 * F, K, device=DEV) * K ** -0.5).to(torch.bfloat16)
+    bias = torch.randn(2 * F, device=DEV)
+    assert ops.gated_linear_fuses(x, w)
+    for kw in ({"bias": bias}, {"clamp": (0.6, 1.702)}, {"clamp": (50.0, 0.7)}, {}):
+        want = twin.gated_linear(x.cpu(), w.cpu(), **{n: _wide(t) for n, t in kw.items()})
+        close(hip().gated_linear(x, w, **kw), want, 1e-2)
+    gu = hip().linear(x, w)
+    close(hip().gated_linear(x, w, bias=bias), hip().silu_and_mul(gu, bias=bias), 3e-2)
+    close(hip().gated_linear(x, w, clamp=(0.6, 1.702)), hip().glu_clamped(gu, 0.6, 1.702), 3e-2)
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
